@@ -1,3 +1,4 @@
-"""Importing this package registers the architectures the library ships (GPT-2, Salopel, Kodatar, Rotutar, Gavasun)."""
+"""Importing this package registers the architectures the library ships (GPT-2, Salopel, Kodatar, Rotutar, Gavasun,
+Loselix)."""
 
-from . import gavasun, gpt2, kodatar, rotutar, salopel  # noqa: F401
+from . import gavasun, gpt2, kodatar, loselix, rotutar, salopel  # noqa: F401

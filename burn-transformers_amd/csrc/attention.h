@@ -37,6 +37,22 @@ struct AttnArgs {
   // query sees: exp(sink[head]) is added once, unscaled, with no key and no value of its own (the
   // weights of a query's keys then add up to less than one).
   const float* sink;
+  // How a score s = q . k * scale weighs its key.
+  //   0: softmax(s) over the keys a query sees
+  //   1: softmax(cap * tanh(s / cap))
+  //   2: sigmoid(s + score_bias[head]), every key by itself: nothing is normalised over the keys (no sink)
+  int form;
+  float cap;                // form 1: positive
+  const float* score_bias;  // form 2: [q_heads], or null for zero
+  // What happens to a head's output row before it is stored: times sigmoid(gate), one float32 logit per head
+  // (`gate_span` 0: column `head` of the token's row) or per channel (1: column head * gate_dim + channel; channels
+  // from gate_dim on hold zeros and have none); null: no factor.  `out_f32`: stored in 32-bit whatever the products'
+  // type.  Forms 1 and 2 and these are in the kernels built with BT_ATTENTION_FORM and in the plain kernel.
+  const float* gate;        // [tokens][ld_gate]
+  int64_t ld_gate;
+  int gate_span;
+  int gate_dim;
+  int out_f32;
 };
 
 // What a sink adds to a softmax's denominator that is kept relative to the maximum `top`.  The plain and
@@ -46,6 +62,28 @@ __device__ __forceinline__ float bt_sink_term(const float* sink, int head, float
 }
 __device__ __forceinline__ float bt_sink_term_pow2(const float* sink, int head, float top) {
   return sink ? exp2f(sink[head] * 1.4426950408889634f - top) : 0.f;
+}
+
+__device__ __forceinline__ float bt_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+
+// The gate's factor on channel `channel` of head `head` of token `tok`.
+__device__ __forceinline__ float bt_output_gate(const AttnArgs& a, int64_t tok, int head, int channel) {
+  if (!a.gate) return 1.f;
+  const int column = a.gate_span == 1 ? head * a.gate_dim + (channel < a.gate_dim ? channel : 0) : head;
+  return bt_sigmoid(a.gate[tok * a.ld_gate + column]);
+}
+
+// What forms and output stages need of their arguments; nullptr, or what is wrong.
+inline const char* bt_check_form(const AttnArgs& a) {
+  if (a.form < 0 || a.form > 2) return "unknown form of the scores";
+  if (a.form == 1 && !(a.cap > 0.f)) return "the scores' cap must be positive";
+  if (a.form == 2 && a.sink) return "a sink stands in a softmax's denominator; sigmoid weights have none";
+  if (a.form != 2 && a.score_bias) return "a bias on the scores goes with sigmoid weights";
+  if (a.gate && (a.gate_span < 0 || a.gate_span > 1 ||
+                 a.ld_gate < (a.gate_span == 1 ? (int64_t)a.q_heads * a.gate_dim : (int64_t)a.q_heads) ||
+                 (a.gate_span == 1 && (a.gate_dim <= 0 || a.gate_dim > a.kv.head_dim))))
+    return "the gate's rows do not hold a logit per head or channel";
+  return nullptr;
 }
 
 // The first position a query at `pos` sees: the later of its window's and its chunk's first key.

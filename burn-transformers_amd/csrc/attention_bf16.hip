@@ -34,6 +34,16 @@
 #error "compile with -DBT_HEAD_DIM=<multiple of 16>"
 #endif
 
+// BT_ATTENTION_FORM (0, 1, 2: AttnArgs.form) builds the module for that form of the scores and with the output stage
+// (gate, 32-bit output); without it the module is the softmax alone.
+#ifdef BT_ATTENTION_FORM
+constexpr int FORM = BT_ATTENTION_FORM;
+constexpr bool STAGED = true;
+#else
+constexpr int FORM = 0;
+constexpr bool STAGED = false;
+#endif
+
 constexpr int HD = BT_HEAD_DIM;
 constexpr int NKS = (HD + 31) / 32;  // steps of 32 channels in q . k
 constexpr int ND = HD / 16;          // blocks of 16 output channels
@@ -70,6 +80,69 @@ __device__ __forceinline__ void load_tile(TileOperands& t, const bf16_t* __restr
   }
 }
 
+#define LOG2_E 1.4426950408889634f
+
+// What turns a raw dot product into the exponent that weighs its key (powers of two):
+//   form 0: x = r * c, c = scale log2(e)
+//   form 1: x = cap2 * tanh(r * scale / cap), cap2 = cap log2(e); with c = 2 scale / cap log2(e) that is
+//           cap2 - 2 cap2 / (2^(r c) + 1): one exponential and one reciprocal
+//   form 2: the weight itself, 1 / (1 + 2^-(r c + bias2))
+struct Scoring {
+  float c, cap2, bias2;
+};
+
+__device__ __forceinline__ Scoring scoring_of(const AttnArgs& a, int head) {
+  Scoring sc;
+  sc.c = FORM == 1 ? 2.0f * a.scale / a.cap * LOG2_E : a.scale * LOG2_E;
+  sc.cap2 = FORM == 1 ? a.cap * LOG2_E : 0.f;
+  sc.bias2 = FORM == 2 && a.score_bias ? a.score_bias[head] * LOG2_E : 0.f;
+  return sc;
+}
+
+// form 1: raw dot product -> capped exponent (before excluded keys are replaced)
+__device__ __forceinline__ float capped_exponent(float r, const Scoring& sc) {
+  return fmaf(-2.0f * sc.cap2, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(r * sc.c) + 1.0f), sc.cap2);
+}
+// form 2: raw dot product -> weight; an excluded key's -inf gives 2^inf and so exactly zero
+__device__ __forceinline__ float sigmoid_weight(float r, const Scoring& sc) {
+  return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-fmaf(r, sc.c, sc.bias2)));
+}
+// the running maximum before the first key: sigmoid weights have none, zero stands for it
+constexpr float FIRST_MAXIMUM = FORM == 2 ? 0.f : -INFINITY;
+
+// Four consecutive channels of one head's output row, gated and in the output's type.
+__device__ __forceinline__ void put4(const AttnArgs& a, int64_t tok, int head, int channel, const float (&v)[4], float head_gate) {
+  if constexpr (STAGED) {
+    float w[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      w[r] = v[r] * (a.gate && a.gate_span == 1 ? bt_output_gate(a, tok, head, channel + r) : head_gate);
+    if (a.out_f32) {
+      *reinterpret_cast<floatx4*>(static_cast<float*>(a.out) + tok * a.ldo + head * HD + channel) = floatx4{w[0], w[1], w[2], w[3]};
+      return;
+    }
+    bf16x4 packed = {(bf16_t)w[0], (bf16_t)w[1], (bf16_t)w[2], (bf16_t)w[3]};
+    *reinterpret_cast<bf16x4*>(static_cast<bf16_t*>(a.out) + tok * a.ldo + head * HD + channel) = packed;
+  } else {
+    bf16x4 packed = {(bf16_t)v[0], (bf16_t)v[1], (bf16_t)v[2], (bf16_t)v[3]};
+    *reinterpret_cast<bf16x4*>(static_cast<bf16_t*>(a.out) + tok * a.ldo + head * HD + channel) = packed;
+  }
+}
+// One channel, row-major or chunk-major.
+__device__ __forceinline__ void put1(const AttnArgs& a, int tok, int head, int channel, float v) {
+  if constexpr (STAGED) {
+    v *= bt_output_gate(a, tok, head, channel);
+    if (a.out_f32) {
+      static_cast<float*>(a.out)[(int64_t)tok * a.ldo + head * HD + channel] = v;
+      return;
+    }
+  }
+  static_cast<bf16_t*>(a.out)[activation_offset<bf16_t>(a.out_rows, a.ldo, tok, head * HD + channel)] = (bf16_t)v;
+}
+__device__ __forceinline__ float head_gate_of(const AttnArgs& a, int64_t tok, int head) {
+  return STAGED && a.gate && a.gate_span == 0 ? bt_output_gate(a, tok, head, 0) : 1.f;
+}
+
 // The online softmax of both forms below works on exponents, x = score * c - (the query's running
 // maximum, which may lag: RESCALE_SLACK), computed by the one FMA that the exponential needs
 // anyway.  A lane looks at its OWN exponents only; the four lanes of a query compare notes, and
@@ -101,13 +174,14 @@ __device__ __forceinline__ float raise_maximum(float& m, float top, float& alpha
 //   qpos[nq]: position of the query in column lane % 16 of tile nq, -1 if there is none.
 //   qlo[nq]: the first position that query sees (its window's or its chunk's first key, else 0).
 //   valid_end: positions >= valid_end hold no token (their values are replaced by zero).
-//   c: the score scale times log2(e), positive; m[] is kept in those units (powers of two).
+//   sc: what makes exponents of the dot products (form 0: one positive factor); m[] is kept in those units
+//   (powers of two).
 //   MASKED = false is for tiles every query of the wave sees whole (all keys at or before the
 //   first query's position, no window): nothing is compared or replaced there.  Columns without
 //   a query then hold numbers nobody reads.
 template <int NQ, bool MASKED>
 __device__ __forceinline__ void attend_tile(const TileOperands& tile, int kb, int valid_end,
-                                            const int (&qpos)[NQ], const int (&qlo)[NQ], float c,
+                                            const int (&qpos)[NQ], const int (&qlo)[NQ], const Scoring& sc,
                                             const bf16x8 (&q)[NQ][NKS], floatx4 (&o)[NQ][ND],
                                             float (&m)[NQ], float (&l)[NQ]) {
   const int lane = threadIdx.x & 63, g = lane >> 4;
@@ -122,6 +196,14 @@ __device__ __forceinline__ void attend_tile(const TileOperands& tile, int kb, in
         acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tile.k[t][ks], q[nq][ks], acc, 0, 0, 0);
       s[nq][t] = acc;
     }
+  }
+  if constexpr (FORM == 1) {
+#pragma unroll
+    for (int nq = 0; nq < NQ; ++nq)
+#pragma unroll
+      for (int t = 0; t < 2; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) s[nq][t][r] = capped_exponent(s[nq][t][r], sc);
   }
   float own[NQ];
   bool behind = false;
@@ -138,11 +220,12 @@ __device__ __forceinline__ void attend_tile(const TileOperands& tile, int kb, in
           s[nq][t][r] = seen ? s[nq][t][r] : -INFINITY;
         }
     }
+    if constexpr (FORM == 2) continue;          // weights that no other key has a part in
     const float m_use = m[nq] == -INFINITY ? 0.f : m[nq];
 #pragma unroll
     for (int t = 0; t < 2; ++t)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) s[nq][t][r] = fmaf(s[nq][t][r], c, -m_use);
+      for (int r = 0; r < 4; ++r) s[nq][t][r] = FORM == 1 ? s[nq][t][r] - m_use : fmaf(s[nq][t][r], sc.c, -m_use);
     own[nq] = fmaxf(fmaxf(fmaxf(s[nq][0][0], s[nq][0][1]), fmaxf(s[nq][0][2], s[nq][0][3])),
                     fmaxf(fmaxf(s[nq][1][0], s[nq][1][1]), fmaxf(s[nq][1][2], s[nq][1][3])));
     behind = behind || own[nq] > (m[nq] == -INFINITY ? -INFINITY : RESCALE_SLACK);
@@ -174,8 +257,8 @@ __device__ __forceinline__ void attend_tile(const TileOperands& tile, int kb, in
     for (int t = 0; t < 2; ++t)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        float p = __builtin_amdgcn_exp2f(s[nq][t][r]);
-        psum += p;
+        float p = FORM == 2 ? sigmoid_weight(s[nq][t][r], sc) : __builtin_amdgcn_exp2f(s[nq][t][r]);
+        if constexpr (FORM != 2) psum += p;
         pop[nq][4 * t + r] = (bf16_t)p;
       }
     l[nq] += psum;  // per-lane part of the sum; the four lanes of a column meet at the end
@@ -197,8 +280,6 @@ __device__ __forceinline__ void attend_tile(const TileOperands& tile, int kb, in
       o[nq][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vop, pop[nq], o[nq][dt], 0, 0, 0);
   }
 }
-
-#define LOG2_E 1.4426950408889634f
 
 // Start of the (block, kv head) plane that holds position kb of a sequence.
 __device__ __forceinline__ int64_t tile_plane(const AttnArgs& a, int seq, int kv_head, int kb) {
@@ -280,7 +361,7 @@ attention_prefill_kernel(AttnArgs a) {
     }
 #pragma unroll
     for (int dt = 0; dt < ND; ++dt) o[nq][dt] = floatx4{0.f, 0.f, 0.f, 0.f};
-    m[nq] = -INFINITY;
+    m[nq] = FIRST_MAXIMUM;
     l[nq] = 0.f;
   }
   const int last = q0 + PREFILL_QUERIES_PER_WAVE < count ? q0 + PREFILL_QUERIES_PER_WAVE : count;
@@ -292,7 +373,7 @@ attention_prefill_kernel(AttnArgs a) {
   // The tiles alternate between two sets of registers, each named at compile time, so nothing
   // is copied: while one is multiplied the other is in flight.  (A third set, two tiles ahead,
   // costs the registers that let two work-groups share a compute unit, and measured slower.)
-  const float c = a.scale * LOG2_E;
+  const Scoring sc = scoring_of(a, head);
   const int whole_until = a.window == 0 && a.chunk == 0 ? start + q0 + 1 : 0;   // tiles ending here or before are seen whole
   // A fetch beyond the last tile reads the first one again instead of being skipped: with the same
   // number of loads in flight on every path, the wait before a tile is for that tile only.
@@ -304,9 +385,9 @@ attention_prefill_kernel(AttnArgs a) {
   };
   auto attend = [&](const TileOperands& tile, int kb) {
     if (kb + 32 <= whole_until)
-      attend_tile<PREFILL_NQ, false>(tile, kb, valid_end, qpos, qlo, c, q, o, m, l);
+      attend_tile<PREFILL_NQ, false>(tile, kb, valid_end, qpos, qlo, sc, q, o, m, l);
     else
-      attend_tile<PREFILL_NQ, true>(tile, kb, valid_end, qpos, qlo, c, q, o, m, l);
+      attend_tile<PREFILL_NQ, true>(tile, kb, valid_end, qpos, qlo, sc, q, o, m, l);
   };
   if (lo >= hi) return;   // (cannot happen: a wave with a query sees at least that query's key)
   fetch(t0, lo);
@@ -317,20 +398,19 @@ attention_prefill_kernel(AttnArgs a) {
     if (kb + 32 < hi) attend(t1, kb + 32);
     fetch(t1, kb + 96);
   }
-  bf16_t* out = static_cast<bf16_t*>(a.out);
 #pragma unroll
   for (int nq = 0; nq < PREFILL_NQ; ++nq) {
     float total = l[nq];
     total += __shfl_xor(total, 16, 64);
     total += __shfl_xor(total, 32, 64);
     total += bt_sink_term_pow2(a.sink, head, m[nq]);
-    float inv = total > 0.f ? 1.0f / total : 0.f;
+    float inv = FORM == 2 ? 1.0f : total > 0.f ? 1.0f / total : 0.f;
     if (qpos[nq] < 0) continue;
+    const float head_gate = head_gate_of(a, tok[nq], head);
 #pragma unroll
     for (int dt = 0; dt < ND; ++dt) {
-      bf16x4 packed = {(bf16_t)(o[nq][dt][0] * inv), (bf16_t)(o[nq][dt][1] * inv), (bf16_t)(o[nq][dt][2] * inv),
-                       (bf16_t)(o[nq][dt][3] * inv)};
-      *reinterpret_cast<bf16x4*>(out + (int64_t)tok[nq] * a.ldo + head * HD + dt * 16 + 4 * g) = packed;
+      const float row[4] = {o[nq][dt][0] * inv, o[nq][dt][1] * inv, o[nq][dt][2] * inv, o[nq][dt][3] * inv};
+      put4(a, tok[nq], head, dt * 16 + 4 * g, row, head_gate);
     }
   }
 }
@@ -353,7 +433,7 @@ struct BlockOperands {
 
 template <int NQ>
 __device__ __forceinline__ void attend_block(const BlockOperands& blk, int kb, int valid_end, bool masked,
-                                             const int (&qpos)[NQ], float c, const bf16x8 (&q)[NQ][NKS],
+                                             const int (&qpos)[NQ], const Scoring& sc, const bf16x8 (&q)[NQ][NKS],
                                              floatx4 (&o)[NQ][ND], float (&m)[NQ], floatx4 (&rows)[NQ]) {
   const int lane = threadIdx.x & 63, g = lane >> 4;
   floatx4 s[NQ][4];
@@ -367,6 +447,14 @@ __device__ __forceinline__ void attend_block(const BlockOperands& blk, int kb, i
         acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(blk.k[t][ks], q[nq][ks], acc, 0, 0, 0);
       s[nq][t] = acc;
     }
+  }
+  if constexpr (FORM == 1) {
+#pragma unroll
+    for (int nq = 0; nq < NQ; ++nq)
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) s[nq][t][r] = capped_exponent(s[nq][t][r], sc);
   }
   if (masked) {
 #pragma unroll
@@ -382,11 +470,12 @@ __device__ __forceinline__ void attend_block(const BlockOperands& blk, int kb, i
   bool behind = false;
 #pragma unroll
   for (int nq = 0; nq < NQ; ++nq) {
+    if constexpr (FORM == 2) continue;
     const float m_use = m[nq] == -INFINITY ? 0.f : m[nq];
 #pragma unroll
     for (int t = 0; t < 4; ++t)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) s[nq][t][r] = fmaf(s[nq][t][r], c, -m_use);
+      for (int r = 0; r < 4; ++r) s[nq][t][r] = FORM == 1 ? s[nq][t][r] - m_use : fmaf(s[nq][t][r], sc.c, -m_use);
     float top = -INFINITY;
 #pragma unroll
     for (int t = 0; t < 4; ++t)
@@ -420,10 +509,12 @@ __device__ __forceinline__ void attend_block(const BlockOperands& blk, int kb, i
 #pragma unroll
     for (int t = 0; t < 4; ++t)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) pop[nq][t >> 1][4 * (t & 1) + r] = (bf16_t)__builtin_amdgcn_exp2f(s[nq][t][r]);
+      for (int r = 0; r < 4; ++r)
+        pop[nq][t >> 1][4 * (t & 1) + r] = (bf16_t)(FORM == 2 ? sigmoid_weight(s[nq][t][r], sc) : __builtin_amdgcn_exp2f(s[nq][t][r]));
   }
   const bf16_t one = (bf16_t)1.0f;
   const bf16x8 ones = {one, one, one, one, one, one, one, one};
+  if constexpr (FORM != 2)
 #pragma unroll
   for (int half = 0; half < 2; ++half)
 #pragma unroll
@@ -622,12 +713,12 @@ attention_prefill_split_kernel(AttnArgs a) {
 #pragma unroll
     for (int dt = 0; dt < ND; ++dt) o[nq][dt] = floatx4{0.f, 0.f, 0.f, 0.f};
     rows[nq] = floatx4{0.f, 0.f, 0.f, 0.f};
-    m[nq] = -INFINITY;
+    m[nq] = FIRST_MAXIMUM;
   }
   const int last = q0 + PREFILL_QUERIES_PER_WAVE < count ? q0 + PREFILL_QUERIES_PER_WAVE : count;
   const int hi = active ? start + last : 0;     // one past the position of this wave's last query
   const int valid_end = start + count;
-  const float c = a.scale * LOG2_E;
+  const Scoring sc = scoring_of(a, head);
   const int whole_until = start + q0 + 1;       // blocks ending here or before are seen whole
 
   if (empty_run) {       // a run beyond the tile's last turn: its records say that it saw no key
@@ -662,7 +753,7 @@ attention_prefill_split_kernel(AttnArgs a) {
         for (int half = 0; half < 2; ++half)
           blk.v[dt][half] = *reinterpret_cast<const bf16x8*>(stage + SHARED_K_BYTES +
                                                              ((4 * half + g) * 64 + dt * 16 + i16) * 16);
-      attend_block<PREFILL_NQ>(blk, kb, valid_end, kb + 64 > whole_until, qpos, c, q, o, m, rows);
+      attend_block<PREFILL_NQ>(blk, kb, valid_end, kb + 64 > whole_until, qpos, sc, q, o, m, rows);
     }
     __syncthreads();   // turn t + 1 is in place, and everyone is done with turn t before it is overwritten
   }
@@ -684,7 +775,6 @@ attention_prefill_split_kernel(AttnArgs a) {
   }
   __syncthreads();
   if (set == 1 || !active) return;
-  bf16_t* out = static_cast<bf16_t*>(a.out);
 #pragma unroll
   for (int nq = 0; nq < PREFILL_NQ; ++nq) {
     const int k0 = nq * PER_QUERY;
@@ -695,7 +785,7 @@ attention_prefill_split_kernel(AttnArgs a) {
     const float theirs = m_other == -INFINITY ? 0.f : exp2f(m_other - top);
     const float total = rows[nq][0] * mine + l_other * theirs;   // (whole sums: see attend_block)
     // (with runs the sink joins the denominator once, where the runs are joined)
-    float inv = total > 0.f ? 1.0f / (total + bt_sink_term_pow2(a.sink, head, top)) : 0.f;
+    float inv = FORM == 2 ? 1.0f : total > 0.f ? 1.0f / (total + bt_sink_term_pow2(a.sink, head, top)) : 0.f;
     if (qpos[nq] < 0) continue;
     if (runs > 1) {      // this run's share of the query's row, relative to its own maximum
       typedef __attribute__((__vector_size__(2 * sizeof(float)))) float float2v;
@@ -715,14 +805,14 @@ attention_prefill_split_kernel(AttnArgs a) {
       }
       continue;
     }
+    const float head_gate = head_gate_of(a, tok[nq], head);
 #pragma unroll
     for (int dt = 0; dt < ND; ++dt) {
       float joined[4];
 #pragma unroll
       for (int r = 0; r < 4; ++r)
         joined[r] = (o[nq][dt][r] * mine + hand[((k0 + 2 + 4 * dt + r) * PREFILL_WAVES + wave) * 64 + lane] * theirs) * inv;
-      bf16x4 packed = {(bf16_t)joined[0], (bf16_t)joined[1], (bf16_t)joined[2], (bf16_t)joined[3]};
-      *reinterpret_cast<bf16x4*>(out + (int64_t)tok[nq] * a.ldo + head * HD + dt * 16 + 4 * g) = packed;
+      put4(a, tok[nq], head, dt * 16 + 4 * g, joined, head_gate);
     }
   }
 }
@@ -775,7 +865,7 @@ attention_decode_kernel(AttnArgs a) {
   int qpos[1] = {has_query ? pos : -1};
   const int qlo[1] = {bt_first_seen(pos, a.window, a.chunk)};
   floatx4 o[1][ND];
-  float m[1] = {-INFINITY}, l[1] = {0.f};
+  float m[1] = {FIRST_MAXIMUM}, l[1] = {0.f};
 #pragma unroll
   for (int dt = 0; dt < ND; ++dt) o[0][dt] = floatx4{0.f, 0.f, 0.f, 0.f};
 
@@ -792,7 +882,7 @@ attention_decode_kernel(AttnArgs a) {
     int block = (early && j < 2) ? (j == 0 ? early_block0 : early_block1) : block_row[kb / BT_KV_BLOCK];
     return kv_plane(a.kv, block, kv_head);
   };
-  const float c = a.scale * LOG2_E;
+  const Scoring sc = scoring_of(a, head);
   auto fetch = [&](TileOperands& into, int kb, int j) {
     if (kb < end) {
       int64_t plane = plane_of(kb, j);
@@ -800,7 +890,7 @@ attention_decode_kernel(AttnArgs a) {
     }
   };
   auto attend = [&](const TileOperands& tile, int kb) {   // one form: this kernel waits for memory, not for the ALU
-    attend_tile<1, true>(tile, kb, pos + 1, qpos, qlo, c, q, o, m, l);
+    attend_tile<1, true>(tile, kb, pos + 1, qpos, qlo, sc, q, o, m, l);
   };
   TileOperands current, next;
   fetch(next, first, 0);
@@ -824,7 +914,6 @@ attention_decode_kernel(AttnArgs a) {
       for (int r = 0; r < 4; ++r) sm_o[(wave * group + i16) * HD + dt * 16 + 4 * g + r] = o[0][dt][r];
   }
   __syncthreads();
-  bf16_t* out = static_cast<bf16_t*>(a.out);
   for (int e = threadIdx.x; e < group * HD; e += DECODE_WAVES * 64) {
     int j = e / HD, channel = e % HD;
     float top = sm_m[j];
@@ -841,8 +930,7 @@ attention_decode_kernel(AttnArgs a) {
     }
     if (splits == 1) {
       den += top != -INFINITY ? bt_sink_term_pow2(a.sink, kv_head * group + j, top) : 0.f;
-      out[activation_offset<bf16_t>(a.out_rows, a.ldo, tok, (kv_head * group + j) * HD + channel)] =
-          (bf16_t)(den > 0.f ? num / den : 0.f);
+      put1(a, tok, kv_head * group + j, channel, FORM == 2 ? num : den > 0.f ? num / den : 0.f);
     } else {     // this run's share, for attention_join_kernel
       float* mine = a.partial + (((int64_t)seq * a.q_heads + kv_head * group + j) * splits + split) * (HD + 2);
       mine[channel] = num;
@@ -902,12 +990,10 @@ attention_join_kernel(AttnArgs a, int n_rows) {
     top = new_top;
   }
   if (top != -INFINITY) den += bt_sink_term_pow2(a.sink, head, top);
-  bf16_t* out = static_cast<bf16_t*>(a.out);
 #pragma unroll
   for (int c = 0; c < NCH; ++c) {
     const int channel = lane + 64 * c;
-    if (channel < HD)
-      out[activation_offset<bf16_t>(a.out_rows, a.ldo, row, head * HD + channel)] = (bf16_t)(den > 0.f ? num[c] / den : 0.f);
+    if (channel < HD) put1(a, row, head, channel, FORM == 2 ? num[c] : den > 0.f ? num[c] / den : 0.f);
   }
 }
 
@@ -919,6 +1005,12 @@ static int check_args(const AttnArgs& a, const char* who) {
   if (!(a.scale > 0.f)) BT_REFUSE("%s: the score scale %g must be positive (the maximum is taken before scaling)", who, a.scale);
   if (!a.q || !a.out || !a.seq_off || !a.seq_start || !a.kv.blocks || !a.kv.keys || !a.kv.values)
     BT_REFUSE("%s: missing operand", who);
+  if (a.form != FORM || (!STAGED && (a.gate || a.out_f32)))
+    BT_REFUSE("%s: built for form %d of the scores%s, asked for form %d%s", who, FORM, STAGED ? "" : " without an output stage",
+              a.form, a.gate || a.out_f32 ? " with one" : "");
+  if (const char* wrong = bt_check_form(a)) BT_REFUSE("%s: %s", who, wrong);
+  if (a.out_f32 && (a.out_rows != 0 || ((uintptr_t)a.out & 15)))
+    BT_REFUSE("%s: a 32-bit output is row-major and 16-byte aligned", who);
   if (a.ldq % 8 != 0 || a.ldo % 4 != 0 || ((uintptr_t)a.q & 15) || ((uintptr_t)a.out & 7))
     BT_REFUSE("%s: query rows must be 16-byte and output rows 8-byte aligned", who);
   return BT_OK;

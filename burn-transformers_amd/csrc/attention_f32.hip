@@ -34,6 +34,23 @@
 #include "attention.h"
 #include "calls.h"
 
+// BT_ATTENTION_FORM (0, 1, 2: AttnArgs.form) builds the module for that form of the scores and with the output stage
+// (gate); without it the module is the softmax alone.
+#ifdef BT_ATTENTION_FORM
+constexpr int FORM = BT_ATTENTION_FORM;
+constexpr bool STAGED = true;
+#else
+constexpr int FORM = 0;
+constexpr bool STAGED = false;
+#endif
+#define LOG2_E 1.4426950408889634f
+// the running maximum before the first key: sigmoid weights have none, zero stands for it
+constexpr float FIRST_MAXIMUM = FORM == 2 ? 0.f : -INFINITY;
+
+__device__ __forceinline__ float output_gate(const AttnArgs& a, int64_t tok, int head, int channel) {
+  return STAGED ? bt_output_gate(a, tok, head, channel) : 1.f;
+}
+
 #define F32M_QUERIES 64
 
 template <int HD>
@@ -115,8 +132,9 @@ attention_f32_mfma_kernel(AttnArgs a) {
     }
   };
 
-  const float c2 = a.scale * 1.4426950408889634f;            // scores to powers of two
-  float run_max = -INFINITY, run_sum = 0.f;                  // run_sum: the lane's share; the four lanes of a query meet at the end
+  const float c2 = FORM == 1 ? LOG2_E : a.scale * LOG2_E;     // scores to powers of two (form 1: they are scaled before)
+  const float bias = FORM == 2 && a.score_bias ? a.score_bias[head] : 0.f;
+  float run_max = FIRST_MAXIMUM, run_sum = 0.f;                  // run_sum: the lane's share; the four lanes of a query meet at the end
   floatx4 o[KS];
 #pragma unroll
   for (int dt = 0; dt < KS; ++dt) o[dt] = floatx4{0.f, 0.f, 0.f, 0.f};
@@ -154,6 +172,12 @@ attention_f32_mfma_kernel(AttnArgs a) {
     floatx4 v4[2][KS];
 #pragma unroll
     for (int dt = 0; dt < KS; ++dt) v4[0][dt] = *reinterpret_cast<const floatx4*>(vcol + 64 * dt);
+    if constexpr (FORM == 1) {
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) s[t][r] = a.cap * tanhf(s[t][r] * a.scale / a.cap);
+    }
     // a block that every query of the wave sees whole needs no comparisons
     const bool whole = kb + BT_KV_BLOCK - 1 <= wave_first && kb >= wave_hi_lo;
     if (!whole) {
@@ -166,29 +190,36 @@ attention_f32_mfma_kernel(AttnArgs a) {
           s[t][r] = seen ? s[t][r] : -INFINITY;
         }
     }
-    float top = -INFINITY;
+    if constexpr (FORM == 2) {           // every key's weight by itself; an excluded key's -inf gives exactly zero
 #pragma unroll
-    for (int t = 0; t < 4; ++t) top = fmaxf(top, fmaxf(fmaxf(s[t][0], s[t][1]), fmaxf(s[t][2], s[t][3])));
-    top = fmaxf(top, __shfl_xor(top, 16, 64));
-    top = fmaxf(top, __shfl_xor(top, 32, 64));
-    const float new_max = fmaxf(run_max, top * c2);          // in powers of two
-    // nothing seen so far, this block included: everything stays at its start
-    const float rescale = new_max == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(run_max - new_max);   // 2^-inf = 0 at the first block seen
-    const float m_use = new_max == -INFINITY ? 0.f : new_max;
-    float block_sum = 0.f;
+      for (int t = 0; t < 4; ++t)
 #pragma unroll
-    for (int t = 0; t < 4; ++t)
+        for (int r = 0; r < 4; ++r) s[t][r] = bt_sigmoid(fmaf(s[t][r], a.scale, bias));
+    } else {
+      float top = -INFINITY;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        s[t][r] = __builtin_amdgcn_exp2f(fmaf(s[t][r], c2, -m_use));
-        block_sum += s[t][r];
-      }
-    run_sum = fmaf(run_sum, rescale, block_sum);
-    run_max = new_max;
+      for (int t = 0; t < 4; ++t) top = fmaxf(top, fmaxf(fmaxf(s[t][0], s[t][1]), fmaxf(s[t][2], s[t][3])));
+      top = fmaxf(top, __shfl_xor(top, 16, 64));
+      top = fmaxf(top, __shfl_xor(top, 32, 64));
+      const float new_max = fmaxf(run_max, top * c2);          // in powers of two
+      // nothing seen so far, this block included: everything stays at its start
+      const float rescale = new_max == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(run_max - new_max);   // 2^-inf = 0 at the first block seen
+      const float m_use = new_max == -INFINITY ? 0.f : new_max;
+      float block_sum = 0.f;
 #pragma unroll
-    for (int dt = 0; dt < KS; ++dt)
+      for (int t = 0; t < 4; ++t)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) o[dt][r] *= rescale;
+        for (int r = 0; r < 4; ++r) {
+          s[t][r] = __builtin_amdgcn_exp2f(fmaf(s[t][r], c2, -m_use));
+          block_sum += s[t][r];
+        }
+      run_sum = fmaf(run_sum, rescale, block_sum);
+      run_max = new_max;
+#pragma unroll
+      for (int dt = 0; dt < KS; ++dt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[dt][r] *= rescale;
+    }
 #pragma unroll
     for (int t = 0; t < 4; ++t) {
       if (t + 1 < 4) {
@@ -206,12 +237,17 @@ attention_f32_mfma_kernel(AttnArgs a) {
   total += __shfl_xor(total, 32, 64);
   total += bt_sink_term_pow2(a.sink, head, run_max);        // (the maximum is the same in a query's four lanes)
   if (exists) {
-    float* out = static_cast<float*>(a.out) + (int64_t)(off + q0 + mine) * a.ldo + head * HD;
+    const int64_t tok = off + q0 + mine;
+    float* out = static_cast<float*>(a.out) + tok * a.ldo + head * HD;
+    const float head_gate = STAGED && a.gate_span == 0 ? output_gate(a, tok, head, 0) : 1.f;
 #pragma unroll
     for (int dt = 0; dt < KS; ++dt) {
       floatx4 r4;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) r4[r] = total > 0.f ? o[dt][r] / total : 0.f;
+      for (int r = 0; r < 4; ++r) {
+        r4[r] = FORM == 2 ? o[dt][r] : total > 0.f ? o[dt][r] / total : 0.f;
+        if constexpr (STAGED) r4[r] *= a.gate_span == 1 ? output_gate(a, tok, head, 16 * dt + 4 * g + r) : head_gate;
+      }
       *reinterpret_cast<floatx4*>(out + 16 * dt + 4 * g) = r4;
     }
   }
@@ -249,7 +285,8 @@ attention_f32_decode_kernel(AttnArgs a) {
   }
   const float* keys = static_cast<const float*>(a.kv.keys);
   const float* values = static_cast<const float*>(a.kv.values);
-  float run_max = -INFINITY, run_sum = 0.f, acc[CPT];
+  const float bias = FORM == 2 && a.score_bias ? a.score_bias[head] : 0.f;
+  float run_max = FIRST_MAXIMUM, run_sum = 0.f, acc[CPT];
 #pragma unroll
   for (int j = 0; j < CPT; ++j) acc[j] = 0.f;
   for (int block = first_block + wave; block <= last_block; block += 4) {
@@ -274,12 +311,18 @@ attention_f32_decode_kernel(AttnArgs a) {
     }
     const int key_pos = block * BT_KV_BLOCK + lane;
     const bool seen = key_pos <= pos && key_pos >= lo;
-    const float score = seen ? s * a.scale : -INFINITY;
-    const float new_max = fmaxf(run_max, wave_max(score));          // finite: the block holds at least one seen key
-    const float p = expf(score - new_max);
-    const float rescale = expf(run_max - new_max);                  // exp(-inf) = 0 at the wave's first block
-    run_sum = fmaf(run_sum, rescale, wave_sum(p));
-    run_max = new_max;
+    float p, rescale = 1.f;
+    if constexpr (FORM == 2) {
+      p = seen ? bt_sigmoid(fmaf(s, a.scale, bias)) : 0.f;
+    } else {
+      const float scaled = FORM == 1 ? a.cap * tanhf(s * a.scale / a.cap) : s * a.scale;
+      const float score = seen ? scaled : -INFINITY;
+      const float new_max = fmaxf(run_max, wave_max(score));        // finite: the block holds at least one seen key
+      p = expf(score - new_max);
+      rescale = expf(run_max - new_max);                            // exp(-inf) = 0 at the wave's first block
+      run_sum = fmaf(run_sum, rescale, wave_sum(p));
+      run_max = new_max;
+    }
     ps[wave][lane] = p;                                             // read back below by this wave only
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
     __builtin_amdgcn_wave_barrier();
@@ -332,7 +375,7 @@ attention_f32_decode_kernel(AttnArgs a) {
       }
       if (splits == 1) {
         den += bt_sink_term(a.sink, head, top);
-        out[channel] = den > 0.f ? num / den : 0.f;
+        out[channel] = (FORM == 2 ? num : den > 0.f ? num / den : 0.f) * output_gate(a, seq, head, channel);
       } else {                                                      // this run's share, for attention_f32_join_kernel
         mine[channel] = num;
         if (channel == 0) {
@@ -362,7 +405,7 @@ attention_f32_join_kernel(AttnArgs a) {
       den = fmaf(runs[s * (hd + 2) + hd + 1], f, den);
     }
     den += bt_sink_term(a.sink, head, top);
-    out[channel] = den > 0.f ? num / den : 0.f;
+    out[channel] = (FORM == 2 ? num : den > 0.f ? num / den : 0.f) * output_gate(a, seq, head, channel);
   }
 }
 
@@ -398,6 +441,10 @@ BT_EXPORT int bt_attention_f32(void* stream, const AttnArgs* args) {
   if (!(a.scale > 0.f)) BT_REFUSE("attention_f32: scale %g must be positive", (double)a.scale);
   if (!a.q || !a.out || !a.seq_off || !a.seq_start || !a.kv.blocks || !a.kv.keys || !a.kv.values)
     BT_REFUSE("attention_f32: missing operand");
+  if (a.form != FORM || (!STAGED && a.gate))
+    BT_REFUSE("attention_f32: built for form %d of the scores%s, asked for form %d%s", FORM,
+              STAGED ? "" : " without an output stage", a.form, a.gate ? " with one" : "");
+  if (const char* wrong = bt_check_form(a)) BT_REFUSE("attention_f32: %s", wrong);
   if (a.ldq % 4 != 0 || ((uintptr_t)a.q & 15) || ((uintptr_t)a.kv.keys & 15) || ((uintptr_t)a.kv.values & 15))
     BT_REFUSE("attention_f32: queries, keys and values are read 16 bytes at a time (row pitch %lld)", (long long)a.ldq);
   if (a.max_count == 1 && a.n_tokens == a.n_seqs) {      // a decode step: one token per sequence, in their order

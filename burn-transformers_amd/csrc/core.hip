@@ -462,7 +462,8 @@ BT_EXPORT int bt_gemm_plain(void* stream, int dtype, const void* A, int64_t lda,
 // Plain attention over the paged cache.  One work-group per (token, query head).
 //   scores s_k = scale * (q . key_k) for keys lo <= k <= pos, lo = max(0, pos - window + 1), or the
 //   first position of pos's chunk if that is later (bt_first_seen)
-//   out = sum_k softmax(s)_k value_k, softmax in 32-bit with a running maximum over chunks.
+//   out = sum_k softmax(s)_k value_k, softmax in 32-bit with a running maximum over chunks; the other forms of
+//   the scores and the output stage (AttnArgs) as in the tiled kernels, decided as the kernel runs.
 // Keys beyond the token's own position are never read.
 // ---------------------------------------------------------------------------------------------
 #define PLAIN_CHUNK 1024
@@ -485,7 +486,8 @@ attention_plain_kernel(AttnArgs a) {
   for (int c = threadIdx.x; c < hd; c += blockDim.x) qs[c] = to_float(q[c]);
   __syncthreads();
   int lo = bt_first_seen(pos, a.window, a.chunk);
-  float run_max = -INFINITY, run_sum = 0.f;
+  float run_max = a.form == 2 ? 0.f : -INFINITY, run_sum = 0.f;
+  const float bias = a.form == 2 && a.score_bias ? a.score_bias[head] : 0.f;
   float acc[PLAIN_PER_THREAD];                          // channels threadIdx.x, threadIdx.x + 256, ... (< hd)
 #pragma unroll
   for (int j = 0; j < PLAIN_PER_THREAD; ++j) acc[j] = 0.f;
@@ -500,16 +502,17 @@ attention_plain_kernel(AttnArgs a) {
       float s = 0.f;
       for (int c = 0; c < hd; ++c) s = fmaf(qs[c], to_float(kr[c]), s);
       s *= a.scale;
+      if (a.form == 1) s = a.cap * tanhf(s / a.cap);
       ps[i] = s;
       local_max = fmaxf(local_max, s);
     }
     float chunk_max = block_max(local_max, scratch);
-    float new_max = fmaxf(run_max, chunk_max);
+    float new_max = a.form == 2 ? 0.f : fmaxf(run_max, chunk_max);
     float rescale = (run_max == -INFINITY) ? 0.f : expf(run_max - new_max);
     float local_sum = 0.f;
     __syncthreads();
     for (int i = threadIdx.x; i < n; i += blockDim.x) {
-      float p = expf(ps[i] - new_max);
+      float p = a.form == 2 ? bt_sigmoid(ps[i] + bias) : expf(ps[i] - new_max);
       ps[i] = p;
       local_sum += p;
     }
@@ -531,11 +534,16 @@ attention_plain_kernel(AttnArgs a) {
     __syncthreads();
   }
   run_sum += bt_sink_term(a.sink, head, run_max);
-  T* o = static_cast<T*>(a.out) + (int64_t)t * a.ldo + head * hd;
+  const int64_t place = (int64_t)t * a.ldo + head * hd;
 #pragma unroll
   for (int j = 0; j < PLAIN_PER_THREAD; ++j) {
     const int channel = threadIdx.x + 256 * j;
-    if (channel < hd) o[channel] = from_float<T>(run_sum > 0.f ? acc[j] / run_sum : 0.f);
+    if (channel >= hd) break;
+    const float v = (a.form == 2 ? acc[j] : run_sum > 0.f ? acc[j] / run_sum : 0.f) * bt_output_gate(a, t, head, channel);
+    if (a.out_f32)
+      static_cast<float*>(a.out)[place + channel] = v;
+    else
+      static_cast<T*>(a.out)[place + channel] = from_float<T>(v);
   }
 }
 
@@ -550,6 +558,7 @@ int bt_check_attention(const AttnArgs& a, const char* who) {
   if (!a.q || !a.out || !a.tok_seq || !a.tok_pos || !a.seq_off || !a.seq_start || !a.kv.blocks ||
       !a.kv.keys || !a.kv.values)
     BT_REFUSE("%s: missing operand", who);
+  if (const char* wrong = bt_check_form(a)) BT_REFUSE("%s: %s", who, wrong);
   return BT_OK;
 }
 

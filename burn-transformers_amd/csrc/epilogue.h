@@ -12,11 +12,14 @@ enum EpilogueMode {
   EPI_F32 = 2,    // out[split][m][n] = acc (+ bias in split 0)  (float; the consumer sums the splits)
   EPI_QKV = 3,    // columns [0,n_q) -> out, [n_q,n_q+n_kv) -> keys, the next n_kv -> values
   EPI_RESIDUAL = 4,  // out[m][n] += acc + bias                  (float: the residual stream itself)
+  EPI_F32_ACT = 5,   // columns [0,n_q) -> out as in EPI_F32, those behind -> act(acc + bias) in out2 (element type T), columns
+                     //   from 0: two products of the same rows as one (the skinny kernel only)
 };
 
 enum Activation {
   ACT_GELU_TANH = 0,
   ACT_GELU_ERF = 1,
+  ACT_SQUARED_RELU = 2,
 };
 
 // Mirrored field by field by a ctypes.Structure on the Python side.
@@ -32,7 +35,9 @@ struct Epilogue {
   const int* tok_seq;    // [M] index of the token's sequence in the step
   const int* tok_pos;    // [M] position of the token in its sequence
   KvView kv;
-  int out_rows;          // EPI_STORE, EPI_ACT: 0, or `out` is chunk-major with that many rows (activation_offset)
+  int out_rows;          // EPI_STORE, EPI_ACT (EPI_F32_ACT: `out2`): 0, or `out` is chunk-major with that many rows (activation_offset)
+  void* out2;            // EPI_F32_ACT only
+  int64_t ldo2;
 };
 
 // 32-bit activations.  The float32 path (T = float) uses the library's tanhf / erff; the
@@ -48,6 +53,7 @@ __device__ __forceinline__ float activate(float x, int act) {
     if (sizeof(T) == 2) return x / (1.0f + __expf(-2.0f * inner));
     return 0.5f * x * (1.0f + tanhf(inner));
   }
+  if (act == ACT_SQUARED_RELU) return x > 0.f ? x * x : 0.f;
   // x (1 + erf(x / sqrt 2)) / 2
   return 0.5f * x * (1.0f + erff(x * 0.7071067811865476f));
 }
@@ -149,6 +155,16 @@ __device__ __forceinline__ void epilogue4_prefetched(const Epilogue& e, int N, i
                   v, count, aligned);
   } else if (e.mode == EPI_RESIDUAL) {
     store4<float>(static_cast<float*>(e.out) + (int64_t)m * e.ldo + n0, v, count, aligned);
+  } else if (e.mode == EPI_F32_ACT) {
+    if (n0 < e.n_q) {
+      store4<float>(static_cast<float*>(e.out) + (int64_t)m * e.ldo + n0, v, count, aligned);
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = activate<T>(v[i], e.act);
+      const int c = n0 - e.n_q;
+      if (e.out_rows == 0) store4<T>(static_cast<T*>(e.out2) + (int64_t)m * e.ldo2 + c, v, count, (e.ldo2 & 3) == 0);
+      else store4<T>(static_cast<T*>(e.out2) + activation_offset<T>(e.out_rows, e.ldo2, m, c), v, count, true);
+    }
   } else {
     if (n0 < e.n_q) {
       store4<T>(static_cast<T*>(e.out) + (int64_t)m * e.ldo + n0, v, count, aligned);

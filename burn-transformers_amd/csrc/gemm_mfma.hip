@@ -840,10 +840,12 @@ static int check_operands(const char* who, int elems, const void* A, int64_t lda
   if (K % elems != 0 || lda % elems != 0)
     BT_REFUSE("%s: K %d and the row pitch %lld must be multiples of %d (16-byte loads)", who, K, (long long)lda, elems);
   if (((uintptr_t)A & 15) || ((uintptr_t)W & 15)) BT_REFUSE("%s: operands must be 16-byte aligned", who);
-  if (e.mode < 0 || e.mode > 4 || e.out == nullptr) BT_REFUSE("%s: bad epilogue", who);
+  if (e.mode < 0 || e.mode > 5 || e.out == nullptr) BT_REFUSE("%s: bad epilogue", who);
+  if (e.mode == EPI_F32_ACT && (!e.out2 || e.n_q <= 0 || e.n_q >= N || e.n_q % 4 != 0))
+    BT_REFUSE("%s: %d of %d columns in 32-bit, the others activated: a multiple of four, and a place for each", who, e.n_q, N);
   if (splits < 1 || (splits > 1 && e.mode != EPI_F32))
     BT_REFUSE("%s: K can be split %d ways only into 32-bit partial sums", who, splits);
-  if (e.out_rows != 0 && ((e.mode != EPI_STORE && e.mode != EPI_ACT) || e.out_rows < M))
+  if (e.out_rows != 0 && ((e.mode != EPI_STORE && e.mode != EPI_ACT && e.mode != EPI_F32_ACT) || e.out_rows < M))
     BT_REFUSE("%s: a chunk-major output of %d rows for %d rows (stored or activated results only)", who, e.out_rows, M);
   if (e.mode == EPI_QKV) {
     if (e.kv.head_dim <= 0 || e.kv.head_dim % 16 != 0)
@@ -906,6 +908,7 @@ BT_EXPORT int bt_gemm_tile(void* stream, int dtype, const void* A, int64_t lda, 
                            const Epilogue* epi, int splits, int variant) {
   if (M <= 0) return BT_OK;
   if (dtype != 0 && dtype != 1) BT_REFUSE("gemm_tile: element type %d is neither float nor bfloat16", dtype);
+  if (epi->mode == EPI_F32_ACT) BT_REFUSE("gemm_tile: 32-bit and activated columns of one product are the skinny kernel's");
   int rc = check_operands("gemm_tile", dtype == 0 ? 4 : 8, A, lda, W, M, N, K, *epi, splits);
   if (rc) return rc;
   hipStream_t s = (hipStream_t)stream;

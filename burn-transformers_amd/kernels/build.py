@@ -87,12 +87,21 @@ def entry_points(name):
 
 
 # the package's own modules
-for _name in ("core", "gemm_mfma", "attention_f32", "sublayer", "latent", "state_space", "rotary", "experts", "linear_attention"):
+for _name in ("core", "gemm_mfma", "attention_f32", "sublayer", "latent", "state_space", "rotary", "experts", "linear_attention",
+              "differential"):
     register_module(_name, _name + ".hip", _own=True)
 register_module("gemm_library", "gemm_library.hip", ["-ldl"], _own=True)   # host code around hipBLASLt, opened at run time
 register_module("program", "program.cpp", _own=True)                       # the host loop that walks a launch list
 for _size in ATTENTION_HEAD_SIZES:                                         # the bfloat16 attention, once per head size
     register_module(f"attention_bf16_hd{_size}", "attention_bf16.hip", [f"-DBT_HEAD_DIM={_size}"], _own=True)
+# the tiled attention kernels with an output stage (gate, 32-bit rows), once per form of the scores: modules of their own,
+# so that the plain softmax's kernels carry none of it
+ATTENTION_FORMS = ("softmax", "capped", "sigmoid")
+for _form, _name in enumerate(ATTENTION_FORMS):
+    register_module(f"attention_f32_{_name}", "attention_f32.hip", [f"-DBT_ATTENTION_FORM={_form}"], _own=True)
+    for _size in ATTENTION_HEAD_SIZES:
+        register_module(f"attention_bf16_hd{_size}_{_name}", "attention_bf16.hip",
+                        [f"-DBT_HEAD_DIM={_size}", f"-DBT_ATTENTION_FORM={_form}"], _own=True)
 
 
 def all_modules():

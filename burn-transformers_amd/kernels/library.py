@@ -17,8 +17,8 @@ from . import build
 FLOAT32, BFLOAT16 = 0, 1
 DTYPE_CODES = {torch.float32: FLOAT32, torch.bfloat16: BFLOAT16}
 
-EPI_STORE, EPI_ACT, EPI_F32, EPI_QKV, EPI_RESIDUAL = 0, 1, 2, 3, 4
-ACTIVATIONS = {"gelu_tanh": 0, "gelu_erf": 1}
+EPI_STORE, EPI_ACT, EPI_F32, EPI_QKV, EPI_RESIDUAL, EPI_F32_ACT = 0, 1, 2, 3, 4, 5
+ACTIVATIONS = {"gelu_tanh": 0, "gelu_erf": 1, "squared_relu": 2}
 NORM_KINDS = {"layer_norm": 0, "rms_norm": 1}
 KV_BLOCK = 64
 
@@ -40,7 +40,8 @@ class KvView(ctypes.Structure):
 class Epilogue(ctypes.Structure):
     _fields_ = [("mode", _c_int), ("act", _c_int), ("bias", _c_ptr), ("out", _c_ptr),
                 ("ldo", _c_i64), ("split_stride", _c_i64), ("n_q", _c_int), ("n_kv", _c_int),
-                ("tok_seq", _c_ptr), ("tok_pos", _c_ptr), ("kv", KvView), ("out_rows", _c_int)]
+                ("tok_seq", _c_ptr), ("tok_pos", _c_ptr), ("kv", KvView), ("out_rows", _c_int), ("out2", _c_ptr),
+                ("ldo2", _c_i64)]
 
 
 class AttnArgs(ctypes.Structure):
@@ -48,7 +49,9 @@ class AttnArgs(ctypes.Structure):
                 ("tok_seq", _c_ptr), ("tok_pos", _c_ptr), ("seq_off", _c_ptr), ("seq_start", _c_ptr),
                 ("kv", KvView), ("q_heads", _c_int), ("n_tokens", _c_int), ("n_seqs", _c_int),
                 ("max_count", _c_int), ("window", _c_int), ("scale", _c_float), ("splits", _c_int),
-                ("partial", _c_ptr), ("out_rows", _c_int), ("chunk", _c_int), ("sink", _c_ptr)]
+                ("partial", _c_ptr), ("out_rows", _c_int), ("chunk", _c_int), ("sink", _c_ptr), ("form", _c_int),
+                ("cap", _c_float), ("score_bias", _c_ptr), ("gate", _c_ptr), ("ld_gate", _c_i64), ("gate_span", _c_int),
+                ("gate_dim", _c_int), ("out_f32", _c_int)]
 
 
 class NormOperand(ctypes.Structure):
@@ -172,7 +175,15 @@ class HeadRotaryCall(ctypes.Structure):
                 ("vdim", _c_int), ("rot_dims", _c_int), ("eps", _c_float), ("input", _c_ptr), ("ld", _c_i64),
                 ("q_gamma", _c_ptr), ("k_gamma", _c_ptr), ("inv_freq", _c_ptr), ("q_out", _c_ptr), ("ld_q", _c_i64),
                 ("tok_seq", _c_ptr), ("tok_pos", _c_ptr), ("kv", KvView), ("pairing", _c_int), ("norm_span", _c_int),
-                ("amplitude", _c_float)]
+                ("amplitude", _c_float), ("maps", _c_int), ("values_from_keys", _c_int), ("temp_coef", _c_float),
+                ("temp_every", _c_int)]
+    _step_fields_ = {"tokens": "tokens"}
+
+
+class DifferentialCall(ctypes.Structure):
+    _fields_ = [("out_dtype", _c_int), ("tokens", _c_int), ("heads", _c_int), ("vdim", _c_int), ("pitch", _c_int),
+                ("out_cols", _c_int), ("out_rows", _c_int), ("lambda_", _c_float), ("post", _c_float), ("eps", _c_float),
+                ("input", _c_ptr), ("ld", _c_i64), ("out", _c_ptr), ("ld_out", _c_i64)]
     _step_fields_ = {"tokens": "tokens"}
 
 
@@ -262,6 +273,13 @@ class Chunked:
         chunk = 64 // (2 if dtype == torch.bfloat16 else 4)
         padded = (columns + chunk - 1) // chunk * chunk
         return cls(step.buffer(key + ".chunked", rows, padded, dtype), rows, columns)
+
+    def columns_from(self, start, columns):
+        """The columns from ``start`` (a multiple of the chunk) on, as a chunk-major matrix of the same rows."""
+        rows = self.shape[0]
+        chunk = 64 // self.data.element_size()
+        padded = (columns + chunk - 1) // chunk * chunk
+        return Chunked(self.data.view(-1)[start * rows:(start + padded) * rows].view(rows, padded), rows, columns)
 
     def to_rows(self):
         """The same values as a row-major tensor (tests)."""
@@ -655,6 +673,14 @@ def epilogue_f32(out, bias=None):
                     split_stride=split_stride)
 
 
+def epilogue_f32_act(sums, columns, out, activation):
+    """Columns [0, ``columns``) of the product into the float32 rows ``sums``, those behind them through ``activation``
+    into ``out`` (the products' type, or a :class:`Chunked`): two projections of the same rows as one product, for
+    steps of up to 64 rows (the skinny kernel)."""
+    return Epilogue(mode=EPI_F32_ACT, act=ACTIVATIONS[activation], out=sums.data_ptr(), ldo=sums.stride(0), n_q=columns,
+                    out2=out.data_ptr(), ldo2=out.stride(0), out_rows=_out_rows(out))
+
+
 def epilogue_residual(x, bias=None):
     """x[m][n] += acc + bias, with x the float32 residual stream [M, N] itself."""
     return Epilogue(mode=EPI_RESIDUAL, bias=_ptr(bias), out=x.data_ptr(), ldo=x.stride(0))
@@ -762,6 +788,14 @@ class PackedWeight:
             fits = (self.copies[columns], columns) if columns in self.copies else False
             self._fits[(m, splits)] = fits
         return fits or None
+
+
+def takes_two_kinds(a):
+    """Whether a product of the rows ``a`` can leave some columns in 32-bit and others activated (``epilogue_f32_act``):
+    the skinny kernel's steps."""
+    if a.shape[0] > 64:
+        return False
+    return a.dtype == torch.bfloat16 or (a.shape[1] % 4 == 0 and a.stride(0) % 4 == 0)
 
 
 def gemm(a, w, epilogue, splits=1, impl="auto", variant=0, packed=None):
@@ -913,7 +947,8 @@ def _library_has_algorithm(lda, m, n, k, epilogue):
 
 
 def attention_args(q, out, kv_view, tok_seq, tok_pos, seq_off, seq_start, q_heads, n_seqs, max_count,
-                   scale, window=0, partial=None, runs=None, chunk=0, sink=None):
+                   scale, window=0, partial=None, runs=None, chunk=0, sink=None, softcap=0.0, sigmoid=False, score_bias=None,
+                   gate=None, gate_dim=0):
     """``partial``: float32 [rows * q_heads * runs, head_dim + 2] for a step whose keys are cut into
     runs that separate work-groups take.  Decode steps (long contexts in small batches): rows are
     the sequences, and ``runs`` follows from the shape.  Prompt steps (few query tiles behind a long
@@ -922,7 +957,15 @@ def attention_args(q, out, kv_view, tok_seq, tok_pos, seq_off, seq_start, q_head
     ``chunk`` > 0: a query at position p sees only the keys from p - p % chunk on (chunks are counted
     from position 0 of its sequence); ``window`` > 0: only the last ``window`` positions.  ``sink``: float32
     [q_heads], a logit per head whose exponential stands in every softmax's denominator beside the keys'
-    (no key, no value, not scaled)."""
+    (no key, no value, not scaled).  ``softcap`` > 0: scores become softcap * tanh(score / softcap) before the
+    softmax.  ``sigmoid``: no softmax; a visible key weighs sigmoid(score + ``score_bias``[head]) (float32 [q_heads]).
+    ``gate``: float32 logits whose sigmoid multiplies the output, [tokens, >= q_heads] a logit per head, or with
+    ``gate_dim`` [tokens, >= q_heads * gate_dim] one per channel.  A float32 ``out`` of bfloat16 queries keeps the
+    output's digits."""
+    if score_bias is not None and (score_bias.dtype != torch.float32 or score_bias.numel() != q_heads or not score_bias.is_contiguous()):
+        raise KernelError(f"attention: the scores' bias is one float32 number per query head, got {tuple(score_bias.shape)} {score_bias.dtype}")
+    if gate is not None and (gate.dtype != torch.float32 or gate.shape[0] < q.shape[0] or gate.stride(1) != 1):
+        raise KernelError(f"attention: the gate's logits are float32 rows of the step's tokens, got {tuple(gate.shape)} {gate.dtype}")
     if sink is not None and (sink.dtype != torch.float32 or sink.numel() != q_heads or not sink.is_contiguous()):
         raise KernelError(f"attention: the sink is one float32 logit per query head, got {tuple(sink.shape)} {sink.dtype}")
     splits = 1
@@ -937,7 +980,15 @@ def attention_args(q, out, kv_view, tok_seq, tok_pos, seq_off, seq_start, q_head
                     q=q.data_ptr(), ldq=q.stride(0), out=out.data_ptr(), ldo=out.stride(0), out_rows=_out_rows(out),
                     tok_seq=tok_seq.data_ptr(), tok_pos=tok_pos.data_ptr(), seq_off=seq_off.data_ptr(),
                     seq_start=seq_start.data_ptr(), kv=kv_view, q_heads=q_heads, n_tokens=q.shape[0],
-                    n_seqs=n_seqs, max_count=max_count, window=window or 0, scale=scale, chunk=chunk or 0, sink=_ptr(sink))
+                    n_seqs=n_seqs, max_count=max_count, window=window or 0, scale=scale, chunk=chunk or 0, sink=_ptr(sink),
+                    form=2 if sigmoid else 1 if softcap else 0, cap=softcap or 0.0, score_bias=_ptr(score_bias),
+                    gate=_ptr(gate), ld_gate=gate.stride(0) if gate is not None else 0, gate_span=1 if gate_dim else 0,
+                    gate_dim=gate_dim, out_f32=1 if out.dtype == torch.float32 and q.dtype != torch.float32 else 0)
+
+
+def attention_variant(args):
+    """What the tiled kernels' module for these arguments is called behind its base name ("" for the softmax alone)."""
+    return "_" + build.ATTENTION_FORMS[args.form] if args.form or args.gate or args.out_f32 else ""
 
 
 def attention(args, dtype, decode, impl="auto"):
@@ -958,11 +1009,11 @@ def attention(args, dtype, decode, impl="auto"):
     if impl == "tiled":
         if code != FLOAT32:
             raise KernelError("attention: the tiled kernel takes float32 only")
-        _launch(_module("attention_f32"), "bt_attention_f32_call", call)
+        _launch(_module("attention_f32" + attention_variant(args)), "bt_attention_f32_call", call)
         return
     if code != BFLOAT16:
         raise KernelError("attention: the MFMA kernels take bfloat16 only")
-    _launch(_module(f"attention_bf16_hd{args.kv.head_dim}"),
+    _launch(_module(f"attention_bf16_hd{args.kv.head_dim}{attention_variant(args)}"),
             "bt_attention_decode_bf16_call" if decode else "bt_attention_prefill_bf16_call", call)
 
 
@@ -1232,7 +1283,7 @@ def gated_norm(y, z, weight, parts, eps, out):
 # --- rotary positions -------------------------------------------------------------------------
 
 def head_rotary(fused, heads, kv_heads, dim, vdim, rot_dims, inv_freq, q_gamma, k_gamma, eps, q_out, tok_seq, tok_pos,
-                kv_view, dtype, neighbours=False, whole_norm=False, amplitude=1.0):
+                kv_view, dtype, neighbours=False, whole_norm=False, amplitude=1.0, maps=1, values_from_keys=False, temperature=None):
     """Behind a fused query/key/value projection with float32 rows ``fused`` (queries heads * dim, keys
     kv_heads * dim, values kv_heads * vdim): every query and key head divided by its root mean square
     times ``q_gamma`` / ``k_gamma`` ([dim] float32; None: no norm), the first ``rot_dims`` channels of each
@@ -1241,14 +1292,31 @@ def head_rotary(fused, heads, kv_heads, dim, vdim, rot_dims, inv_freq, q_gamma, 
     channels), keys and values into the paged cache at each token's position.
     ``neighbours``: channel 2 i turns with channel 2 i + 1 instead.  ``whole_norm``: the root mean square is
     taken over the token's whole query (key) projection and the scales are [heads * dim] ([kv_heads * dim]).
-    ``amplitude``: a factor on every sine and cosine."""
+    ``amplitude``: a factor on every sine and cosine.
+    ``maps`` 2: a head has two query and two key parts of ``dim`` channels, part by part behind each other in the rows
+    (heads * 2 * dim query columns); part m of query head j becomes query head 2 j + m of ``q_out``, its channels at
+    m * dim and zeros elsewhere, and a key head's parts lie side by side in one cached head.  ``values_from_keys``: the
+    values are the key columns as they come (no value columns).  ``temperature`` (coef, every): queries times
+    1 + coef * ln(floor((position + 1) / every) + 1)."""
+    coef, every = temperature or (0.0, 1)
     _launch(_module("rotary"), "bt_head_rotary_call",
             HeadRotaryCall(dtype=DTYPE_CODES[dtype], tokens=fused.shape[0], heads=heads, kv_heads=kv_heads, dim=dim,
                            vdim=vdim, rot_dims=rot_dims, eps=eps, input=fused.data_ptr(), ld=fused.stride(0),
                            q_gamma=_ptr(q_gamma), k_gamma=_ptr(k_gamma), inv_freq=_ptr(inv_freq),
                            q_out=q_out.data_ptr(), ld_q=q_out.stride(0), tok_seq=tok_seq.data_ptr(),
                            tok_pos=tok_pos.data_ptr(), kv=kv_view, pairing=1 if neighbours else 0,
-                           norm_span=1 if whole_norm else 0, amplitude=amplitude))
+                           norm_span=1 if whole_norm else 0, amplitude=amplitude, maps=maps,
+                           values_from_keys=1 if values_from_keys else 0, temp_coef=coef, temp_every=every))
+
+
+def differential(rows, heads, vdim, pitch, weight, post, eps, out):
+    """out[t, h * vdim + i] = post * d / sqrt(mean_i(d^2) + eps), d = rows[t, 2 h * pitch + i] - weight * rows[t,
+    (2 h + 1) * pitch + i]: the second of a head's two maps taken off the first, normalised per head.  ``rows`` float32;
+    ``out`` may be a :class:`Chunked`; columns behind the heads are set to zero."""
+    _launch(_module("differential"), "bt_differential_call",
+            DifferentialCall(out_dtype=DTYPE_CODES[out.dtype], tokens=rows.shape[0], heads=heads, vdim=vdim, pitch=pitch,
+                             out_cols=out.shape[1], out_rows=_out_rows(out), lambda_=weight, post=post, eps=eps,
+                             input=rows.data_ptr(), ld=rows.stride(0), out=out.data_ptr(), ld_out=out.stride(0)))
 
 
 # --- routed feed-forward ----------------------------------------------------------------------

@@ -168,6 +168,45 @@ class SublayerOutput(ResidualStream):
         return delta
 
 
+class JoinedProduct:
+    """The last products of several parts that add to the stream side by side, x += sum_i W_i a_i, as ONE product: the
+    parts' operands lie beside each other in one buffer, the matrices' columns likewise, and the sum is the product's
+    own.  A part that can be joined has ``last_matrix()`` ([width, columns], which it gives up), writes its operand to
+    ``last_operand`` and leaves the product out where ``joined`` is set; ``chunk_major(step, rows)`` says whether it
+    can write a chunk-major operand in a step."""
+
+    def __init__(self, parts):
+        self.parts, matrices = list(parts), [part.last_matrix() for part in parts]
+        self.weight = torch.cat(matrices, dim=1).contiguous()
+        self.packed = packed_for_stream(self.weight) if self.weight.is_cuda else None
+        self.spans, at = {}, 0
+        for part, matrix in zip(self.parts, matrices):
+            self.spans[id(part)] = (at, matrix.shape[1])
+            at += matrix.shape[1]
+            part.joined = self
+        self.chunk = 64 // self.weight.element_size()
+        self.aligned = all(start % self.chunk == 0 for start, _ in self.spans.values())
+        self.operand = None
+
+    def begin(self, step, rows):
+        """Lays the operand out for a step of so many rows."""
+        columns = self.weight.shape[1]
+        if self.aligned and K.Chunked.wanted(rows) and all(part.chunk_major(step, rows) for part in self.parts):
+            self.operand = K.Chunked.take(step, "joined.operand", rows, columns, step.dtype)
+        else:
+            self.operand = step.buffer("joined.operand", rows, columns, step.dtype)
+
+    def share(self, part, rows):
+        start, columns = self.spans[id(part)]
+        if isinstance(self.operand, K.Chunked):
+            return self.operand.columns_from(start, columns)
+        return self.operand[:, start:start + columns]
+
+    def add_to(self, stream, step):
+        operand, self.operand = self.operand, None
+        stream.add_product(step, operand, self.weight, packed=self.packed)
+
+
 class Memory:
     """What a mixer gets of the cache for one run of its layer."""
 
@@ -191,9 +230,18 @@ class Part:
     # reads the step's host tables or allocates in its step leaves this False, and every step of a
     # model that holds such a part is issued from Python, call by call.
     only_launches_kernels = False
+    # set by a block that runs this part's last product together with another part's (JoinedProduct)
+    joined = None
 
     def __init__(self, params, tensors):
         self.params, self.tensors = params, tensors
+
+    def last_operand(self, step, key, rows, columns, chunked=False):
+        """Where the operand [rows, columns] of this part's last product goes: a buffer of its own (chunk-major if
+        ``chunked``), or its share of a joined product's operand, which decides the layout itself."""
+        if self.joined is not None:
+            return self.joined.share(self, rows)
+        return K.Chunked.take(step, key, rows, columns, step.dtype) if chunked else step.buffer(key, rows, columns, step.dtype)
 
     def kernel_modules(self, dtype):
         """Names of kernel modules (``kernels.build.register_module``) that must be built and loaded
@@ -246,6 +294,14 @@ class Mixer(Part):
     def forward(self, h, step, memory, stream):
         """Adds the mixer's contribution to ``stream`` (or returns it as a Delta)."""
         raise NotImplementedError
+
+    def carry(self, weight, activation):
+        """Optional.  A mixer whose first product leaves 32-bit sums may take another part's first projection of the same
+        rows along in it where a step is small (``kernels.library.takes_two_kinds``): ``weight`` [rows, columns of
+        h], activated by ``activation``.  It returns the one matrix of both, the other part's rows last (from then on
+        the other part's own matrix is a view of it), and its ``forward`` takes ``carried=``, the rows' place in
+        such a step; None (the default): it takes none."""
+        return None
 
     def ride_along(self, weight, bias=None):
         """Optional.  A mixer that starts with ONE product of ``h`` that leaves 32-bit sums may take another

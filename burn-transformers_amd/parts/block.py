@@ -12,11 +12,16 @@ output is multiplied, element by element, by sigmoid(gate(x)) before it is norma
 sandwich_norm: y = x + post(mixer(pre(x))); z = y + post'(feed_forward(pre'(y))), the feed-forward
 optional: a norm before AND behind every sublayer, four norms a layer with tensors of their own.
 
+parallel: y = x + mixer(norm(x)) + feed_forward(norm(x)), the feed-forward optional: ONE norm whose rows both
+sublayers read.  Where the parts allow, their first products run as one in small steps (``Mixer.carry``) and their last
+ones as one always (``JoinedProduct``), so that the sublayers' sum costs no kernel of its own.
+
 transform: x = t(x), one part of role "transform" and nothing else: what stands between two runs of
 layers (it keeps nothing in the cache; its schedule entry names no cache entry).
 """
 
-from .base import Block, SublayerOutput, Transform, offers_chunked
+from ..kernels import library as K
+from .base import Block, JoinedProduct, SublayerOutput, Transform, offers_chunked
 from .registry import register
 
 # Most rows of a step whose first norm is folded too.  Measured at GPT-2 XL sizes, ms a decode step
@@ -168,6 +173,51 @@ class SandwichNormBlock(Block):
             h = _apply(parts["ff_norm"], stream, step, ff.takes_deferred_norm)
             delta = ff.forward(h, step, output)
             stream.defer_output(parts["ff_post"], step, delta if delta is not None else output.take())
+
+
+@register("block", "parallel")
+class ParallelBlock(Block):
+    """Both sublayers read one norm of the stream and add to the stream side by side."""
+    ROLES = {"norm": "norm", "mixer": "mixer", "ff": "feed_forward"}
+    OPTIONAL = ("ff",)
+    only_launches_kernels = True
+
+    def __init__(self, parts, params=None):
+        super().__init__(parts, params)
+        mixer, ff = parts["mixer"], parts.get("ff")
+        self.output, self.carries = None, False
+        if ff is None:
+            return
+        if getattr(ff, "can_ride", False):
+            matrix = mixer.carry(ff.up_weight, ff.activation)
+            if matrix is not None:
+                ff.ride(matrix[matrix.shape[0] - ff.up_weight.shape[0]:])
+                self.carries = True
+        if all(hasattr(part, "last_matrix") for part in (mixer, ff)):
+            self.output = JoinedProduct([mixer, ff])
+
+    def forward(self, stream, step, memory):
+        parts = self.parts
+        mixer, ff, norm = parts["mixer"], parts.get("ff"), parts["norm"]
+        rows = stream.x.shape[0]
+        if ff is None:
+            delta = mixer.forward(_apply(norm, stream, step, mixer.takes_deferred_norm), step, memory, stream)
+            if delta is not None:
+                stream.add(delta)
+            return
+        # both parts hand the rows to products only: a small step's rows may be chunk-major
+        h = _apply(norm, stream, step, self.carries or (mixer.takes_deferred_norm and ff.takes_deferred_norm))
+        if self.output is not None:
+            self.output.begin(step, rows)
+        extra = {}
+        if self.carries and K.takes_two_kinds(h):
+            extra = {"carried": ff.hidden_rows(step, rows)}
+        for delta in (mixer.forward(h, step, memory, stream, **extra),
+                      ff.forward(h, step, stream, **({"hidden": extra["carried"]} if extra else {}))):
+            if delta is not None:
+                stream.add(delta)
+        if self.output is not None:
+            self.output.add_to(stream, step)
 
 
 @register("block", "transform")

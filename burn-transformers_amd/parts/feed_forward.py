@@ -1,7 +1,8 @@
 """Dense feed-forward: down(act(up(x)))  (src/feed_forward.rs:111-114).
 
 Parameters: width, inner, activation ("gelu_tanh": 0.5x(1+tanh(sqrt(2/pi)(x+0.044715x^3))),
-"gelu_erf": x(1+erf(x/sqrt 2))/2; src/feed_forward.rs:351-387).  The activation runs in 32-bit
+"gelu_erf": x(1+erf(x/sqrt 2))/2; src/feed_forward.rs:351-387; "squared_relu": max(x, 0)^2), padded_rows (the
+rows come with zero columns up to what a product's operand takes, as rms_norm leaves them: any width runs).  The activation runs in 32-bit
 inside the up projection's epilogue (src/feed_forward.rs:397-406 widens half inputs too); the
 down projection adds into the residual stream.
 
@@ -47,11 +48,13 @@ class DenseFeedForward(FeedForward):
             raise ValueError(f"feed-forward: projections are {tuple(self.up_weight.shape)} and "
                              f"{tuple(self.down_weight.shape)}, expected {(self.inner, self.width)} and "
                              f"{(self.width, self.inner)}")
+        if params.get("padded_rows"):
+            self.up_weight = pad_columns(self.up_weight, operand_columns(self.width, self.up_weight.dtype))
         self.padded = (self.inner + 7) // 8 * 8
         extra = self.padded - self.inner
         if extra:
             up, down = self.up_weight, self.down_weight
-            self.up_weight = torch.cat([up, up.new_zeros(extra, self.width)]).contiguous()
+            self.up_weight = torch.cat([up, up.new_zeros(extra, up.shape[1])]).contiguous()
             self.down_weight = torch.cat([down, down.new_zeros(self.width, extra)], dim=1).contiguous()
             if self.up_bias is not None:
                 self.up_bias = torch.cat([self.up_bias, self.up_bias.new_zeros(extra)]).contiguous()
@@ -60,21 +63,42 @@ class DenseFeedForward(FeedForward):
         self.up_packed = K.PackedWeight(self.up_weight) if self.up_weight.is_cuda else None
         self.down_packed = packed_for_stream(self.down_weight) if self.down_weight.is_cuda else None
 
-    def forward(self, h, step, stream):
+        # whether the up projection may run inside another part's first product (Mixer.carry)
+        self.can_ride = self.activation in K.ACTIVATIONS and self.up_bias is None
+
+    def ride(self, up_weight):
+        """The up projection as a view of the matrix that small steps multiply by in the other part's product."""
+        self.up_weight, self.up_packed = up_weight, None
+
+    def last_matrix(self):
+        if self.down_bias is not None:
+            raise ValueError("feed-forward: a product with a bias of its own is not joined with another")
+        matrix, self.down_weight, self.down_packed = self.down_weight, None, None
+        return matrix
+
+    def chunk_major(self, step, rows):
+        return self.activation != "poly_norm"
+
+    def hidden_rows(self, step, tokens):
+        return self.last_operand(step, "feed_forward.hidden", tokens, self.padded,
+                                 K.Chunked.wanted(tokens) and (step.dtype_is_bf16 or self.padded % 4 == 0))   # read by the next product only
+
+    def forward(self, h, step, stream, hidden=None):
+        """``hidden``: the activated rows, where another part's product made them already."""
         tokens = h.shape[0]
         if self.activation == "poly_norm":
             z = step.buffer("feed_forward.sums", tokens, self.padded, "float32")
-            hidden = step.buffer("feed_forward.hidden", tokens, self.padded, step.dtype)
+            hidden = self.last_operand(step, "feed_forward.hidden", tokens, self.padded)
             K.gemm(h, self.up_weight, K.epilogue_f32(z, self.up_bias), packed=self.up_packed)
             K.poly_norm(z, self.inner, self.coefficients, self.eps, hidden)
-            stream.add_product(step, hidden, self.down_weight, self.down_bias, packed=self.down_packed)
+            if self.joined is None:
+                stream.add_product(step, hidden, self.down_weight, self.down_bias, packed=self.down_packed)
             return
-        if K.Chunked.wanted(tokens) and (step.dtype_is_bf16 or self.padded % 4 == 0):
-            hidden = K.Chunked.take(step, "feed_forward.hidden", tokens, self.padded, step.dtype)   # read by the next product only
-        else:
-            hidden = step.buffer("feed_forward.hidden", tokens, self.padded, step.dtype)
-        K.gemm(h, self.up_weight, K.epilogue_act(hidden, self.activation, self.up_bias), packed=self.up_packed)
-        stream.add_product(step, hidden, self.down_weight, self.down_bias, packed=self.down_packed)
+        if hidden is None:
+            hidden = self.hidden_rows(step, tokens)
+            K.gemm(h, self.up_weight, K.epilogue_act(hidden, self.activation, self.up_bias), packed=self.up_packed)
+        if self.joined is None:
+            stream.add_product(step, hidden, self.down_weight, self.down_bias, packed=self.down_packed)
 
 
 @register("feed_forward", "gated_dense")

@@ -5,10 +5,12 @@ with ``keep_origin``), W ``weight`` [width, 2 * width] (the stream's columns fir
 ``row`` of ``shift`` [rows, width] (a model that runs a stretch of layers several times enters every
 pass through such a part, each pass with a row of its own).  The two streams are laid side by side
 in the products' type, one product leaves the new stream in 32-bit, the shift added.
+
+add_origin: x <- x + x0.  The sum is left pending for the next norm, which adds it while it reads the stream.
 """
 
 from ..kernels import library as K
-from .base import Transform, operand_columns, pad_columns
+from .base import Delta, Transform, operand_columns, pad_columns
 from .registry import register
 
 
@@ -43,3 +45,13 @@ class JoinedProjection(Transform):
         K.join_rows(stream.x, stream.origin, joined)
         stream.cast = None
         K.gemm(joined, self.weight, K.epilogue_f32(stream.x, self.shift), packed=self.packed)
+
+
+@register("transform", "add_origin")
+class AddOrigin(Transform):
+    only_launches_kernels = True
+
+    def forward(self, stream, step):
+        if stream.origin is None:
+            raise ValueError("add_origin: the embedding does not keep its output (keep_origin)")
+        stream.add(Delta(stream.origin.unsqueeze(0)))

@@ -21,13 +21,21 @@ passes a short causal convolution over its sequence's tokens, tensors ``q_conv``
 [channels, taps], the last tap meeting the current token, no bias, no activation, before norms and rotation;
 the projections' last taps - 1 outputs are then a state of the sequence beside its keys and values).  Optional
 tensors ``q_bias`` / ``k_bias`` / ``v_bias``: added in the projection.  Optional tensor ``sink`` [heads]: a learned logit per head that stands in the softmax's
-denominator beside the keys', with no key and no value.  Tensors: q_weight [heads * dim, width], k_weight [kv_heads * dim, width],
+denominator beside the keys', with no key and no value.  softcap (default 0: none; scores become softcap *
+tanh(score / softcap) before the softmax); weights ("softmax", the default; "sigmoid": a visible key weighs
+sigmoid(score + b), b the tensor ``score_bias`` [heads], and nothing is normalised over the keys); values
+("projected", the default; "keys": the projected keys before norm and rotation, vdim = dim and no ``v_weight``);
+temperature (None, or coef / every: queries times 1 + coef * ln(floor((position + 1) / every) + 1)); gate (None;
+"head": a head's output times sigmoid of one row of the tensor ``gate_weight`` [heads, width] on the mixer's input;
+"channel": every channel times its own, ``gate_weight`` [heads * vdim, width]).  Tensors: q_weight [heads * dim, width], k_weight [kv_heads * dim, width],
 v_weight [kv_heads * vdim, width], out_weight [width, heads * vdim], no biases.
 
-One step: ONE product with the three projections laid one behind the other leaves 32-bit sums; a
+One step: ONE product with the projections (the gate's too) laid one behind the other leaves 32-bit sums; a
 kernel normalises and turns the heads, writes the queries to a buffer and the keys (turned) and
 values straight into the cache at each token's position; the framework's attention kernels read the
-cache; the output projection adds to the stream.  The cache keeps heads of one size, max(dim, vdim)
+cache (and gate what they store); the output projection adds to the stream.  Beside another part that reads the
+same rows the first product also carries that part's first projection in small steps (``carry``), and the output
+projection may be joined with its last (``last_matrix``).  The cache keeps heads of one size, max(dim, vdim)
 rounded up to what the kernels take, with zeros behind a head's own channels; the output
 projection's columns are spread the same way, so the zeros meet zeros.
 """
@@ -39,7 +47,7 @@ import torch
 from ..cache.storage import StateSpec
 from ..kernels import library as K
 from .attention import CausalSelfAttention
-from .base import Mixer, operand_columns, packed_for_stream, pad_columns
+from .base import Mixer, operand_columns, packed_for_stream, pad_columns, pad_rows
 from .registry import register
 
 
@@ -74,6 +82,7 @@ def rotary_amplitude(scaling=None):
 class RotaryAttention(CausalSelfAttention):
     takes_deferred_norm = False          # (its first product leaves 32-bit sums; the rows come normalised)
     only_launches_kernels = True
+    maps = 1                             # score maps a head: how many queries and key parts it has (see DifferentialAttention)
 
     def __init__(self, params, tensors):
         Mixer.__init__(self, params, tensors)
@@ -87,17 +96,38 @@ class RotaryAttention(CausalSelfAttention):
             raise ValueError(f"rotary attention: {self.heads} query heads cannot share {self.kv_heads} key/value heads")
         if self.rot_dims % 2 != 0 or self.rot_dims > self.dim:
             raise ValueError(f"rotary attention: {self.rot_dims} turned channels must be even and at most the head size {self.dim}")
-        shapes = {"q_weight": (self.heads * self.dim, self.width), "k_weight": (self.kv_heads * self.dim, self.width),
-                  "v_weight": (self.kv_heads * self.vdim, self.width), "out_weight": (self.width, self.heads * self.vdim)}
+        # columns of the queries, the keys and the values in the first product
+        n_qk = (self.heads * self.maps * self.dim, self.kv_heads * self.maps * self.dim)
+        self.values_from_keys = {"projected": False, "keys": True}[p.get("values", "projected")]
+        n_v = 0 if self.values_from_keys else self.kv_heads * self.vdim
+        if self.values_from_keys and (self.vdim != self.dim or self.maps != 1):
+            raise ValueError(f"rotary attention: values that are the keys have the keys' size {self.dim}, not {self.vdim}")
+        shapes = {"q_weight": (n_qk[0], self.width), "k_weight": (n_qk[1], self.width),
+                  "out_weight": (self.width, self.heads * self.vdim)}
+        if not self.values_from_keys:
+            shapes["v_weight"] = (n_v, self.width)
+        self.softcap = float(p.get("softcap") or 0.0)
+        self.sigmoid = {"softmax": False, "sigmoid": True}[p.get("weights", "softmax")]
+        if self.softcap < 0.0 or (self.sigmoid and self.softcap):
+            raise ValueError("rotary attention: a cap on the scores is positive and goes with the softmax")
+        if self.sigmoid:
+            shapes["score_bias"] = (self.heads,)
+        temperature = p.get("temperature")
+        self.temperature = (float(temperature["coef"]), int(temperature["every"])) if temperature else None
+        self.gate_kind = p.get("gate")
+        self.gate_cols = {None: 0, "head": self.heads, "channel": self.heads * self.vdim}[self.gate_kind]
+        if self.gate_cols:
+            shapes["gate_weight"] = (self.gate_cols, self.width)
         self.neighbours = {"halves": False, "neighbours": True}[p.get("rot_pairing", "halves")]
         self.whole_norm = {"head": False, "whole": True}[p.get("norm_span", "head")]
         if p.get("head_norm", True):
-            shapes.update(q_norm=(self.heads * self.dim,), k_norm=(self.kv_heads * self.dim,)) if self.whole_norm else \
+            shapes.update(q_norm=(n_qk[0],), k_norm=(n_qk[1],)) if self.whole_norm else \
                 shapes.update(q_norm=(self.dim,), k_norm=(self.dim,))
         if "sink" in tensors:
             shapes["sink"] = (self.heads,)
         self.taps = int(p.get("taps") or 0)
-        for name, rows in (("q", self.heads * self.dim), ("k", self.kv_heads * self.dim), ("v", self.kv_heads * self.vdim)):
+        projections = [(name, rows) for name, rows in (("q", n_qk[0]), ("k", n_qk[1]), ("v", n_v)) if rows]
+        for name, rows in projections:
             if name + "_bias" in tensors:
                 shapes[name + "_bias"] = (rows,)
             if self.taps:
@@ -107,24 +137,23 @@ class RotaryAttention(CausalSelfAttention):
                 raise ValueError(f"rotary attention: {role} is {tuple(tensors[role].shape)}, expected {shape}")
         self.q_norm, self.k_norm = tensors.get("q_norm"), tensors.get("k_norm")
         self.sink = tensors["sink"].float().contiguous() if "sink" in tensors else None
+        self.score_bias = tensors["score_bias"].float().contiguous() if self.sigmoid else None
         dtype = tensors["q_weight"].dtype
         bf16 = dtype == torch.bfloat16
         # the cached head: the larger of the two head sizes, in the steps of 16 the MFMA kernels take
-        self.head_dim = (max(self.dim, self.vdim) + 15) // 16 * 16
-        if self.head_dim > 256:
+        self.head_dim = (max(self.maps * self.dim, self.vdim) + 15) // 16 * 16
+        if max(self.dim, self.vdim) > 256:
             raise ValueError(f"rotary attention: heads of {max(self.dim, self.vdim)} are beyond 256, the most any kernel here takes")
         # the MFMA kernels take heads of up to 128 in bfloat16; larger ones run on the plain attention kernel
         self.plain_only = bf16 and self.head_dim > 128
-        self.plain_decode = bf16 and self.heads // self.kv_heads > 16
-        self.n_q, self.n_kv = self.heads * self.head_dim, self.kv_heads * self.head_dim
-        self.fused_cols = (self.heads + self.kv_heads) * self.dim + self.kv_heads * self.vdim
-        self.qkv_weight = pad_columns(torch.cat([tensors["q_weight"], tensors["k_weight"], tensors["v_weight"]]),
-                                      operand_columns(self.width, dtype))
-        # the output projection reads heads of head_dim: its columns are spread, zeros between them
-        out = tensors["out_weight"]
-        spread = out.new_zeros(self.width, self.heads, self.head_dim)
-        spread[:, :, :self.vdim] = out.view(self.width, self.heads, self.vdim)
-        self.out_weight = spread.view(self.width, self.n_q).contiguous()
+        self.q_heads = self.heads * self.maps                   # queries the attention kernels see
+        self.plain_decode = bf16 and self.q_heads // self.kv_heads > 16
+        self.n_q, self.n_kv = self.q_heads * self.head_dim, self.kv_heads * self.head_dim
+        self.fused_cols = n_qk[0] + n_qk[1] + n_v               # what a convolution passes over
+        self.first_cols = self.fused_cols + self.gate_cols
+        first = [tensors[name + "_weight"] for name, _ in projections] + ([tensors["gate_weight"]] if self.gate_cols else [])
+        self.qkv_weight = pad_columns(torch.cat(first), operand_columns(self.width, dtype))
+        self.out_weight = self.output_matrix(tensors["out_weight"])
         self.out_bias = None
         device = self.qkv_weight.device
         self.inv_freq = rotary_frequencies(self.rot_dims, p["rot_base"], p.get("rot_scaling")).to(torch.float32).to(device) \
@@ -134,30 +163,69 @@ class RotaryAttention(CausalSelfAttention):
         if any(name + "_bias" in tensors for name in "qkv"):
             self.qkv_bias = torch.cat([tensors[name + "_bias"].float() if name + "_bias" in tensors
                                        else torch.zeros(rows, dtype=torch.float32, device=device)
-                                       for name, rows in (("q", self.heads * self.dim), ("k", self.kv_heads * self.dim),
-                                                          ("v", self.kv_heads * self.vdim))]).contiguous()
+                                       for name, rows in projections + [("gate", self.gate_cols)]]).contiguous()
         self.conv_weight, self.conv_state = None, 0
         if self.taps:
-            self.conv_weight = torch.cat([tensors["q_conv"], tensors["k_conv"], tensors["v_conv"]]).float().contiguous()
+            self.conv_weight = torch.cat([tensors[name + "_conv"] for name, _ in projections]).float().contiguous()
             self.conv_state = (self.taps - 1) * self.fused_cols
             self.no_state = torch.zeros(1, 1, dtype=torch.float32, device=device)       # what one tap keeps: nothing
         on_gpu = self.qkv_weight.is_cuda
         self.qkv_packed = K.PackedWeight(self.qkv_weight) if on_gpu else None
         self.out_packed = packed_for_stream(self.out_weight) if on_gpu else None
+        self.first_matrix, self.first_packed = None, None       # with another part's rows behind its own: see ``carry``
+
+    def output_matrix(self, out):
+        """The output projection as it reads heads of head_dim: its columns spread, zeros between them."""
+        spread = out.new_zeros(self.width, self.heads, self.head_dim)
+        spread[:, :, :self.vdim] = out.view(self.width, self.heads, self.vdim)
+        return spread.view(self.width, self.heads * self.head_dim).contiguous()
+
+    def wide_output(self, dtype):
+        """Whether the attention kernels store 32-bit rows in a model of this type that keeps bfloat16 ones."""
+        return False
 
     def kernel_modules(self, dtype):
-        return ("rotary",) + (("state_space",) if self.taps else ()) + tuple(super().kernel_modules(dtype))
+        modules = tuple(super().kernel_modules(dtype))
+        if self.softcap or self.sigmoid or self.gate_cols or self.wide_output(dtype):
+            variant = "_sigmoid" if self.sigmoid else "_capped" if self.softcap else "_softmax"
+            modules = tuple(name + variant for name in modules)
+        return ("rotary",) + (("state_space",) if self.taps else ()) + modules
+
+    def carry(self, weight, activation):
+        if self.qkv_bias is not None or weight.shape[1] != self.qkv_weight.shape[1]:
+            return None
+        own = (self.first_cols + 3) // 4 * 4                    # (the product's epilogue works on four columns at a time)
+        self.first_matrix = torch.cat([pad_rows(self.qkv_weight, own), weight]).contiguous()
+        self.qkv_weight, self.first_cols, self.carried_activation = self.first_matrix[:own], own, activation
+        if self.first_matrix.is_cuda:                           # small steps run the product of both
+            self.qkv_packed, self.first_packed = None, K.PackedWeight(self.first_matrix)
+        return self.first_matrix
+
+    def last_matrix(self):
+        matrix, self.out_weight, self.out_packed = self.out_weight, None, None
+        return matrix
+
+    def chunk_major(self, step, rows):
+        return step.decode and step.dtype_is_bf16 and not self.runs_plain(step)
+
+    def runs_plain(self, step):
+        """(the bfloat16 decode kernel takes up to 16 query heads on a cached head; beyond, the plain kernel)"""
+        return self.plain_only or (self.plain_decode and step.decode)
 
     def state_spec(self):
         return StateSpec((self.conv_state,), "float32") if self.conv_state else None
 
-    def forward(self, h, step, memory, stream):
+    def forward(self, h, step, memory, stream, carried=None):
         tokens = h.shape[0]
         if not memory.writes:
             raise ValueError("rotary attention: every run keeps a cache entry of its own")
         kv = memory.kv()
-        fused = step.buffer("rotary.fused", tokens, self.fused_cols, "float32")
-        K.gemm(h, self.qkv_weight, K.epilogue_f32(fused, self.qkv_bias), packed=self.qkv_packed)
+        first = fused = step.buffer("rotary.fused", tokens, self.first_cols, "float32")
+        if carried is not None:
+            K.gemm(h, self.first_matrix, K.epilogue_f32_act(fused, self.first_cols, carried, self.carried_activation),
+                   packed=self.first_packed)
+        else:
+            K.gemm(h, self.qkv_weight, K.epilogue_f32(fused, self.qkv_bias), packed=self.qkv_packed)
         if self.taps:
             mixed_in_time = step.buffer("rotary.conv", tokens, self.fused_cols, "float32")
             K.causal_conv(fused, self.conv_weight, None, mixed_in_time, memory.state() if self.conv_state else self.no_state,
@@ -166,18 +234,28 @@ class RotaryAttention(CausalSelfAttention):
         q = step.buffer("attention.q", tokens, self.n_q, step.dtype)
         K.head_rotary(fused, self.heads, self.kv_heads, self.dim, self.vdim, self.rot_dims, self.inv_freq,
                       self.q_norm, self.k_norm, self.eps, q, step.tok_seq, step.tok_pos, kv, step.dtype,
-                      neighbours=self.neighbours, whole_norm=self.whole_norm, amplitude=self.amplitude)
-        plain = self.plain_only or (self.plain_decode and step.decode)
-        if step.decode and step.dtype_is_bf16 and K.Chunked.wanted(tokens) and not plain:
-            mixed = K.Chunked.take(step, "attention.mixed", tokens, self.n_q, step.dtype)
-        else:
-            mixed = step.buffer("attention.mixed", tokens, self.n_q, step.dtype)
-        partial, runs = None, 1 if plain else self.decode_runs(step, h.device)
+                      neighbours=self.neighbours, whole_norm=self.whole_norm, amplitude=self.amplitude, maps=self.maps,
+                      values_from_keys=self.values_from_keys, temperature=self.temperature)
+        gate = first[:, self.fused_cols:] if self.gate_cols else None
+        mixed = self.attend(q, gate, kv, step)
+        if self.joined is None:
+            stream.add_product(step, mixed, self.out_weight, None, packed=self.out_packed)
+
+    def attend(self, q, gate, kv, step):
+        """The operand of the output projection."""
+        tokens = q.shape[0]
+        mixed = self.last_operand(step, "attention.mixed", tokens, self.n_q,
+                                  K.Chunked.wanted(tokens) and self.chunk_major(step, tokens))
+        self.run_attention(q, mixed, gate, kv, step)
+        return mixed
+
+    def run_attention(self, q, out, gate, kv, step):
+        plain, partial = self.runs_plain(step), None
+        runs = 1 if plain else self.decode_runs(step, q.device)
         if runs > 1:
-            partial = step.buffer("attention.partial", step.n_seqs * self.heads * runs, self.head_dim + 2, "float32")
-        args = K.attention_args(q, mixed, kv, step.tok_seq, step.tok_pos, step.seq_off, step.seq_start,
-                                self.heads, step.n_seqs, step.max_count, self.scale, self.window, partial,
-                                chunk=self.chunk, sink=self.sink)
-        # (the bfloat16 decode kernel takes up to 16 query heads on a cached head; beyond, the plain kernel)
+            partial = step.buffer("attention.partial", step.n_seqs * self.q_heads * runs, self.head_dim + 2, "float32")
+        args = K.attention_args(q, out, kv, step.tok_seq, step.tok_pos, step.seq_off, step.seq_start,
+                                self.q_heads, step.n_seqs, step.max_count, self.scale, self.window, partial,
+                                chunk=self.chunk, sink=self.sink, softcap=self.softcap, sigmoid=self.sigmoid,
+                                score_bias=self.score_bias, gate=gate, gate_dim=self.vdim if self.gate_kind == "channel" else 0)
         K.attention(args, step.dtype, step.decode, impl="plain" if plain else "auto")
-        stream.add_product(step, mixed, self.out_weight, None, packed=self.out_packed)
