@@ -69,8 +69,10 @@ __device__ __forceinline__ float bt_sigmoid(float z) { return 1.0f / (1.0f + exp
 // The gate's factor on channel `channel` of head `head` of token `tok`.
 __device__ __forceinline__ float bt_output_gate(const AttnArgs& a, int64_t tok, int head, int channel) {
   if (!a.gate) return 1.f;
-  const int column = a.gate_span == 1 ? head * a.gate_dim + (channel < a.gate_dim ? channel : 0) : head;
-  return bt_sigmoid(a.gate[tok * a.ld_gate + column]);
+  const bool none = a.gate_span == 1 && channel >= a.gate_dim;
+  const int column = a.gate_span == 1 ? head * a.gate_dim + (none ? 0 : channel) : head;
+  const float factor = bt_sigmoid(a.gate[tok * a.ld_gate + column]);
+  return none ? 1.f : factor;
 }
 
 // What forms and output stages need of their arguments; nullptr, or what is wrong.

@@ -106,6 +106,8 @@ class ResidualStream:
         rows, width = a.shape[0], weight.shape[0]
         splits = 1 if self.in_place else stream_product_splits(step, a, weight)
         if splits > 1:
+            if self.pending is not None:       # (a part beside this one: its sums may lie in the buffer this product writes)
+                self.flush()
             partials = step.partial_sums("stream.partials", splits, rows, width)
             K.gemm(a, weight, K.epilogue_f32(partials), splits=splits, packed=packed)
             self.add(Delta(partials, bias))

@@ -118,7 +118,8 @@ def sigmoid_attention(h, w, prefix, sizes, eps):
     q = (unit_rms(h @ w[prefix + "q"].T, eps) * w[prefix + "q.norm"]).view(T, H, D)
     k = (unit_rms(k_rows, eps) * w[prefix + "k.norm"]).view(T, G, D)
     v = k_rows.view(T, G, D)
-    q = q * temperature(positions, sizes["q_temp"]["coef"], sizes["q_temp"]["every"])[:, None, None]
+    if sizes.get("q_temp"):
+        q = q * temperature(positions, sizes["q_temp"]["coef"], sizes["q_temp"]["every"])[:, None, None]
     out = torch.zeros(T, H, D, dtype=F64)
     for head in range(H):
         shared = head // (H // G)
