@@ -1,7 +1,7 @@
 """Throughput of GPT-2 generation on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--layers 48] [--dtype bf16]
-                    [--repetitions 10] [--workload xl|small|medium|sweep|salopel|kodatar|rotutar|gavasun] [--model xl|medium|small]
+                    [--repetitions 10] [--workload xl|small|medium|sweep|salopel|kodatar|rotutar|gavasun|loselix] [--model xl|medium|small]
                     [--kernel-batches 1,64] [--sweep-part all|decode|prompts] [--no-points] [--no-kernels] [--no-own]
 
 The default workload (``xl``) has the layer sizes of GPT-2 XL with random weights: a batch of 8
@@ -55,6 +55,9 @@ family, at equal width, layers and vocabulary.
 ``--workload gavasun`` runs the fifth family, Gavasun (chunk attention behind short convolutions, latent attention
 with a shared turned key part in a window, a delta rule with one decay a head, ungated experts), beside Rotutar,
 the library's closest family, at equal width, layers and vocabulary.
+``--workload loselix`` runs the sixth family, Loselix (differential attention with capped scores, attention with a gate per
+head, sigmoid attention on its own keys, mixer and feed-forward side by side, a stretch of layers that runs twice), beside
+GPT-2 (whole contexts, dense feed-forwards) at equal width, runs of layers, feed-forward and vocabulary.
 """
 
 import argparse
@@ -197,7 +200,8 @@ def _class_of(name, call):
         return f"{short} {call.M}x{call.N}x{call.K}", weights + rows, 2.0 * call.M * call.N * call.K
     if short.startswith("attention"):
         args = call.args                                           # (bytes and flops are filled in by the caller, who knows the contexts)
-        return f"{short} {args.n_tokens}tok {args.q_heads}x{args.kv.head_dim} on {args.kv.kv_heads}", None, None
+        form = ("", " capped", " sigmoid")[args.form] + (" gated" if args.gate else "")
+        return f"{short} {args.n_tokens}tok {args.q_heads}x{args.kv.head_dim} on {args.kv.kv_heads}{form}", None, None
     if short == "add_norm":
         return f"add_norm {call.n_rows}x{call.width}", (call.n_delta + 2) * call.n_rows * call.width * 4, 0.0
     if short == "embed":
@@ -207,6 +211,8 @@ def _class_of(name, call):
     if short == "output_norm":
         return f"output_norm {call.tokens}x{call.width}", (call.n_delta + 2) * call.tokens * call.width * 4 + \
             (call.tokens * call.cast_cols * 2 if call.cast else 0), 0.0
+    if short == "activate":
+        return f"activate {call.tokens}x{call.columns}", call.tokens * call.columns * 2 * (4 if call.dtype == 0 else 2), 0.0
     if short == "poly_norm":
         return f"poly_norm {call.tokens}x{call.columns}", call.tokens * call.columns * 6, 0.0
     if short == "latent_norm":
@@ -234,8 +240,12 @@ def _class_of(name, call):
             call.n_seqs * inner * call.state * 8 + call.tokens * (inner * 8 + call.groups * call.state * 8), \
             6.0 * call.tokens * inner * call.state
     if short == "head_rotary":
-        columns = (call.heads + call.kv_heads) * call.dim + call.kv_heads * call.vdim
-        return f"head_rotary {call.tokens}tok", call.tokens * columns * 6, 0.0
+        columns = (call.heads + call.kv_heads) * call.maps * call.dim + call.kv_heads * call.vdim
+        kind = " two maps" if call.maps == 2 else " values from keys" if call.values_from_keys else ""
+        return f"head_rotary {call.tokens}tok{kind}", call.tokens * columns * 6, 0.0
+    if short == "differential":
+        return f"differential {call.tokens}x{call.heads * call.vdim}", \
+            call.tokens * call.heads * (8 * call.pitch + call.vdim * (4 if call.out_dtype == 0 else 2)), 0.0
     if short == "route":
         return f"route {call.tokens}x{call.experts}", call.experts * call.width * 4 + call.tokens * call.width * 2, \
             2.0 * call.tokens * call.experts * call.width
@@ -265,7 +275,8 @@ def _class_of(name, call):
 
 def kernel_classes(engine, entries, attention_bytes, attention_flops, peak_flops, replays=20):
     """Runs one step of ``entries`` to get its launch list, then replays each class of calls alone
-    from a HIP graph.  Returns {label: {"n": calls a step, "us": per call, "hbm": fraction of the
+    from a HIP graph (``attention_bytes`` and ``attention_flops``: numbers, or functions of an attention call's
+    arguments where a model's attention layers differ).  Returns {label: {"n": calls a step, "us": per call, "hbm": fraction of the
     HBM roofline, "mfma": fraction of the MFMA peak}}."""
     import torch
     from burn_transformers_amd.kernels import library as K
@@ -290,7 +301,7 @@ def kernel_classes(engine, entries, attention_bytes, attention_flops, peak_flops
     for lib, name, call in program.calls:
         label, nbytes, flops = _class_of(name, call)
         if nbytes is None:
-            nbytes, flops = attention_bytes, attention_flops
+            nbytes, flops = (f(call.args) if callable(f) else f for f in (attention_bytes, attention_flops))
         classes.setdefault(label, []).append((lib, name, call, nbytes, flops))
     out = {}
     for label, calls in classes.items():
@@ -636,6 +647,34 @@ def gavasun_config(width, layers, vocab):
             "loop": None, "layers": [dict(group[i % 4]) for i in range(layers)]}
 
 
+def loselix_config(width, layers, vocab):
+    """Loselix at layer sizes that resemble a real model's: ``layers`` runs of layers, of which the first two thirds are one
+    stretch of a third run twice; groups of four (differential attention with two maps of 64 channels a head, two layers of
+    attention with a gate per head, sigmoid attention), heads of 128 on a quarter as many key/value heads, the temperature's
+    steps 512 positions apart, a feed-forward of 4 x width beside every mixer."""
+    heads = max(4, width // 128)
+    shared = {"heads": heads, "kv_heads": heads // 4, "vdim": 128}
+    pair = ("attention", {**shared, "dim": 64, "scale": 64 ** -0.5, "rot": {"dims": 64, "base": 500000.0}, "softcap": 50.0, "diff": 0.3})
+    gated = ("attention_2", {**shared, "dim": 128, "scale": 128 ** -0.5, "rot": {"dims": 64, "base": 500000.0}})
+    sigmoid = ("attention_3", {**shared, "dim": 128, "scale": 128 ** -0.5, "q_temp": {"coef": 0.1, "every": 512}})
+    group = [pair, gated, gated, sigmoid]
+    third = max(1, layers // 3)
+    return {"architecture": "Loselix", "vocab": vocab, "width": width, "norm": {"eps": 1e-5},
+            "loop": {"start": 0, "stop": third, "times": 2},
+            "layers": [{"type": group[i % 4][0], "mixer": dict(group[i % 4][1]), "mlp": {"kind": "dense", "ff": 4 * width}}
+                       for i in range(layers - third)]}
+
+
+def run_loselix(args):
+    """Loselix beside GPT-2 at equal width, runs of layers, feed-forward and vocabulary."""
+    def values_and_columns(attention):
+        # cached values a token (a differential head's two maps share one cached head) and channels its queries meet:
+        # a map's queries meet half of the cached key and all of the value
+        heads, size = attention.q_heads, attention.kv.head_dim
+        return 2 * size * attention.kv.kv_heads, heads * size * (0.75 if attention.form == 1 else 1.0)
+    run_beside_gpt2(args, "loselix", loselix_config, None, of_call=values_and_columns)
+
+
 def run_gavasun(args):
     """Gavasun beside the library's closest family, Rotutar (a delta rule with a matrix state, rotary attention on
     grouped heads, routed experts), at equal width, layers and vocabulary."""
@@ -664,9 +703,10 @@ def run_kodatar(args):
                     lambda width: (2 * 128 * (max(4, width // 128) // 4), 128 * max(4, width // 128)))
 
 
-def run_beside_gpt2(args, family, config_of, attention_sizes, other=None):
+def run_beside_gpt2(args, family, config_of, attention_sizes, other=None, of_call=None):
     """``attention_sizes(width)``: (cached values a token and layer, columns of a token's queries), for
-    the attention kernels' bytes and flops.  ``other``: (family, its configuration, its attention sizes) of the
+    the attention kernels' bytes and flops; ``of_call``: the same as a function of an attention call's arguments, for a
+    family whose attention layers differ.  ``other``: (family, its configuration, its attention sizes) of the
     model that runs beside, GPT-2 without."""
     import torch
 
@@ -682,7 +722,8 @@ def run_beside_gpt2(args, family, config_of, attention_sizes, other=None):
             if name == family or other:
                 config = (config_of if name == family else other[1])(width, layers, vocab)
                 model = build_salopel(config, dtype)
-                cached, columns = (attention_sizes if name == family else other[2])(width)
+                sizes = attention_sizes if name == family else other[2]
+                cached, columns = sizes(width) if sizes else (None, None)
             else:
                 config = dict(XL, n_layer=layers, n_embd=width, n_head=width // 64, n_inner=4 * width, vocab_size=vocab,
                               n_positions=2048)
@@ -702,18 +743,19 @@ def run_beside_gpt2(args, family, config_of, attention_sizes, other=None):
                 engine.step(list(zip(slots, prompts)))
                 if name == "gpt2":
                     cached, columns = 2 * width, width
-                kv = batch * context * cached * ELEMENT_BYTES[dtype]
-                flops = 4.0 * batch * context * columns
+                element, per_call = ELEMENT_BYTES[dtype], name == family and of_call
+                kv = (lambda a: batch * context * of_call(a)[0] * element) if per_call else batch * context * cached * element
+                flops = (lambda a: 4.0 * batch * context * of_call(a)[1]) if per_call else 4.0 * batch * context * columns
                 result["decode_kernels"] = kernel_classes(engine, [(slot, [5]) for slot in slots], kv, flops, PEAK_FLOPS[dtype])
                 for slot in slots:
                     engine.close(slot)
                 prompts = synthetic_prompts(PREFILL_SEQS, PREFILL_LEN, vocab, seed=8)
                 slots = [engine.open() for _ in prompts]
                 tokens = PREFILL_SEQS * PREFILL_LEN
-                per_token = columns
-                result["prefill_kernels"] = kernel_classes(engine, list(zip(slots, prompts)), 4 * tokens * per_token * ELEMENT_BYTES[dtype],
-                                                           PREFILL_SEQS * 2.0 * per_token * PREFILL_LEN * (PREFILL_LEN + 1),
-                                                           PEAK_FLOPS[dtype], replays=10)
+                kv = (lambda a: 4 * tokens * of_call(a)[1] * element) if per_call else 4 * tokens * columns * element
+                pairs = PREFILL_SEQS * 2.0 * PREFILL_LEN * (PREFILL_LEN + 1)
+                flops = (lambda a: pairs * of_call(a)[1]) if per_call else pairs * columns
+                result["prefill_kernels"] = kernel_classes(engine, list(zip(slots, prompts)), kv, flops, PEAK_FLOPS[dtype], replays=10)
                 for slot in slots:
                     engine.close(slot)
             line[name] = result
@@ -734,7 +776,7 @@ def main():
     parser.add_argument("--kernel-batches", default="", help="further batch sizes whose decode kernel classes are timed, e.g. 1,64")
     parser.add_argument("--dtype", choices=["bf16", "fp32"], default=None)
     parser.add_argument("--repetitions", type=int, default=10, help="measured repetitions, each on fresh sequences")
-    parser.add_argument("--workload", choices=["xl", "small", "medium", "sweep", "salopel", "kodatar", "rotutar", "gavasun"], default="xl")
+    parser.add_argument("--workload", choices=["xl", "small", "medium", "sweep", "salopel", "kodatar", "rotutar", "gavasun", "loselix"], default="xl")
     parser.add_argument("--sweep-part", choices=["all", "decode", "prompts"], default="all",
                         help="which table of --workload sweep to run")
     parser.add_argument("--no-points", action="store_true", help="skip batch 1 and 64")
@@ -747,8 +789,9 @@ def main():
     if args.repetitions < 1:
         parser.error("--repetitions must be at least 1")
     args.kernel_batches = [int(b) for b in args.kernel_batches.split(",") if b]
-    if args.workload in ("salopel", "kodatar", "rotutar", "gavasun"):
-        {"salopel": run_salopel, "kodatar": run_kodatar, "rotutar": run_rotutar, "gavasun": run_gavasun}[args.workload](args)
+    families = {"salopel": run_salopel, "kodatar": run_kodatar, "rotutar": run_rotutar, "gavasun": run_gavasun, "loselix": run_loselix}
+    if args.workload in families:
+        families[args.workload](args)
         return
     if args.layers is None:
         args.layers = XL["n_layer"] if args.workload == "sweep" else MODELS[args.model]["n_layer"]

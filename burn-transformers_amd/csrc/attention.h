@@ -22,7 +22,7 @@ struct AttnArgs {
   // With splits > 1 the keys are cut into that many runs, each run is a work-group of its own that
   // leaves (output row, maximum, sum) in `partial` [rows][q_heads][splits][head_dim + 2], and a
   // second kernel joins them into `out`.  Decode: the runs of every sequence's keys, a row is a
-  // sequence.  Prompts (bfloat16, heads of 64, no window): the runs of every query tile's keys, a
+  // sequence.  Prompts (bfloat16, heads of 64 to 128, no window): the runs of every query tile's keys, a
   // row is a token of the step.
   int splits;
   float* partial;

@@ -110,23 +110,60 @@ __device__ __forceinline__ float sigmoid_weight(float r, const Scoring& sc) {
 // the running maximum before the first key: sigmoid weights have none, zero stands for it
 constexpr float FIRST_MAXIMUM = FORM == 2 ? 0.f : -INFINITY;
 
-// Four consecutive channels of one head's output row, gated and in the output's type.
-__device__ __forceinline__ void put4(const AttnArgs& a, int64_t tok, int head, int channel, const float (&v)[4], float head_gate) {
+// A query's gate for the channels 16 dt + 4 g + r that a lane stores, all asked for before the first store (a store may
+// touch what a later load reads, as far as the compiler knows, and each would then wait for the one before).
+struct RowGate {
+  float factor[STAGED ? HD / 16 : 1][4];
+};
+__device__ __forceinline__ void load_gate(RowGate& gate, const AttnArgs& a, int64_t tok, int head) {
   if constexpr (STAGED) {
-    float w[4];
+    const int g = (threadIdx.x & 63) >> 4;
+    const float whole = a.gate && a.gate_span == 0 ? bt_output_gate(a, tok, head, 0) : 1.f;
 #pragma unroll
-    for (int r = 0; r < 4; ++r)
-      w[r] = v[r] * (a.gate && a.gate_span == 1 ? bt_output_gate(a, tok, head, channel + r) : head_gate);
+    for (int dt = 0; dt < HD / 16; ++dt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) gate.factor[dt][r] = whole;
+    if (a.gate && a.gate_span == 1) {
+      // (16 lanes read 16 rows: 16 bytes at a time where the rows allow, or every load touches as many cache lines again)
+      const float* row = a.gate + tok * a.ld_gate + (int64_t)head * a.gate_dim;
+      floatx4 z[HD / 16];
+      if ((((uintptr_t)a.gate & 15) | (a.ld_gate & 3) | (a.gate_dim & 3)) == 0) {
+#pragma unroll
+        for (int dt = 0; dt < HD / 16; ++dt) {
+          const int channel = 16 * dt + 4 * g;
+          z[dt] = *reinterpret_cast<const floatx4*>(row + (channel < a.gate_dim ? channel : 0));
+        }
+      } else {
+#pragma unroll
+        for (int dt = 0; dt < HD / 16; ++dt)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int channel = 16 * dt + 4 * g + r;
+            z[dt][r] = row[channel < a.gate_dim ? channel : 0];
+          }
+      }
+#pragma unroll
+      for (int dt = 0; dt < HD / 16; ++dt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) gate.factor[dt][r] = 16 * dt + 4 * g + r < a.gate_dim ? bt_sigmoid(z[dt][r]) : 1.f;
+    }
+  }
+}
+
+// Four consecutive channels 16 dt + 4 g .. + 3 of one head's output row, gated and in the output's type.
+__device__ __forceinline__ void put4(const AttnArgs& a, int64_t tok, int head, int dt, const float (&v)[4], const RowGate& gate) {
+  const int64_t place = tok * a.ldo + head * HD + dt * 16 + 4 * ((threadIdx.x & 63) >> 4);
+  float w[4];
+#pragma unroll
+  for (int r = 0; r < 4; ++r) w[r] = STAGED ? v[r] * gate.factor[STAGED ? dt : 0][r] : v[r];
+  if constexpr (STAGED) {
     if (a.out_f32) {
-      *reinterpret_cast<floatx4*>(static_cast<float*>(a.out) + tok * a.ldo + head * HD + channel) = floatx4{w[0], w[1], w[2], w[3]};
+      *reinterpret_cast<floatx4*>(static_cast<float*>(a.out) + place) = floatx4{w[0], w[1], w[2], w[3]};
       return;
     }
-    bf16x4 packed = {(bf16_t)w[0], (bf16_t)w[1], (bf16_t)w[2], (bf16_t)w[3]};
-    *reinterpret_cast<bf16x4*>(static_cast<bf16_t*>(a.out) + tok * a.ldo + head * HD + channel) = packed;
-  } else {
-    bf16x4 packed = {(bf16_t)v[0], (bf16_t)v[1], (bf16_t)v[2], (bf16_t)v[3]};
-    *reinterpret_cast<bf16x4*>(static_cast<bf16_t*>(a.out) + tok * a.ldo + head * HD + channel) = packed;
   }
+  bf16x4 packed = {(bf16_t)w[0], (bf16_t)w[1], (bf16_t)w[2], (bf16_t)w[3]};
+  *reinterpret_cast<bf16x4*>(static_cast<bf16_t*>(a.out) + place) = packed;
 }
 // One channel, row-major or chunk-major.
 __device__ __forceinline__ void put1(const AttnArgs& a, int tok, int head, int channel, float v) {
@@ -138,9 +175,6 @@ __device__ __forceinline__ void put1(const AttnArgs& a, int tok, int head, int c
     }
   }
   static_cast<bf16_t*>(a.out)[activation_offset<bf16_t>(a.out_rows, a.ldo, tok, head * HD + channel)] = (bf16_t)v;
-}
-__device__ __forceinline__ float head_gate_of(const AttnArgs& a, int64_t tok, int head) {
-  return STAGED && a.gate && a.gate_span == 0 ? bt_output_gate(a, tok, head, 0) : 1.f;
 }
 
 // The online softmax of both forms below works on exponents, x = score * c - (the query's running
@@ -406,11 +440,12 @@ attention_prefill_kernel(AttnArgs a) {
     total += bt_sink_term_pow2(a.sink, head, m[nq]);
     float inv = FORM == 2 ? 1.0f : total > 0.f ? 1.0f / total : 0.f;
     if (qpos[nq] < 0) continue;
-    const float head_gate = head_gate_of(a, tok[nq], head);
+    RowGate gate;
+    load_gate(gate, a, tok[nq], head);
 #pragma unroll
     for (int dt = 0; dt < ND; ++dt) {
       const float row[4] = {o[nq][dt][0] * inv, o[nq][dt][1] * inv, o[nq][dt][2] * inv, o[nq][dt][3] * inv};
-      put4(a, tok[nq], head, dt * 16 + 4 * g, row, head_gate);
+      put4(a, tok[nq], head, dt, row, gate);
     }
   }
 }
@@ -426,25 +461,34 @@ attention_prefill_kernel(AttnArgs a) {
 //   `masked` (the same for the whole wave) says that some query of the wave does not see the
 //   whole block; both kinds of block run the same instructions but for the replacement of the
 //   excluded scores, so the compiler keeps every running sum in one place.
+//   `Operands` hands out the block's operands: k(t, ks) keys 16 t .. + 15 and channels 32 ks .. + 31,
+//   v(dt, half) channels 16 dt .. + 15 and positions 32 half .. + 31.  BOUNDED: a query may also have a
+//   first key that it sees (qlo).  RAGGED: positions from valid_end on may lie in the block.
 struct BlockOperands {
-  bf16x8 k[4][NKS];
-  bf16x8 v[ND][2];   // [block of 16 channels][half of the block's positions]: see SHARED_V_BYTES
+  bf16x8 keys[4][NKS];
+  bf16x8 values[ND][2];   // [block of 16 channels][half of the block's positions]: see SHARED_V_BYTES
+  __device__ __forceinline__ bf16x8 k(int t, int ks) const { return keys[t][ks]; }
+  __device__ __forceinline__ bf16x8 v(int dt, int half) const { return values[dt][half]; }
 };
 
-template <int NQ>
-__device__ __forceinline__ void attend_block(const BlockOperands& blk, int kb, int valid_end, bool masked,
-                                             const int (&qpos)[NQ], const Scoring& sc, const bf16x8 (&q)[NQ][NKS],
-                                             floatx4 (&o)[NQ][ND], float (&m)[NQ], floatx4 (&rows)[NQ]) {
+template <int NQ, bool BOUNDED, bool RAGGED, typename Operands>
+__device__ __forceinline__ void attend_block(const Operands& blk, int kb, int valid_end, bool masked,
+                                             const int (&qpos)[NQ], const int (&qlo)[NQ], const Scoring& sc,
+                                             const bf16x8 (&q)[NQ][NKS], floatx4 (&o)[NQ][ND], float (&m)[NQ],
+                                             floatx4 (&rows)[NQ]) {
   const int lane = threadIdx.x & 63, g = lane >> 4;
   floatx4 s[NQ][4];
 #pragma unroll
   for (int t = 0; t < 4; ++t) {
+    bf16x8 key[NKS];
+#pragma unroll
+    for (int ks = 0; ks < NKS; ++ks) key[ks] = blk.k(t, ks);
 #pragma unroll
     for (int nq = 0; nq < NQ; ++nq) {
       floatx4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int ks = 0; ks < NKS; ++ks)
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(blk.k[t][ks], q[nq][ks], acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(key[ks], q[nq][ks], acc, 0, 0, 0);
       s[nq][t] = acc;
     }
   }
@@ -463,7 +507,10 @@ __device__ __forceinline__ void attend_block(const BlockOperands& blk, int kb, i
 #pragma unroll
       for (int t = 0; t < 4; ++t)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) s[nq][t][r] = kb + 16 * t + 4 * g + r <= qp ? s[nq][t][r] : -INFINITY;
+        for (int r = 0; r < 4; ++r) {
+          const int kp = kb + 16 * t + 4 * g + r;
+          s[nq][t][r] = kp <= qp && (!BOUNDED || kp >= qlo[nq]) ? s[nq][t][r] : -INFINITY;
+        }
     }
   }
   float own[NQ];
@@ -520,12 +567,12 @@ __device__ __forceinline__ void attend_block(const BlockOperands& blk, int kb, i
 #pragma unroll
     for (int nq = 0; nq < NQ; ++nq)
       rows[nq] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pop[nq][half], rows[nq], 0, 0, 0);
-  const bool ragged = masked && kb + 64 > valid_end;
+  const bool ragged = RAGGED && masked && kb + 64 > valid_end;
 #pragma unroll
   for (int dt = 0; dt < ND; ++dt) {
 #pragma unroll
     for (int half = 0; half < 2; ++half) {
-      bf16x8 vop = blk.v[dt][half];
+      bf16x8 vop = blk.v(dt, half);
       if (ragged) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
@@ -536,6 +583,74 @@ __device__ __forceinline__ void attend_block(const BlockOperands& blk, int kb, i
 #pragma unroll
       for (int nq = 0; nq < NQ; ++nq)
         o[nq][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vop, pop[nq][half], o[nq][dt], 0, 0, 0);
+    }
+  }
+}
+
+// Two sets of waves that took different keys of the same queries: the second set's results go to the first through
+// LDS, lane to lane: value k of lane `lane` of wave `wave` at float (k * PREFILL_WAVES + wave) * 64 + lane.
+constexpr int HAND_PER_QUERY = 2 + 4 * ND;
+template <int NQ>
+__device__ __forceinline__ void hand_over(float* hand, int wave, const floatx4 (&o)[NQ][ND], const float (&m)[NQ],
+                                          const floatx4 (&rows)[NQ]) {
+  const int lane = threadIdx.x & 63;
+#pragma unroll
+  for (int nq = 0; nq < NQ; ++nq) {
+    const int k0 = nq * HAND_PER_QUERY;
+    hand[((k0 + 0) * PREFILL_WAVES + wave) * 64 + lane] = m[nq];
+    hand[((k0 + 1) * PREFILL_WAVES + wave) * 64 + lane] = rows[nq][0];
+#pragma unroll
+    for (int dt = 0; dt < ND; ++dt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) hand[((k0 + 2 + 4 * dt + r) * PREFILL_WAVES + wave) * 64 + lane] = o[nq][dt][r];
+  }
+}
+
+// The first set joins both and stores its queries' rows, or with runs of keys this run's records.
+template <int NQ>
+__device__ __forceinline__ void finish_rows(const AttnArgs& a, const float* hand, int wave, int head, int runs, int run,
+                                            const int (&qpos)[NQ], const int (&tok)[NQ], const floatx4 (&o)[NQ][ND],
+                                            const float (&m)[NQ], const floatx4 (&rows)[NQ]) {
+  const int lane = threadIdx.x & 63, g = lane >> 4;
+#pragma unroll
+  for (int nq = 0; nq < NQ; ++nq) {
+    const int k0 = nq * HAND_PER_QUERY;
+    const float m_other = hand[((k0 + 0) * PREFILL_WAVES + wave) * 64 + lane];
+    const float l_other = hand[((k0 + 1) * PREFILL_WAVES + wave) * 64 + lane];
+    const float top = fmaxf(m[nq], m_other);                       // (the maxima are kept in powers of two)
+    const float mine = m[nq] == -INFINITY ? 0.f : exp2f(m[nq] - top);
+    const float theirs = m_other == -INFINITY ? 0.f : exp2f(m_other - top);
+    const float total = rows[nq][0] * mine + l_other * theirs;   // (whole sums: see attend_block)
+    // (with runs the sink joins the denominator once, where the runs are joined)
+    float inv = FORM == 2 ? 1.0f : total > 0.f ? 1.0f / (total + bt_sink_term_pow2(a.sink, head, top)) : 0.f;
+    if (qpos[nq] < 0) continue;
+    if (runs > 1) {      // this run's share of the query's row, relative to its own maximum
+      typedef __attribute__((__vector_size__(2 * sizeof(float)))) float float2v;
+      float* record = a.partial + (((int64_t)tok[nq] * a.q_heads + head) * runs + run) * (HD + 2);
+#pragma unroll
+      for (int dt = 0; dt < ND; ++dt) {
+        float joined[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          joined[r] = o[nq][dt][r] * mine + hand[((k0 + 2 + 4 * dt + r) * PREFILL_WAVES + wave) * 64 + lane] * theirs;
+        *reinterpret_cast<float2v*>(record + dt * 16 + 4 * g) = float2v{joined[0], joined[1]};
+        *reinterpret_cast<float2v*>(record + dt * 16 + 4 * g + 2) = float2v{joined[2], joined[3]};
+      }
+      if (g == 0) {
+        record[HD] = top;
+        record[HD + 1] = total;
+      }
+      continue;
+    }
+    RowGate gate;
+    load_gate(gate, a, tok[nq], head);
+#pragma unroll
+    for (int dt = 0; dt < ND; ++dt) {
+      float joined[4];
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        joined[r] = (o[nq][dt][r] * mine + hand[((k0 + 2 + 4 * dt + r) * PREFILL_WAVES + wave) * 64 + lane] * theirs) * inv;
+      put4(a, tok[nq], head, dt, joined, gate);
     }
   }
 }
@@ -745,78 +860,225 @@ attention_prefill_split_kernel(AttnArgs a) {
 #pragma unroll
         for (int ks = 0; ks < NKS; ++ks) {
           int row = 16 * kt + i16, chunk = ks * 4 + g;
-          blk.k[kt][ks] = *reinterpret_cast<const bf16x8*>(stage + row * 128 + ((chunk ^ ((row >> 1) & 7)) << 4));
+          blk.keys[kt][ks] = *reinterpret_cast<const bf16x8*>(stage + row * 128 + ((chunk ^ ((row >> 1) & 7)) << 4));
         }
 #pragma unroll
       for (int dt = 0; dt < ND; ++dt)
 #pragma unroll
         for (int half = 0; half < 2; ++half)
-          blk.v[dt][half] = *reinterpret_cast<const bf16x8*>(stage + SHARED_K_BYTES +
+          blk.values[dt][half] = *reinterpret_cast<const bf16x8*>(stage + SHARED_K_BYTES +
                                                              ((4 * half + g) * 64 + dt * 16 + i16) * 16);
-      attend_block<PREFILL_NQ>(blk, kb, valid_end, kb + 64 > whole_until, qpos, sc, q, o, m, rows);
+      attend_block<PREFILL_NQ, false, true>(blk, kb, valid_end, kb + 64 > whole_until, qpos, qpos, sc, q, o, m, rows);
     }
     __syncthreads();   // turn t + 1 is in place, and everyone is done with turn t before it is overwritten
   }
-  // The second set's results go to the first, lane to lane: value k of lane `lane` of wave `wave`
-  // at float (k * PREFILL_WAVES + wave) * 64 + lane (everyone is past the last turn's barrier).
-  float* hand = reinterpret_cast<float*>(split_lds);
-  constexpr int PER_QUERY = 2 + 4 * ND;
-  if (set == 1) {
-#pragma unroll
-    for (int nq = 0; nq < PREFILL_NQ; ++nq) {
-      const int k0 = nq * PER_QUERY;
-      hand[((k0 + 0) * PREFILL_WAVES + wave) * 64 + lane] = m[nq];
-      hand[((k0 + 1) * PREFILL_WAVES + wave) * 64 + lane] = rows[nq][0];
-#pragma unroll
-      for (int dt = 0; dt < ND; ++dt)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) hand[((k0 + 2 + 4 * dt + r) * PREFILL_WAVES + wave) * 64 + lane] = o[nq][dt][r];
-    }
-  }
+  float* hand = reinterpret_cast<float*>(split_lds);   // (everyone is past the last turn's barrier)
+  if (set == 1) hand_over<PREFILL_NQ>(hand, wave, o, m, rows);
   __syncthreads();
   if (set == 1 || !active) return;
-#pragma unroll
-  for (int nq = 0; nq < PREFILL_NQ; ++nq) {
-    const int k0 = nq * PER_QUERY;
-    const float m_other = hand[((k0 + 0) * PREFILL_WAVES + wave) * 64 + lane];
-    const float l_other = hand[((k0 + 1) * PREFILL_WAVES + wave) * 64 + lane];
-    const float top = fmaxf(m[nq], m_other);                       // (the maxima are kept in powers of two)
-    const float mine = m[nq] == -INFINITY ? 0.f : exp2f(m[nq] - top);
-    const float theirs = m_other == -INFINITY ? 0.f : exp2f(m_other - top);
-    const float total = rows[nq][0] * mine + l_other * theirs;   // (whole sums: see attend_block)
-    // (with runs the sink joins the denominator once, where the runs are joined)
-    float inv = FORM == 2 ? 1.0f : total > 0.f ? 1.0f / (total + bt_sink_term_pow2(a.sink, head, top)) : 0.f;
-    if (qpos[nq] < 0) continue;
-    if (runs > 1) {      // this run's share of the query's row, relative to its own maximum
-      typedef __attribute__((__vector_size__(2 * sizeof(float)))) float float2v;
-      float* record = a.partial + (((int64_t)tok[nq] * a.q_heads + head) * runs + run) * (HD + 2);
-#pragma unroll
-      for (int dt = 0; dt < ND; ++dt) {
-        float joined[4];
-#pragma unroll
-        for (int r = 0; r < 4; ++r)
-          joined[r] = o[nq][dt][r] * mine + hand[((k0 + 2 + 4 * dt + r) * PREFILL_WAVES + wave) * 64 + lane] * theirs;
-        *reinterpret_cast<float2v*>(record + dt * 16 + 4 * g) = float2v{joined[0], joined[1]};
-        *reinterpret_cast<float2v*>(record + dt * 16 + 4 * g + 2) = float2v{joined[2], joined[3]};
-      }
-      if (g == 0) {
-        record[HD] = top;
-        record[HD + 1] = total;
-      }
-      continue;
-    }
-    const float head_gate = head_gate_of(a, tok[nq], head);
-#pragma unroll
-    for (int dt = 0; dt < ND; ++dt) {
-      float joined[4];
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        joined[r] = (o[nq][dt][r] * mine + hand[((k0 + 2 + 4 * dt + r) * PREFILL_WAVES + wave) * 64 + lane] * theirs) * inv;
-      put4(a, tok[nq], head, dt * 16 + 4 * g, joined, head_gate);
-    }
-  }
+  finish_rows<PREFILL_NQ>(a, hand, wave, head, runs, run, qpos, tok, o, m, rows);
 }
 #endif  // BT_HEAD_DIM == 64
+
+#if BT_HEAD_DIM > 64 && BT_HEAD_DIM <= 128
+#define BT_WIDE_PREFILL 1
+// Heads of 80 to 128: a work-group of eight waves takes one tile of 128 queries of one head in two sets of four waves, as
+// above (the same queries, the even and the odd blocks of keys), with windows and chunks too.  A turn is two blocks of keys
+// and values, 80 to 128 KiB in two stages, and there is neither room nor a register to spare for waves that only bring
+// them: every wave starts its share of the next turn's planes as loads straight into LDS (global_load_lds, a
+// contiguous KiB an instruction) and then multiplies the turn that is in place.  One barrier a turn.  The swizzles that
+// keep the operand reads free of bank conflicts are applied on the memory side: a lane fetches the 16 bytes that belong
+// where its piece of the KiB lands.
+//   keys:   row r keeps its 16-byte chunk c at c ^ key_swizzle(r): sixteen rows of one chunk then lie in different banks
+//           whatever the rows' length does to them;
+//   values: as in the cache, [16][HD][4]: an operand is two 8-byte reads, four rows of 8 * HD bytes apart; where those
+//           rows fall on the same banks (HD a multiple of 32), odd rows have each pair of blocks of 16 channels exchanged.
+constexpr int WIDE_PLANE = BT_KV_BLOCK * HD * 2;     // bytes of a block's keys, or of its values
+constexpr int WIDE_STAGE = 2 * WIDE_PLANE;
+constexpr int WIDE_TURN = 2 * WIDE_STAGE;
+constexpr int WIDE_LDS_BYTES = 2 * WIDE_TURN;
+constexpr int WIDE_LOADS = HD / 16;                  // a wave's instructions for its half of one plane of a turn
+#define WIDE_THREADS (2 * PREFILL_WAVES * 64)
+static_assert(PREFILL_NQ * HAND_PER_QUERY * PREFILL_WAVES * 64 * 4 <= WIDE_LDS_BYTES, "the second set's results fit where the keys were");
+
+__device__ __forceinline__ int key_swizzle(int row) {
+  return HD == 128 ? row & 15 : HD == 96 ? (row >> 2) & 3 : (row >> 3) & 1;
+}
+__device__ __forceinline__ int value_swap(int four) { return HD % 32 == 0 ? four & 1 : 0; }
+
+struct WideOperands {
+  const unsigned char* stage;
+  int key_at[NKS];        // of the lane's row i16 of a tile of 16 keys, for every step of 32 channels
+  int value_at[2];        // of the lane's channel and group of positions, for even and odd blocks of 16 channels
+  __device__ __forceinline__ bf16x8 k(int t, int ks) const {
+    return *reinterpret_cast<const bf16x8*>(stage + key_at[ks] + t * 32 * HD);
+  }
+  __device__ __forceinline__ bf16x8 v(int dt, int half) const {
+    const unsigned char* p = stage + WIDE_PLANE + value_at[dt & 1] + dt * 128 + half * 64 * HD;
+    const bf16x4 a = *reinterpret_cast<const bf16x4*>(p), b = *reinterpret_cast<const bf16x4*>(p + 32 * HD);
+    return bf16x8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+  }
+};
+
+__global__ void __launch_bounds__(WIDE_THREADS)
+attention_prefill_wide_kernel(AttnArgs a) {
+  extern __shared__ __attribute__((aligned(16))) unsigned char wide_lds[];   // [2 turns][2 blocks][WIDE_STAGE]
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int wave8 = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int set = wave8 / PREFILL_WAVES, wave = wave8 % PREFILL_WAVES;
+  const int i16 = lane & 15, g = lane >> 4;
+  // Work-groups that read the same keys and values lie on one XCD, latest tiles first (as above).  With fewer such units
+  // than XCDs every query head is a unit of its own, so that no XCD stays empty.
+  const int runs = a.splits > 1 ? a.splits : 1;
+  const int q_tiles = (a.max_count + PREFILL_QUERIES - 1) / PREFILL_QUERIES;
+  const int by_kv = a.n_seqs * a.kv.kv_heads * runs;
+  const bool fine = by_kv < 8;
+  const int group = fine ? 1 : a.q_heads / a.kv.kv_heads;                  // heads of a unit
+  const int unit_heads = fine ? a.q_heads : a.kv.kv_heads;
+  const int units = a.n_seqs * unit_heads * runs, units_per_xcd = (units + 7) / 8;
+  const int xcd = blockIdx.x & 7, slot = blockIdx.x >> 3;
+  const int per_rank = units_per_xcd * group;
+  const int rank = slot / per_rank, inside = slot % per_rank;
+  const int unit = (inside / group) * 8 + xcd;
+  if (unit >= units || rank >= q_tiles) return;             // the whole work-group
+  const int pair = unit / runs, run = unit % runs;
+  const int seq = pair / unit_heads;
+  const int head = (pair % unit_heads) * group + inside % group;
+  const int kv_head = head / (a.q_heads / a.kv.kv_heads);
+  const int q_tile = q_tiles - 1 - rank;
+  const int off = a.seq_off[seq], count = a.seq_off[seq + 1] - off, start = a.seq_start[seq];
+  if (q_tile * PREFILL_QUERIES >= count) return;            // the whole work-group: this sequence is shorter
+  const int reach = (q_tile + 1) * PREFILL_QUERIES < count ? (q_tile + 1) * PREFILL_QUERIES : count;
+  const int first_block = bt_first_seen(start + q_tile * PREFILL_QUERIES, a.window, a.chunk) / BT_KV_BLOCK;
+  const int last_block = (start + reach - 1) / BT_KV_BLOCK;
+  const int n_turns = (last_block - first_block + 2) / 2;
+  const int per_run = (n_turns + runs - 1) / runs;
+  const int t_begin = run * per_run;
+  const int t_end = t_begin + per_run < n_turns ? t_begin + per_run : n_turns;
+
+  // the wave's half of one plane of every turn: block `bring_block` of the turn, its keys or its values
+  const int bring_block = wave8 >> 2, bring_values = (wave8 >> 1) & 1, bring_half = wave8 & 1;
+  unsigned from[WIDE_LOADS];
+#pragma unroll
+  for (int j = 0; j < WIDE_LOADS; ++j) {
+    const int piece = (bring_half * WIDE_LOADS + j) * 64 + lane;              // 16 bytes each, in the order of the LDS
+    const int line = bring_values ? HD / 2 : HD / 8;                          // pieces of a row
+    const int row = piece / line, c = piece % line;
+    from[j] = (unsigned)(row * line + (c ^ (bring_values ? value_swap(row) << 3 : key_swizzle(row)))) * 16u;
+  }
+  const unsigned char* planes = static_cast<const unsigned char*>(bring_values ? a.kv.values : a.kv.keys);
+  const int* block_row = a.kv.blocks + (int64_t)seq * a.kv.max_blocks;
+  auto block_of = [&](int turn) {                           // where the wave's block of a turn lies
+    const int block = first_block + 2 * turn + bring_block;
+    return block_row[block < last_block ? block : last_block];                // (one too many: brought again, never multiplied)
+  };
+  auto bring = [&](int physical, int stage) {
+    const unsigned char* src = planes + kv_plane(a.kv, __builtin_amdgcn_readfirstlane(physical), kv_head) * 2;
+    unsigned char* dst = wide_lds + stage * WIDE_TURN + bring_block * WIDE_STAGE + bring_values * WIDE_PLANE +
+                         bring_half * WIDE_LOADS * 1024;
+#pragma unroll
+    for (int j = 0; j < WIDE_LOADS; ++j)
+      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src + from[j]),
+                                       (__attribute__((address_space(3))) void*)(dst + j * 1024), 16, 0, 0);
+  };
+  int next_block = 0;                                       // of the turn after next, asked for a turn ahead
+  if (t_begin < t_end) {
+    bring(block_of(t_begin), 0);
+    next_block = block_of(t_begin + 1);
+  }
+
+  const int q0 = q_tile * PREFILL_QUERIES + wave * PREFILL_QUERIES_PER_WAVE;
+  const bool active = q0 < count;
+  const bf16_t* Q = static_cast<const bf16_t*>(a.q);
+  const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
+  int qpos[PREFILL_NQ], qlo[PREFILL_NQ], tok[PREFILL_NQ];
+  bf16x8 q[PREFILL_NQ][NKS];
+  floatx4 o[PREFILL_NQ][ND], rows[PREFILL_NQ];
+  float m[PREFILL_NQ];
+#pragma unroll
+  for (int nq = 0; nq < PREFILL_NQ; ++nq) {
+    const int qi = q0 + nq * 16 + i16;
+    const bool exists = active && qi < count;
+    qpos[nq] = exists ? start + qi : -1;
+    qlo[nq] = exists ? bt_first_seen(start + qi, a.window, a.chunk) : 0;
+    tok[nq] = off + (exists ? qi : count - 1);
+#pragma unroll
+    for (int ks = 0; ks < NKS; ++ks) {
+      const int channel = ks * 32 + g * 8;
+      q[nq][ks] = channel < HD ? load_bf16x8(Q + (int64_t)tok[nq] * a.ldq + head * HD + channel) : zero8;
+    }
+#pragma unroll
+    for (int dt = 0; dt < ND; ++dt) o[nq][dt] = floatx4{0.f, 0.f, 0.f, 0.f};
+    rows[nq] = floatx4{0.f, 0.f, 0.f, 0.f};
+    m[nq] = FIRST_MAXIMUM;
+  }
+  const int last = q0 + PREFILL_QUERIES_PER_WAVE < count ? q0 + PREFILL_QUERIES_PER_WAVE : count;
+  const int hi = active ? start + last : 0;                 // one past the position of the wave's last query
+  const int lo = active ? bt_first_seen(start + q0, a.window, a.chunk) : 0;             // the first key that any of its queries sees ...
+  const int lo_last = active ? bt_first_seen(start + last - 1, a.window, a.chunk) : 0;  // ... and the first that all of them do
+  const int valid_end = start + count;
+  const Scoring sc = scoring_of(a, head);
+
+  if (t_begin >= t_end) {     // a run beyond the tile's last turn: its records say that it saw no key
+    if (set == 0 && g == 0) {
+#pragma unroll
+      for (int nq = 0; nq < PREFILL_NQ; ++nq)
+        if (qpos[nq] >= 0) {
+          float* record = a.partial + (((int64_t)tok[nq] * a.q_heads + head) * runs + run) * (HD + 2);
+          record[HD] = -INFINITY;
+          record[HD + 1] = 0.f;
+        }
+    }
+    return;
+  }
+  WideOperands ops;
+#pragma unroll
+  for (int ks = 0; ks < NKS; ++ks) {
+    int chunk = ks * 4 + g;
+    chunk = chunk < HD / 8 ? chunk : HD / 8 - 1;            // (channels behind the head meet zeros of the query)
+    ops.key_at[ks] = i16 * HD * 2 + ((chunk ^ key_swizzle(i16)) << 4);
+  }
+  const int swap = value_swap(g) * 128;
+  ops.value_at[0] = g * HD * 8 + i16 * 8 + swap;
+  ops.value_at[1] = g * HD * 8 + i16 * 8 - swap;
+  for (int t = t_begin; t < t_end; ++t) {
+    // my share of turn t has landed, and my reads of turn t - 1 are done; behind the barrier so are everyone's
+    // (the builtin, not an instruction by hand: the compiler then knows that the queries have arrived too and does not
+    // wait for the planes on their way when it first multiplies by them)
+    asm volatile("" ::: "memory");
+    __builtin_amdgcn_s_waitcnt(0x0070);                     // vmcnt(0) lgkmcnt(0)
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+    if (t + 1 < t_end) {
+      bring(next_block, (t + 1 - t_begin) & 1);
+      next_block = block_of(t + 2);
+    }
+    // values of positions that hold no token (they may be anything, and 0 * NaN is NaN) become zero where they lie, once,
+    // in the turn that holds the sequence's last block: a test before every operand would keep their reads from flying together
+    const int beyond = valid_end - last_block * BT_KV_BLOCK;
+    if (beyond < BT_KV_BLOCK && first_block + 2 * t + 1 >= last_block) {      // (the same for the whole work-group)
+      unsigned short* v = reinterpret_cast<unsigned short*>(wide_lds + ((t - t_begin) & 1) * WIDE_TURN +
+                                                            ((last_block - first_block) & 1) * WIDE_STAGE + WIDE_PLANE);
+      for (int e = (beyond >> 2) * 4 * HD + tid; e < BT_KV_BLOCK * HD; e += WIDE_THREADS)
+        if (e / (4 * HD) * 4 + (e & 3) >= beyond) v[e] = 0;
+      __syncthreads();
+    }
+    const int block = first_block + 2 * t + set;
+    const int kb = block * BT_KV_BLOCK;
+    if (block <= last_block && kb < hi && kb + BT_KV_BLOCK > lo) {           // (the same for the whole wave)
+      ops.stage = wide_lds + ((t - t_begin) & 1) * WIDE_TURN + set * WIDE_STAGE;
+      attend_block<PREFILL_NQ, true, false>(ops, kb, valid_end, kb + BT_KV_BLOCK > start + q0 + 1 || kb < lo_last, qpos, qlo, sc, q,
+                                            o, m, rows);
+    }
+  }
+  __syncthreads();                                          // everyone is done with the last turn
+  float* hand = reinterpret_cast<float*>(wide_lds);
+  if (set == 1) hand_over<PREFILL_NQ>(hand, wave, o, m, rows);
+  __syncthreads();
+  if (set == 1 || !active) return;
+  finish_rows<PREFILL_NQ>(a, hand, wave, head, runs, run, qpos, tok, o, m, rows);
+}
+#endif  // BT_HEAD_DIM > 64 && BT_HEAD_DIM <= 128
 
 // Eight waves: measured against sixteen and four at batches 1 to 64 (contexts of 500 to 900), eight
 // are never slower, and at batch 64 a compute unit then holds two work-groups, so that one's
@@ -1025,8 +1287,8 @@ BT_EXPORT int bt_attention_prefill_bf16(void* stream, const AttnArgs* args) {
   if (rc) return rc;
   if (args->max_count <= 0) BT_REFUSE("attention_prefill_bf16: max_count %d must be positive", args->max_count);
   const int runs = args->splits > 1 ? args->splits : 1;
-  if (runs > 1 && (HD != 64 || args->window != 0 || args->chunk != 0 || !args->partial || runs > 64))
-    BT_REFUSE("attention_prefill_bf16: runs of keys (%d) are for heads of 64 without a window, at most 64, and need a place "
+  if (runs > 1 && (HD < 64 || HD > 128 || args->window != 0 || args->chunk != 0 || !args->partial || runs > 64))
+    BT_REFUSE("attention_prefill_bf16: runs of keys (%d) are for heads of 64 to 128 without a window, at most 64, and need a place "
               "for their partial results", runs);
   const int q_tiles = (args->max_count + PREFILL_QUERIES - 1) / PREFILL_QUERIES;
   const int group = args->q_heads / args->kv.kv_heads;
@@ -1055,6 +1317,31 @@ BT_EXPORT int bt_attention_prefill_bf16(void* stream, const AttnArgs* args) {
     const int64_t split_groups = 8 * ((units * runs + 7) / 8) * group * q_tiles;
     if (split_groups > 0x7fffffff) BT_REFUSE("attention_prefill_bf16: %lld work-groups are too many", (long long)split_groups);
     hipLaunchKernelGGL(attention_prefill_split_kernel, dim3((unsigned)split_groups), dim3(SPLIT_THREADS), SPLIT_LDS_BYTES,
+                       (hipStream_t)stream, *args);
+    if (runs > 1) {
+      rc = bt_check_launch("attention_prefill_bf16");
+      if (rc) return rc;
+      if ((int64_t)args->n_tokens * args->q_heads > 0x7fffffff) BT_REFUSE("attention_prefill_bf16: too many rows to join");
+      hipLaunchKernelGGL(attention_join_kernel, dim3((unsigned)(((int64_t)args->n_tokens * args->q_heads + 3) / 4)), dim3(256), 0,
+                         (hipStream_t)stream, *args, args->n_tokens);
+    }
+    return bt_check_launch("attention_prefill_bf16");
+  }
+#endif
+#if BT_WIDE_PREFILL
+  {
+    static bool raised = false;                 // up to 128 KiB: beyond what a kernel gets without asking
+    if (!raised) {
+      hipError_t err = hipFuncSetAttribute((const void*)attention_prefill_wide_kernel,
+                                           hipFuncAttributeMaxDynamicSharedMemorySize, (int)WIDE_LDS_BYTES);
+      if (err != hipSuccess) BT_REFUSE("attention_prefill_bf16: cannot get %d bytes of LDS: %s", (int)WIDE_LDS_BYTES, hipGetErrorString(err));
+      raised = true;
+    }
+    const bool fine = units * runs < 8;
+    const int64_t shares = fine ? (int64_t)args->n_seqs * args->q_heads * runs : units * runs;
+    const int64_t wide_groups = 8 * ((shares + 7) / 8) * (fine ? 1 : group) * q_tiles;
+    if (wide_groups > 0x7fffffff) BT_REFUSE("attention_prefill_bf16: %lld work-groups are too many", (long long)wide_groups);
+    hipLaunchKernelGGL(attention_prefill_wide_kernel, dim3((unsigned)wide_groups), dim3(WIDE_THREADS), WIDE_LDS_BYTES,
                        (hipStream_t)stream, *args);
     if (runs > 1) {
       rc = bt_check_launch("attention_prefill_bf16");

@@ -132,8 +132,9 @@ __device__ __forceinline__ EpiloguePrefetch epilogue_prefetch(const Epilogue& e,
   return p;
 }
 
-// The epilogue with everything but the accumulators already in registers.
-template <typename T>
+// The epilogue with everything but the accumulators already in registers.  TWO: the mode is EPI_F32_ACT (a form of the
+// kernel of its own, so that the others carry none of it).
+template <typename T, bool TWO = false>
 __device__ __forceinline__ void epilogue4_prefetched(const Epilogue& e, int N, int m, int n0, const float* acc,
                                                      int split, const EpiloguePrefetch& p) {
   int count = N - n0 < 4 ? N - n0 : 4;
@@ -142,6 +143,18 @@ __device__ __forceinline__ void epilogue4_prefetched(const Epilogue& e, int N, i
 #pragma unroll
   for (int i = 0; i < 4; ++i) v[i] = acc[i] + p.add[i];
   bool aligned = (e.ldo & 3) == 0;
+  if constexpr (TWO) {
+    if (n0 < e.n_q) {
+      store4<float>(static_cast<float*>(e.out) + (int64_t)m * e.ldo + n0, v, count, aligned);
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = activate<T>(v[i], e.act);
+      const int c = n0 - e.n_q;
+      if (e.out_rows == 0) store4<T>(static_cast<T*>(e.out2) + (int64_t)m * e.ldo2 + c, v, count, (e.ldo2 & 3) == 0);
+      else store4<T>(static_cast<T*>(e.out2) + activation_offset<T>(e.out_rows, e.ldo2, m, c), v, count, true);
+    }
+    return;
+  }
   if (e.mode == EPI_STORE) {
     if (e.out_rows == 0) store4<T>(static_cast<T*>(e.out) + (int64_t)m * e.ldo + n0, v, count, aligned);     // (one branch for all threads)
     else store4<T>(static_cast<T*>(e.out) + activation_offset<T>(e.out_rows, e.ldo, m, n0), v, count, true);
@@ -155,16 +168,6 @@ __device__ __forceinline__ void epilogue4_prefetched(const Epilogue& e, int N, i
                   v, count, aligned);
   } else if (e.mode == EPI_RESIDUAL) {
     store4<float>(static_cast<float*>(e.out) + (int64_t)m * e.ldo + n0, v, count, aligned);
-  } else if (e.mode == EPI_F32_ACT) {
-    if (n0 < e.n_q) {
-      store4<float>(static_cast<float*>(e.out) + (int64_t)m * e.ldo + n0, v, count, aligned);
-    } else {
-#pragma unroll
-      for (int i = 0; i < 4; ++i) v[i] = activate<T>(v[i], e.act);
-      const int c = n0 - e.n_q;
-      if (e.out_rows == 0) store4<T>(static_cast<T*>(e.out2) + (int64_t)m * e.ldo2 + c, v, count, (e.ldo2 & 3) == 0);
-      else store4<T>(static_cast<T*>(e.out2) + activation_offset<T>(e.out_rows, e.ldo2, m, c), v, count, true);
-    }
   } else {
     if (n0 < e.n_q) {
       store4<T>(static_cast<T*>(e.out) + (int64_t)m * e.ldo + n0, v, count, aligned);

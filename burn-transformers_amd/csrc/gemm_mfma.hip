@@ -636,7 +636,7 @@ gemm_tile_deep_kernel(const bf16_t* __restrict__ A, int64_t lda, const bf16_t* _
 // statistics are computed while the weights are on their way.
 __device__ float bt_norm_zeros[4] = {0.f, 0.f, 0.f, 0.f};
 
-template <typename T, int MT, int NT, int U, int WAVES, int QPL = 0, bool CHUNKED = false>
+template <typename T, int MT, int NT, int U, int WAVES, int QPL = 0, bool CHUNKED = false, bool TWO = false>
 __global__ void __launch_bounds__(WAVES * 64)
 gemm_skinny_kernel(const T* __restrict__ A, int64_t lda, const T* __restrict__ W, int M, int N,
                    int K, Epilogue epi, int tile_columns, NormOperand norm, int packed, int a_rows) {
@@ -830,7 +830,7 @@ gemm_skinny_kernel(const T* __restrict__ A, int64_t lda, const T* __restrict__ W
     for (int w = 0; w < WAVES; ++w)
 #pragma unroll
       for (int r = 0; r < 4; ++r) v[r] += red[w][wave][lane][r];
-    if (out_m < M) epilogue4_prefetched<T>(epi, n_end, out_m, out_n0, v, split, pre);   // nothing beyond n_end
+    if (out_m < M) epilogue4_prefetched<T, TWO>(epi, n_end, out_m, out_n0, v, split, pre);   // nothing beyond n_end
   }
 }
 
@@ -953,9 +953,16 @@ static void launch_skinny(hipStream_t s, const T* a, int64_t lda, const T* w, in
                           int splits, int columns, int packed, int a_rows) {
   dim3 grid((N + columns - 1) / columns, splits), block(512);
   const NormOperand none = {};
+  const bool two = epi.mode == EPI_F32_ACT;
 #define LAUNCH_SKINNY(MT, NT, U)                                                                                   \
   do {                                                                                                             \
-    if (a_rows > 0)                                                                                                \
+    if (two && a_rows > 0)                                                                                         \
+      hipLaunchKernelGGL((gemm_skinny_kernel<T, MT, NT, U, 8, 0, true, true>), grid, block, 0, s, a, lda, w, M, N, K, \
+                         epi, columns, none, packed, a_rows);                                                      \
+    else if (two)                                                                                                  \
+      hipLaunchKernelGGL((gemm_skinny_kernel<T, MT, NT, U, 8, 0, false, true>), grid, block, 0, s, a, lda, w, M, N, K, \
+                         epi, columns, none, packed, 0);                                                           \
+    else if (a_rows > 0)                                                                                           \
       hipLaunchKernelGGL((gemm_skinny_kernel<T, MT, NT, U, 8, 0, true>), grid, block, 0, s, a, lda, w, M, N, K, epi, \
                          columns, none, packed, a_rows);                                                           \
     else                                                                                                           \
@@ -1021,6 +1028,8 @@ BT_EXPORT int bt_gemm_skinny(void* stream, int dtype, const void* A, int64_t lda
   if (a_rows != 0 && (norm != nullptr || a_rows < M))
     BT_REFUSE("gemm_skinny: chunk-major activations of %d rows for a product of %d rows%s", a_rows, M,
               norm != nullptr ? " that normalises its rows itself" : "");
+  if (norm != nullptr && epi->mode == EPI_F32_ACT)
+    BT_REFUSE("gemm_skinny: 32-bit and activated columns of one product come from rows that are normalised already");
   if (norm != nullptr) {
     if (dtype != 1 || M > 16 || K > 2048)
       BT_REFUSE("gemm_skinny: the fused norm takes bfloat16 weights, up to 16 rows and K up to 2048 (got %d rows, K %d)", M, K);

@@ -54,6 +54,7 @@ struct HeadRotaryCall {
 template <typename T>
 __global__ void __launch_bounds__(HR_WAVES * 64) head_rotary_kernel(HeadRotaryCall c) {
   __shared__ float rows[HR_WAVES][HR_MAX_DIM];
+  __shared__ float sines[HR_MAX_DIM / 2], cosines[HR_MAX_DIM / 2];      // of the token's position: the same for all its heads
   const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int unit = blockIdx.y * HR_WAVES + wave;           // a query head, then a key head, then a value head
   const int n_q = c.heads * c.maps, n_k = c.kv_heads * c.maps;
@@ -89,10 +90,16 @@ __global__ void __launch_bounds__(HR_WAVES * 64) head_rotary_kernel(HeadRotaryCa
       for (int col = lane; col < n; col += 64) row[col] = row[col] * rstd * gamma[col];
     }
   }
-  __syncthreads();
-  if (!active) return;
   const int pos = c.tok_pos[t];
   const int half = c.rot_dims >> 1;
+  for (int i = threadIdx.x; i < half; i += HR_WAVES * 64) {
+    float sn, cs;
+    sincosf((float)pos * c.inv_freq[i], &sn, &cs);
+    sines[i] = sn * c.amplitude;
+    cosines[i] = cs * c.amplitude;
+  }
+  __syncthreads();
+  if (!active) return;
   const bool turned = (is_q || is_k) && half > 0;
   T* q_out = static_cast<T*>(c.q_out) + (int64_t)t * c.ld_q + (int64_t)head * hd;
   T* keys = nullptr;
@@ -112,13 +119,10 @@ __global__ void __launch_bounds__(HR_WAVES * 64) head_rotary_kernel(HeadRotaryCa
     else
       values[value_offset(hd, pos, col)] = from_float<T>(v);
   };
-  // a lane takes a pair of channels: the angle's sine and cosine are computed once for both
+  // a lane takes a pair of channels
   if (turned)
     for (int i = lane; i < half; i += 64) {
-      float sn, cs;
-      sincosf((float)pos * c.inv_freq[i], &sn, &cs);
-      sn *= c.amplitude;
-      cs *= c.amplitude;
+      const float sn = sines[i], cs = cosines[i];
       const int first = c.pairing == 1 ? 2 * i : i, second = c.pairing == 1 ? 2 * i + 1 : i + half;
       const float u = row[first], v = row[second];
       store(offset + first, u * cs - v * sn);

@@ -4,8 +4,10 @@
 //     its bias), N an RMS norm, v / sqrt(mean(v^2) + eps) * gamma, or a layer norm,
 //     (v - mean) / sqrt(var + eps) * gamma + beta; and a copy of the new x in the products' type
 //   * joined rows: [x | y] side by side in the products' type, the operand of a product that reads two streams
+//   * an activation in place, behind products whose kernel has none
 //   * PolyNorm: a N(z) + b N(z^2) + c N(z^3) + e, N(v) = v / sqrt(mean(v^2) + eps) over a row
 #include "host.h"
+#include "epilogue.h"
 
 struct OutputNormCall {
   int cast_dtype;        // element type of `cast`: 0 float32, 1 bfloat16
@@ -608,4 +610,52 @@ BT_EXPORT int bt_soft_cap_call(void* stream, const SoftCapCall* c) {
   if (per_row > 64) per_row = 64;
   hipLaunchKernelGGL(soft_cap_kernel, dim3(c->rows, per_row), dim3(256), 0, (hipStream_t)stream, *c);
   return bt_check_launch("soft_cap");
+}
+
+// ---------------------------------------------------------------------------------------------
+// An activation in place on a product's stored result: behind products whose kernel (the vendor's library) has no such
+// epilogue.  Rows of `columns` values, 16 bytes a thread where pitch and width allow.
+// ---------------------------------------------------------------------------------------------
+struct ActivateCall {
+  int dtype;
+  int tokens;
+  int columns;
+  int act;               // Activation (epilogue.h)
+  void* rows;            // [tokens][ld]
+  int64_t ld;
+};
+
+template <typename T>
+__global__ void __launch_bounds__(256) activate_kernel(ActivateCall c) {
+  constexpr int V = 16 / (int)sizeof(T);
+  T* row = static_cast<T*>(c.rows) + (int64_t)blockIdx.y * c.ld;
+  const int col = (blockIdx.x * 256 + threadIdx.x) * V;
+  if (col >= c.columns) return;
+  T v[V];
+  const bool whole = col + V <= c.columns && (((uintptr_t)(row + col)) & 15) == 0;
+  if (whole)
+    *reinterpret_cast<float4*>(v) = *reinterpret_cast<const float4*>(row + col);
+  else
+    for (int i = 0; i < V; ++i) v[i] = col + i < c.columns ? row[col + i] : from_float<T>(0.f);
+#pragma unroll
+  for (int i = 0; i < V; ++i) v[i] = from_float<T>(activate<T>(to_float(v[i]), c.act));
+  if (whole)
+    *reinterpret_cast<float4*>(row + col) = *reinterpret_cast<const float4*>(v);
+  else
+    for (int i = 0; i < V; ++i)
+      if (col + i < c.columns) row[col + i] = v[i];
+}
+
+BT_EXPORT int bt_activate_call(void* stream, const ActivateCall* c) {
+  if (c->tokens <= 0) return BT_OK;
+  if (c->columns <= 0 || !c->rows || c->ld < c->columns || c->act < 0 || c->act > 2)
+    BT_REFUSE("activate: %d columns of rows %lld apart, activation %d", c->columns, (long long)c->ld, c->act);
+  if (c->tokens > 65535) BT_REFUSE("activate: %d rows in one call, at most 65535", c->tokens);
+  const int per = 256 * (c->dtype == 0 ? 4 : 8);
+  dim3 grid((c->columns + per - 1) / per, c->tokens), block(256);
+  if (c->dtype == 0)
+    hipLaunchKernelGGL(activate_kernel<float>, grid, block, 0, (hipStream_t)stream, *c);
+  else
+    hipLaunchKernelGGL(activate_kernel<bf16_t>, grid, block, 0, (hipStream_t)stream, *c);
+  return bt_check_launch("activate");
 }

@@ -103,6 +103,11 @@ class JoinRowsCall(ctypes.Structure):
     _step_fields_ = {"tokens": "tokens"}
 
 
+class ActivateCall(ctypes.Structure):
+    _fields_ = [("dtype", _c_int), ("tokens", _c_int), ("columns", _c_int), ("act", _c_int), ("rows", _c_ptr), ("ld", _c_i64)]
+    _step_fields_ = {"tokens": "tokens"}
+
+
 class PolyNormCall(ctypes.Structure):
     _fields_ = [("out_dtype", _c_int), ("tokens", _c_int), ("columns", _c_int), ("out_cols", _c_int), ("eps", _c_float),
                 ("z", _c_ptr), ("ldz", _c_i64), ("coefficients", _c_ptr), ("out", _c_ptr), ("ldo", _c_i64)]
@@ -1143,6 +1148,23 @@ def join_rows(x, y, out):
     _launch(_module("sublayer"), "bt_join_rows_call",
             JoinRowsCall(out_dtype=DTYPE_CODES[out.dtype], tokens=x.shape[0], width=x.shape[1], out_cols=out.shape[1],
                          x=x.data_ptr(), y=y.data_ptr(), out=out.data_ptr(), ldo=out.stride(0)))
+
+
+def activate(rows, activation):
+    """rows <- activation(rows), in place (row-major, float32 or bfloat16, rows may be strided)."""
+    _launch(_module("sublayer"), "bt_activate_call",
+            ActivateCall(dtype=DTYPE_CODES[rows.dtype], tokens=rows.shape[0], columns=rows.shape[1], act=ACTIVATIONS[activation],
+                         rows=rows.data_ptr(), ld=rows.stride(0)))
+
+
+def activation_needs_a_pass(a, w, activation):
+    """Whether a product of these operands is the vendor's library's if only the activation were its own: it then runs
+    there without one, and ``activate`` follows (2,048 rows of 4096 x 1024: 24 + 8 us where the tile kernel with
+    the activation in its epilogue takes 43)."""
+    if a.dtype != torch.bfloat16 or isinstance(a, (Chunked, Normalized)) or not 64 < a.shape[0] <= 65535 or \
+            deep_form_rows(a.shape[0], a.shape[1], a.stride(0), w.shape[0]):
+        return False
+    return activation == "squared_relu" and library_products() is not None
 
 
 def poly_norm(z, columns, coefficients, eps, out):

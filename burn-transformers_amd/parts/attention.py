@@ -57,6 +57,7 @@ class CausalSelfAttention(Mixer):
             raise ValueError(f"attention: head size {self.head_dim} must be positive")
         if self.heads % self.kv_heads != 0:
             raise ValueError(f"attention: {self.heads} query heads cannot share {self.kv_heads} key/value heads")
+        self.q_heads = self.heads                         # queries the attention kernels see
         self.n_q, self.n_kv = self.heads * self.head_dim, self.kv_heads * self.head_dim
         self.qkv_weight, self.qkv_bias = tensors["qkv_weight"], tensors.get("qkv_bias")
         self.out_weight, self.out_bias = tensors["out_weight"], tensors.get("out_bias")
@@ -120,13 +121,13 @@ class CausalSelfAttention(Mixer):
         1,024 tokens 16.6 / 16.9 / 17.3 / 18.0, 2,048: 25.9 / 21.9 / 20.4 / 20.8, 4,096: 45.7 / 31.9 /
         25.5 / 25.3, 8,192: 84.5 / 51.9 / 35.6 / 33.7; two sequences (100 work-groups) 4,096: 48.1 /
         36.9, 8,192: 88.4 / 57.7."""
-        if step.decode or not step.dtype_is_bf16 or self.head_dim != 64 or self.window or self.chunk or self.plain_only:
+        if step.decode or not step.dtype_is_bf16 or not 64 <= self.head_dim <= 128 or self.window or self.chunk or self.plain_only:
             return 1
         if step.context_limit <= PROMPT_RUN_MIN_CONTEXT:
             return 1
         tiles = -(-step.token_capacity // 128) + step.n_seqs - 1          # at most so many hold queries
         blocks = PROMPT_RUN_BLOCKS * -(-step.token_capacity // 256)       # (joining costs by the token)
-        return max(1, min(compute_units(device) // (tiles * self.heads), step.context_limit // (64 * blocks), 8))
+        return max(1, min(compute_units(device) // (tiles * self.q_heads), step.context_limit // (64 * blocks), 8))
 
     def forward(self, h, step, memory, stream):
         tokens = h.shape[0]

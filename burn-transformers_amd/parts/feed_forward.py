@@ -66,6 +66,9 @@ class DenseFeedForward(FeedForward):
         # whether the up projection may run inside another part's first product (Mixer.carry)
         self.can_ride = self.activation in K.ACTIVATIONS and self.up_bias is None
 
+    def kernel_modules(self, dtype):
+        return ("sublayer",) if self.activation in ("poly_norm", "squared_relu") else ()
+
     def ride(self, up_weight):
         """The up projection as a view of the matrix that small steps multiply by in the other part's product."""
         self.up_weight, self.up_packed = up_weight, None
@@ -96,7 +99,11 @@ class DenseFeedForward(FeedForward):
             return
         if hidden is None:
             hidden = self.hidden_rows(step, tokens)
-            K.gemm(h, self.up_weight, K.epilogue_act(hidden, self.activation, self.up_bias), packed=self.up_packed)
+            if K.activation_needs_a_pass(h, self.up_weight, self.activation):
+                K.gemm(h, self.up_weight, K.epilogue_store(hidden, self.up_bias))
+                K.activate(hidden, self.activation)
+            else:
+                K.gemm(h, self.up_weight, K.epilogue_act(hidden, self.activation, self.up_bias), packed=self.up_packed)
         if self.joined is None:
             stream.add_product(step, hidden, self.down_weight, self.down_bias, packed=self.down_packed)
 

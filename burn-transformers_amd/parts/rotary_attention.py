@@ -251,11 +251,13 @@ class RotaryAttention(CausalSelfAttention):
 
     def run_attention(self, q, out, gate, kv, step):
         plain, partial = self.runs_plain(step), None
-        runs = 1 if plain else self.decode_runs(step, q.device)
+        runs, prompt_runs = (1, 1) if plain else (self.decode_runs(step, q.device), self.prompt_runs(step, q.device))
         if runs > 1:
             partial = step.buffer("attention.partial", step.n_seqs * self.q_heads * runs, self.head_dim + 2, "float32")
+        elif prompt_runs > 1:
+            partial = step.buffer("attention.partial", q.shape[0] * self.q_heads * prompt_runs, self.head_dim + 2, "float32")
         args = K.attention_args(q, out, kv, step.tok_seq, step.tok_pos, step.seq_off, step.seq_start,
                                 self.q_heads, step.n_seqs, step.max_count, self.scale, self.window, partial,
-                                chunk=self.chunk, sink=self.sink, softcap=self.softcap, sigmoid=self.sigmoid,
+                                runs=prompt_runs if prompt_runs > 1 else None, chunk=self.chunk, sink=self.sink, softcap=self.softcap, sigmoid=self.sigmoid,
                                 score_bias=self.score_bias, gate=gate, gate_dim=self.vdim if self.gate_kind == "channel" else 0)
         K.attention(args, step.dtype, step.decode, impl="plain" if plain else "auto")

@@ -239,6 +239,12 @@ def test_decoding_far_out_in_runs_of_keys(kind, dtype):
     slot = engine.open()
     first = engine.step([(slot, ids[:2395])], want=[[0, 1023, 1024, 2099, 2394]]).clone()
     check(first, want[[0, 1023, 1024, 2099, 2394]], dtype, f"{kind} prompt")
+    engine.close(slot)
+    slot = engine.open()                   # the same in portions: those behind 1,024 tokens cut their keys into runs too
+    for begin, end in ((0, 1500), (1500, 1630), (1630, 1640), (1640, 2200), (2200, 2395)):
+        places = [0, (end - begin) // 2, end - begin - 1]
+        part = engine.step([(slot, ids[begin:end])], want=[places]).clone()
+        check(part, want[[begin + p for p in places]], dtype, f"{kind} portion {begin} to {end}")
     rows = torch.cat([engine.step([(slot, [token])]).clone() for token in ids[2395:]])
     check(rows, want[2395:], dtype, f"{kind} decoded behind 2,395 tokens")
     engine.close(slot)

@@ -105,21 +105,53 @@ def test_32_bit_rows_of_bfloat16_attention(form, hd):
     run_case("bfloat16", form, None, [40], [40], 2, 1, hd, impl="plain", f32_out=True, seed=hd)
 
 
-def test_chunks_of_prompts_in_runs_of_heads_of_64():
-    """The prompt kernel of heads of 64 with its keys in runs (joined by a second kernel), all forms."""
-    for form in ("softmax", "capped", "sigmoid"):
-        case = PagedCase([900], [130], 2, 64, torch.bfloat16, DEV, seed=3, poison=True)
+@pytest.mark.parametrize("hd", [64, 80, 96, 112, 128])
+def test_chunks_of_prompts_in_runs(hd):
+    """The prompt kernels of heads of 64 to 128 with their keys in runs (joined by a second kernel), some of them empty for
+    the early tiles and the short sequence, all forms; a gate whose rows take 16-byte loads and one whose rows do not."""
+    for number, form in enumerate(("softmax", "capped", "sigmoid")):
+        counts, totals, runs = [130, 40], [900, 40], 5
+        case = PagedCase(totals, counts, 2, hd, torch.bfloat16, DEV, seed=3, poison=True)
         gen = torch.Generator().manual_seed(1)
-        q = (torch.randn(130, 4 * 64, generator=gen) * 0.6).to(torch.bfloat16)
-        gate = torch.randn(130, 4 * 64, generator=gen)
+        tokens = sum(counts)
+        q = (torch.randn(tokens, 4 * hd, generator=gen) * 0.6).to(torch.bfloat16)
+        gate = torch.randn(tokens, 4 * hd + number, generator=gen)
         bias = torch.randn(4, generator=gen) - 2.0 if form == "sigmoid" else None
-        out = torch.full((130, 256), float("nan"), dtype=torch.bfloat16, device=DEV)
-        partial = torch.full((130 * 4 * 3, 66), float("nan"), device=DEV)
-        args = K.attention_args(q.to(DEV), out, case.view(), case.tok_seq, case.tok_pos, case.seq_off, case.seq_start, 4, 1, 130, 0.125, 0,
-                                partial, runs=3, softcap=4.0 if form == "capped" else 0.0, sigmoid=form == "sigmoid",
-                                score_bias=bias.to(DEV) if bias is not None else None, gate=gate.to(DEV), gate_dim=64)
+        out = torch.full((tokens, 4 * hd), float("nan"), dtype=torch.bfloat16, device=DEV)
+        partial = torch.full((tokens * 4 * runs, hd + 2), float("nan"), device=DEV)
+        args = K.attention_args(q.to(DEV), out, case.view(), case.tok_seq, case.tok_pos, case.seq_off, case.seq_start, 4, 2, 130, 0.125, 0,
+                                partial, runs=runs, softcap=4.0 if form == "capped" else 0.0, sigmoid=form == "sigmoid",
+                                score_bias=bias.to(DEV) if bias is not None else None, gate=gate.to(DEV), gate_dim=hd)
         K.attention(args, torch.bfloat16, False)
-        assert rel_err(out, reference(case, q, 4, 0.125, form, 4.0, bias, gate, 64)) < 1.5e-2, form
+        assert rel_err(out, reference(case, q, 4, 0.125, form, 4.0, bias, gate, hd)) < 1.5e-2, form
+
+
+@pytest.mark.parametrize("hd", [80, 96, 112, 128])
+@pytest.mark.parametrize("window,chunk", [(0, 0), (70, 0), (1, 0), (200, 0), (0, 50), (0, 128), (90, 100)])
+def test_prompts_of_wide_heads_with_windows_and_chunks(hd, window, chunk):
+    """The prompt kernel of heads of 80 to 128: windows and chunks that begin inside blocks, at their borders and blocks
+    apart; prompts and chunks of prompts of unequal sequences, one cached head for many query heads, many units."""
+    for q_heads, kv_heads, totals, counts in ((4, 1, [300, 5], [300, 5]), (6, 2, [500, 129, 64, 1, 260], [140, 129, 64, 1, 2])):
+        case = PagedCase(totals, counts, kv_heads, hd, torch.bfloat16, DEV, seed=hd, poison=True)
+        gen = torch.Generator().manual_seed(window + chunk)
+        q = (torch.randn(case.n_tokens, q_heads * hd, generator=gen) * 0.6).to(torch.bfloat16)
+        out = torch.full((case.n_tokens, q_heads * hd), float("nan"), dtype=torch.bfloat16, device=DEV)
+        args = K.attention_args(q.to(DEV), out, case.view(), case.tok_seq, case.tok_pos, case.seq_off, case.seq_start, q_heads,
+                                len(totals), max(counts), 1.0 / math.sqrt(hd), window, chunk=chunk)
+        K.attention(args, torch.bfloat16, False)
+        want = torch.zeros(case.n_tokens, q_heads, hd, dtype=F64)
+        row = 0
+        for s, (total, count) in enumerate(zip(totals, counts)):
+            k = case.k_rows[s].double().view(total, kv_heads, hd)
+            v = case.v_rows[s].double().view(total, kv_heads, hd)
+            for pos in range(total - count, total):
+                lo = max(pos - window + 1 if window else 0, pos - pos % chunk if chunk else 0, 0)
+                for h in range(q_heads):
+                    j = h // (q_heads // kv_heads)
+                    scores = (k[lo:pos + 1, j] @ q[row, h * hd:(h + 1) * hd].double()) / math.sqrt(hd)
+                    want[row, h] = torch.softmax(scores, 0) @ v[lo:pos + 1, j]
+                row += 1
+        assert rel_err(out, want.reshape(case.n_tokens, -1)) < 1.5e-2, (q_heads, totals, counts)
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
