@@ -996,7 +996,11 @@ static int launch_skinny_norm(hipStream_t s, const NormOperand& norm, const bf16
   size_t lds = (size_t)16 * (K * 2 + 16);
 #define LAUNCH_NORM(NT, QPL)                                                                                   \
   do {                                                                                                         \
-    auto kernel = gemm_skinny_kernel<bf16_t, 1, NT, 8, 8, QPL>;                                                \
+    if (epi.mode == EPI_F32_ACT) LAUNCH_NORM_FORM(NT, QPL, true); else LAUNCH_NORM_FORM(NT, QPL, false);       \
+  } while (0)
+#define LAUNCH_NORM_FORM(NT, QPL, TWO)                                                                         \
+  do {                                                                                                         \
+    auto kernel = gemm_skinny_kernel<bf16_t, 1, NT, 8, 8, QPL, false, TWO>;                                                \
     static size_t granted = 0;    /* statically allocated LDS comes on top: ask for room beyond the default */ \
     if (lds > granted) {                                                                                       \
       hipError_t err = hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); \
@@ -1011,6 +1015,7 @@ static int launch_skinny_norm(hipStream_t s, const NormOperand& norm, const bf16
     if (columns <= 16) LAUNCH_NORM(1, 8); else LAUNCH_NORM(2, 8);
   }
 #undef LAUNCH_NORM
+#undef LAUNCH_NORM_FORM
   return BT_OK;
 }
 
@@ -1028,8 +1033,6 @@ BT_EXPORT int bt_gemm_skinny(void* stream, int dtype, const void* A, int64_t lda
   if (a_rows != 0 && (norm != nullptr || a_rows < M))
     BT_REFUSE("gemm_skinny: chunk-major activations of %d rows for a product of %d rows%s", a_rows, M,
               norm != nullptr ? " that normalises its rows itself" : "");
-  if (norm != nullptr && epi->mode == EPI_F32_ACT)
-    BT_REFUSE("gemm_skinny: 32-bit and activated columns of one product come from rows that are normalised already");
   if (norm != nullptr) {
     if (dtype != 1 || M > 16 || K > 2048)
       BT_REFUSE("gemm_skinny: the fused norm takes bfloat16 weights, up to 16 rows and K up to 2048 (got %d rows, K %d)", M, K);

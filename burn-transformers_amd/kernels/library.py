@@ -800,7 +800,7 @@ def takes_two_kinds(a):
     the skinny kernel's steps."""
     if a.shape[0] > 64:
         return False
-    return a.dtype == torch.bfloat16 or (a.shape[1] % 4 == 0 and a.stride(0) % 4 == 0)
+    return isinstance(a, Normalized) or a.dtype == torch.bfloat16 or (a.shape[1] % 4 == 0 and a.stride(0) % 4 == 0)
 
 
 def gemm(a, w, epilogue, splits=1, impl="auto", variant=0, packed=None):

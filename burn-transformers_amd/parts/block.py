@@ -30,6 +30,11 @@ from .registry import register
 # With the limit at eight rows instead, ms a step of eight rows at widths 768 / 1,024 / 1,600 (12, 24
 # and 12 layers): 0.395 -> 0.388, 0.781 -> 0.785, 0.531 -> 0.546; so four at every width.
 MIXER_FOLD_ROWS = 4
+# ... and in a parallel block the widest stream: its one output product is long (mixer and feed-forward together), and
+# without its split of K it loses more than the norm costs where the matrix is large.  Measured as ms a decode step of 12
+# layers without / with the fold at 1, 2, 4, 8 rows: width 1,024 0.363 / 0.359, 0.378 / 0.361, 0.386 / 0.377, 0.389 / 0.392;
+# width 2,048 0.532 / 0.541, 0.539 / 0.556, 0.543 / 0.566, 0.549 / 0.613.
+PARALLEL_FOLD_WIDTH = 1024
 
 
 @register("block", "pre_norm")
@@ -205,8 +210,12 @@ class ParallelBlock(Block):
             if delta is not None:
                 stream.add(delta)
             return
-        # both parts hand the rows to products only: a small step's rows may be chunk-major
-        h = _apply(norm, stream, step, self.carries or (mixer.takes_deferred_norm and ff.takes_deferred_norm))
+        # In the smallest steps the norm is folded into the one product that both parts' first projections are, if the
+        # layer before left its sum in the stream itself (see PreNormBlock).
+        fold = self.carries and rows <= MIXER_FOLD_ROWS and stream.x.shape[1] <= PARALLEL_FOLD_WIDTH and _can_defer(norm, step, rows)
+        h = norm.deferred(stream, step) if fold else None
+        if h is None:         # both parts hand the rows to products only: a small step's rows may be chunk-major
+            h = _apply(norm, stream, step, self.carries or (mixer.takes_deferred_norm and ff.takes_deferred_norm))
         if self.output is not None:
             self.output.begin(step, rows)
         extra = {}
@@ -217,7 +226,9 @@ class ParallelBlock(Block):
             if delta is not None:
                 stream.add(delta)
         if self.output is not None:
+            stream.in_place = fold            # for the next layer's norm
             self.output.add_to(stream, step)
+            stream.in_place = False
 
 
 @register("block", "transform")

@@ -292,6 +292,21 @@ def test_a_product_with_32_bit_and_activated_columns(dtype, m, n, sums, k):
     assert torch.equal(again, first) and torch.equal(chunked.to_rows()[:, :n - sums], act[:, :n - sums])
 
 
+@pytest.mark.parametrize("m", [1, 4, 11])
+def test_a_product_of_two_kinds_that_normalises_its_rows_itself(m):
+    gen = torch.Generator().manual_seed(m)
+    k, n, sums, eps = 72, 130, 68, 1e-4
+    x, gamma = torch.randn(m, k, generator=gen), torch.randn(k, generator=gen)
+    w = (torch.randn(n, k, generator=gen) / 8).to(torch.bfloat16)
+    want = (plain.unit_rms(x.double(), eps) * gamma.double()).to(torch.bfloat16).double() @ w.double().T
+    first, act = torch.zeros(m, sums, device=DEV), torch.zeros(m, 64, dtype=torch.bfloat16, device=DEV)
+    rows = K.Normalized(x.to(DEV), gamma.to(DEV), None, eps, "rms_norm")
+    assert K.takes_two_kinds(rows)
+    K.gemm(rows, w.to(DEV), K.epilogue_f32_act(first, sums, act, "squared_relu"))
+    assert rel_err(first, want[:, :sums]) < 5e-3
+    assert rel_err(act[:, :n - sums], plain.squared_relu(want[:, sums:])) < 1.5e-2
+
+
 @pytest.mark.parametrize("impl,m", [("plain", 70), ("tile", 70), ("tile", 300), ("skinny", 20)])
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 def test_the_square_of_relu_in_every_product(dtype, impl, m):
