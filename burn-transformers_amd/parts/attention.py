@@ -57,7 +57,6 @@ class CausalSelfAttention(Mixer):
             raise ValueError(f"attention: head size {self.head_dim} must be positive")
         if self.heads % self.kv_heads != 0:
             raise ValueError(f"attention: {self.heads} query heads cannot share {self.kv_heads} key/value heads")
-        self.q_heads = self.heads                         # queries the attention kernels see
         self.n_q, self.n_kv = self.heads * self.head_dim, self.kv_heads * self.head_dim
         self.qkv_weight, self.qkv_bias = tensors["qkv_weight"], tensors.get("qkv_bias")
         self.out_weight, self.out_bias = tensors["out_weight"], tensors.get("out_bias")
@@ -111,11 +110,11 @@ class CausalSelfAttention(Mixer):
         pairs = step.n_seqs * self.kv_heads
         return max(1, min(compute_units(device) // pairs, pair_bytes // RUN_BYTES, 64))
 
-    def prompt_runs(self, step, device):
+    def prompt_runs(self, step, device, q_heads=None):
         """Into how many runs a prompt step's query tiles cut their keys: a chunk of a prompt behind
         a long context has few tiles of 128 queries (a work-group each) and many keys for each, so
         the keys are shared out until the work-groups fill the chip, a run keeping at least
-        ``PROMPT_RUN_BLOCKS`` blocks of keys.  Planned from what the steps that share a launch list
+        ``PROMPT_RUN_BLOCKS`` blocks of keys (``q_heads``: queries a token brings, where they are not the heads).  Planned from what the steps that share a launch list
         have in common (most tokens, sequences, the class of context), like ``decode_runs``.
         Measured at 25 heads of 64, a chunk of 256 tokens, us a call with 1 / 2 / 4 / 5 runs: behind
         1,024 tokens 16.6 / 16.9 / 17.3 / 18.0, 2,048: 25.9 / 21.9 / 20.4 / 20.8, 4,096: 45.7 / 31.9 /
@@ -127,7 +126,7 @@ class CausalSelfAttention(Mixer):
             return 1
         tiles = -(-step.token_capacity // 128) + step.n_seqs - 1          # at most so many hold queries
         blocks = PROMPT_RUN_BLOCKS * -(-step.token_capacity // 256)       # (joining costs by the token)
-        return max(1, min(compute_units(device) // (tiles * self.q_heads), step.context_limit // (64 * blocks), 8))
+        return max(1, min(compute_units(device) // (tiles * (q_heads or self.heads)), step.context_limit // (64 * blocks), 8))
 
     def forward(self, h, step, memory, stream):
         tokens = h.shape[0]

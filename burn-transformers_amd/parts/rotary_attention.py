@@ -251,7 +251,7 @@ class RotaryAttention(CausalSelfAttention):
 
     def run_attention(self, q, out, gate, kv, step):
         plain, partial = self.runs_plain(step), None
-        runs, prompt_runs = (1, 1) if plain else (self.decode_runs(step, q.device), self.prompt_runs(step, q.device))
+        runs, prompt_runs = (1, 1) if plain else (self.decode_runs(step, q.device), self.prompt_runs(step, q.device, self.q_heads))
         if runs > 1:
             partial = step.buffer("attention.partial", step.n_seqs * self.q_heads * runs, self.head_dim + 2, "float32")
         elif prompt_runs > 1:

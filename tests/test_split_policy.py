@@ -75,7 +75,7 @@ def test_prompt_runs_for_chunks_behind_long_contexts(monkeypatch):
     """A chunk of a prompt has few tiles of 128 queries: their keys are cut into runs until the
     work-groups fill the chip, each run at least 8 blocks of keys per 256 tokens of the step, none
     while the class of context is 1,024 tokens or less, and only where the kernel that takes runs
-    is the one that runs (bfloat16, heads of 64, no window)."""
+    is the one that runs (bfloat16, heads of 64 to 128, no window)."""
     assert _prompt_runs(monkeypatch, 256, 1, 1024) == 1
     assert _prompt_runs(monkeypatch, 256, 1, 2048) == 4            # 32 blocks in runs of 8
     assert _prompt_runs(monkeypatch, 256, 1, 4096) == 5            # 2 tiles x 25 heads x 5 = 250 work-groups
@@ -87,6 +87,8 @@ def test_prompt_runs_for_chunks_behind_long_contexts(monkeypatch):
     assert _prompt_runs(monkeypatch, 2048, 1, 8192) == 1           # 16 tiles x 25 heads fill the chip already
     assert _prompt_runs(monkeypatch, 256, 1, 8192, bf16=False) == 1
     assert _prompt_runs(monkeypatch, 256, 1, 8192, head_dim=32) == 1
+    assert _prompt_runs(monkeypatch, 256, 1, 8192, head_dim=128) == 5
+    assert _prompt_runs(monkeypatch, 256, 1, 8192, head_dim=144) == 1
     assert _prompt_runs(monkeypatch, 256, 1, 8192, window=512) == 1
     assert _prompt_runs(monkeypatch, 256, 1, 8192, chunk=512) == 1
     assert _prompt_runs(monkeypatch, 256, 1, 8192, heads=4) == 8   # few heads: the runs are what fills the chip
