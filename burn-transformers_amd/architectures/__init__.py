@@ -1,4 +1,4 @@
 """Importing this package registers the architectures the library ships (GPT-2, Salopel, Kodatar, Rotutar, Gavasun,
-Loselix)."""
+Loselix, Rirovik)."""
 
-from . import gavasun, gpt2, kodatar, loselix, rotutar, salopel  # noqa: F401
+from . import gavasun, gpt2, kodatar, loselix, rirovik, rotutar, salopel  # noqa: F401

@@ -60,9 +60,11 @@ class CacheLedger:
     sequence has grown past them, and their places in the sequence's list read RELEASED.
     ``chunks[g]`` > 0 says that a token of group g reads only the positions of its own chunk of that
     many positions (chunks are counted from position 0): the blocks that lie wholly before the chunk
-    of the next token go back the same way."""
+    of the next token go back the same way.
+    ``keeps[g]`` > 0 says that group g reads the first ``keeps[g]`` positions of a sequence as long as it lives: their
+    blocks stay."""
 
-    def __init__(self, n_groups, blocks_per_group, max_slots, max_blocks_per_sequence, windows=None, chunks=None):
+    def __init__(self, n_groups, blocks_per_group, max_slots, max_blocks_per_sequence, windows=None, chunks=None, keeps=None):
         self.n_groups = n_groups
         self.max_blocks_per_sequence = max_blocks_per_sequence
         self.windows = list(windows) if windows is not None else [0] * n_groups
@@ -71,6 +73,9 @@ class CacheLedger:
         self.chunks = list(chunks) if chunks is not None else [0] * n_groups
         if len(self.chunks) != n_groups or any(c < 0 for c in self.chunks):
             raise ValueError(f"{n_groups} groups need {n_groups} chunk sizes that are not negative, got {self.chunks}")
+        self.keeps = list(keeps) if keeps is not None else [0] * n_groups
+        if len(self.keeps) != n_groups or any(k < 0 for k in self.keeps):
+            raise ValueError(f"{n_groups} groups need {n_groups} numbers of kept positions that are not negative, got {self.keeps}")
         self.slots = FreeList(max_slots)
         self.blocks = [FreeList(blocks_per_group) for _ in range(n_groups)]
         self.lengths = [0] * max_slots
@@ -107,7 +112,7 @@ class CacheLedger:
 
     def first_kept(self, group, length):
         """Number of the first block of a sequence of ``length`` tokens that group ``group`` still
-        needs: the next token (position ``length``) reads back to position length - window + 1, and
+        needs, the blocks of kept first positions aside: the next token (position ``length``) reads back to position length - window + 1, and
         not beyond the first position of its chunk."""
         window, chunk = self.windows[group], self.chunks[group]
         first = max(0, length - window + 1) if window > 0 else 0
@@ -184,7 +189,7 @@ class CacheLedger:
             if self.windows[group] <= 0 and self.chunks[group] <= 0:
                 continue
             held = self.held_blocks[group][slot]
-            for index in range(min(self.first_kept(group, length), len(held))):
+            for index in range(self.blocks_for(self.keeps[group]), min(self.first_kept(group, length), len(held))):
                 if held[index] != RELEASED:
                     self.blocks[group].give(held[index])
                     held[index] = RELEASED
@@ -205,6 +210,8 @@ class CacheLedger:
                 assert len(held) >= needed, f"slot {slot} is longer than its blocks"
                 assert RELEASED not in held[self.first_kept(group, self.lengths[slot]):], \
                     f"slot {slot} has given back a block of group {group} that it still reads"
+                assert RELEASED not in held[:self.blocks_for(self.keeps[group])], \
+                    f"slot {slot} has given back a block of group {group} with kept first positions"
                 for block in held:
                     if block == RELEASED:
                         continue

@@ -25,11 +25,20 @@ class KVSpec:
     """What a mixer keeps per token: heads and head size; ``window`` > 0 means that only the last
     ``window`` positions are ever read; ``chunk`` > 0 that a token reads only the positions of its own
     chunk of that many (counted from position 0), so that everything before the chunk the next token
-    falls into is never read again."""
+    falls into is never read again.  The first ``keep`` positions are read whatever these two say."""
     kv_heads: int
     head_dim: int
     window: int = 0
     chunk: int = 0
+    keep: int = 0
+
+    def joined(self, other):
+        """What an entry has to keep whose keys and values mixers with this spec and with ``other`` both read."""
+        if (self.kv_heads, self.head_dim) != (other.kv_heads, other.head_dim):
+            raise ValueError(f"{self.kv_heads} heads of {self.head_dim} and {other.kv_heads} of {other.head_dim} cannot share a cache entry")
+        window = max(self.window, other.window) if self.window and other.window else 0
+        chunk = self.chunk if self.chunk == other.chunk else 0
+        return KVSpec(self.kv_heads, self.head_dim, window, chunk, max(self.keep, other.keep) if window or chunk else 0)
 
 
 @dataclass(frozen=True)
@@ -109,7 +118,8 @@ class Cache:
             self.state_groups.append(group)
         self.ledger = CacheLedger(len(self.kv_groups), n_blocks, self.max_slots, self.max_blocks,
                                   windows=[group.spec.window for group in self.kv_groups],
-                                  chunks=[group.spec.chunk for group in self.kv_groups])
+                                  chunks=[group.spec.chunk for group in self.kv_groups],
+                                  keeps=[group.spec.keep for group in self.kv_groups])
 
     # --- slots -----------------------------------------------------------------------------
     def acquire(self):
@@ -139,7 +149,7 @@ class Cache:
     def block_rows(self, slots):
         """For a step's block tables: [group][sequence] -> block list, a released block's place
         filled with block 0 (a valid block that no kernel reads for this sequence: a query's keys
-        start inside its window)."""
+        start inside its window, but for kept first tokens, whose blocks are not released)."""
         return [[[block if block >= 0 else 0 for block in self.ledger.held_blocks[group][slot]] for slot in slots]
                 for group in range(len(self.kv_groups))]
 

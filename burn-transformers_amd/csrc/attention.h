@@ -53,6 +53,8 @@ struct AttnArgs {
   int gate_span;
   int gate_dim;
   int out_f32;
+  // The first `keep` positions of a sequence are seen by every later query of it, whatever window and chunk say.
+  int keep;
 };
 
 // What a sink adds to a softmax's denominator that is kept relative to the maximum `top`.  The plain and
@@ -88,11 +90,44 @@ inline const char* bt_check_form(const AttnArgs& a) {
   return nullptr;
 }
 
-// The first position a query at `pos` sees: the later of its window's and its chunk's first key.
-// It never decreases as `pos` grows, so the first query of a run of queries has the lowest.
+// The first position a query at `pos` sees: the later of its window's and its chunk's first key (kept first
+// positions aside).  It never decreases as `pos` grows, so the first query of a run of queries has the lowest.
 __host__ __device__ __forceinline__ int bt_first_seen(int pos, int window, int chunk) {
   int lo = 0;
   if (window > 0 && pos - window + 1 > lo) lo = pos - window + 1;
   if (chunk > 0 && pos - pos % chunk > lo) lo = pos - pos % chunk;
   return lo;
+}
+
+// The positions that queries whose first key is `from` or later walk, as one range 0 .. without a gap: the kept first
+// positions (in whole tiles), then everything from `from` on.  With nothing kept the range starts at `from`.
+struct KeyWalk {
+  int kept, skip;
+  // the position at place v of the range
+  __device__ __forceinline__ int at(int v) const { return v < kept ? v : v + skip; }
+  // the place that stands for position `end` (one past the last key, beyond `from`)
+  __device__ __forceinline__ int places(int end) const { return end - skip; }
+};
+// `from` is a multiple of `tile` (a power of two).
+__device__ __forceinline__ KeyWalk bt_key_walk(int from, int keep, int tile) {
+  KeyWalk walk;
+  const int whole = (keep + tile - 1) & ~(tile - 1);
+  walk.kept = whole < from ? whole : from;
+  walk.skip = from - walk.kept;
+  return walk;
+}
+
+// Which keys a query sees, for a test of two comparisons: those from `lo` through its own position, and those below `kept`.
+struct SeenKeys {
+  int lo, kept;
+  unsigned span;
+  __device__ __forceinline__ bool operator()(int key) const { return (unsigned)(key - lo) <= span || key < kept; }
+};
+// A column without a query (pos < 0) sees nothing.
+__device__ __forceinline__ SeenKeys bt_seen_keys(int pos, int first_seen, int keep) {
+  SeenKeys seen;
+  seen.lo = pos < 0 ? 1 << 30 : first_seen;
+  seen.span = (unsigned)(pos - seen.lo);
+  seen.kept = keep < pos + 1 ? keep : pos + 1;
+  return seen;
 }

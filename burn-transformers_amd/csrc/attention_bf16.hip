@@ -206,7 +206,8 @@ __device__ __forceinline__ float raise_maximum(float& m, float top, float& alpha
 
 // One tile of 32 keys starting at position kb against NQ tiles of 16 queries.
 //   qpos[nq]: position of the query in column lane % 16 of tile nq, -1 if there is none.
-//   qlo[nq]: the first position that query sees (its window's or its chunk's first key, else 0).
+//   qlo[nq]: the first position that query sees (its window's or its chunk's first key, else 0); it also sees the
+//   positions below `keep`.
 //   valid_end: positions >= valid_end hold no token (their values are replaced by zero).
 //   sc: what makes exponents of the dot products (form 0: one positive factor); m[] is kept in those units
 //   (powers of two).
@@ -215,7 +216,7 @@ __device__ __forceinline__ float raise_maximum(float& m, float top, float& alpha
 //   a query then hold numbers nobody reads.
 template <int NQ, bool MASKED>
 __device__ __forceinline__ void attend_tile(const TileOperands& tile, int kb, int valid_end,
-                                            const int (&qpos)[NQ], const int (&qlo)[NQ], const Scoring& sc,
+                                            const int (&qpos)[NQ], const int (&qlo)[NQ], int keep, const Scoring& sc,
                                             const bf16x8 (&q)[NQ][NKS], floatx4 (&o)[NQ][ND],
                                             float (&m)[NQ], float (&l)[NQ]) {
   const int lane = threadIdx.x & 63, g = lane >> 4;
@@ -244,15 +245,11 @@ __device__ __forceinline__ void attend_tile(const TileOperands& tile, int kb, in
 #pragma unroll
   for (int nq = 0; nq < NQ; ++nq) {
     if (MASKED) {
-      const int qp = qpos[nq], ql = qlo[nq];
+      const SeenKeys seen = bt_seen_keys(qpos[nq], qlo[nq], keep);
 #pragma unroll
       for (int t = 0; t < 2; ++t)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          int kp = kb + 16 * t + 4 * g + r;
-          bool seen = kp <= qp && kp >= ql;
-          s[nq][t][r] = seen ? s[nq][t][r] : -INFINITY;
-        }
+        for (int r = 0; r < 4; ++r) s[nq][t][r] = seen(kb + 16 * t + 4 * g + r) ? s[nq][t][r] : -INFINITY;
     }
     if constexpr (FORM == 2) continue;          // weights that no other key has a part in
     const float m_use = m[nq] == -INFINITY ? 0.f : m[nq];
@@ -400,7 +397,9 @@ attention_prefill_kernel(AttnArgs a) {
   }
   const int last = q0 + PREFILL_QUERIES_PER_WAVE < count ? q0 + PREFILL_QUERIES_PER_WAVE : count;
   const int hi = start + last;  // one past the position of this wave's last query
-  const int lo = bt_first_seen(start + q0, a.window, a.chunk) & ~31;      // (the wave's first query sees furthest back)
+  // (the wave's first query sees furthest back)
+  const KeyWalk walk = bt_key_walk(bt_first_seen(start + q0, a.window, a.chunk) & ~31, a.keep, 32);
+  const int places = walk.places(hi);
   const int valid_end = start + count;
   const bf16_t* keys = static_cast<const bf16_t*>(a.kv.keys);
   const bf16_t* values = static_cast<const bf16_t*>(a.kv.values);
@@ -412,25 +411,26 @@ attention_prefill_kernel(AttnArgs a) {
   // A fetch beyond the last tile reads the first one again instead of being skipped: with the same
   // number of loads in flight on every path, the wait before a tile is for that tile only.
   TileOperands t0, t1;
-  auto fetch = [&](TileOperands& into, int kb) {
-    const int kf = kb < hi ? kb : lo;
+  auto fetch = [&](TileOperands& into, int place) {
+    const int kf = walk.at(place < places ? place : 0);
     int64_t plane = tile_plane(a, seq, kv_head, kf);
     load_tile(into, keys + plane, values + plane, kf);
   };
-  auto attend = [&](const TileOperands& tile, int kb) {
+  auto attend = [&](const TileOperands& tile, int place) {
+    const int kb = walk.at(place);
     if (kb + 32 <= whole_until)
-      attend_tile<PREFILL_NQ, false>(tile, kb, valid_end, qpos, qlo, sc, q, o, m, l);
+      attend_tile<PREFILL_NQ, false>(tile, kb, valid_end, qpos, qlo, a.keep, sc, q, o, m, l);
     else
-      attend_tile<PREFILL_NQ, true>(tile, kb, valid_end, qpos, qlo, sc, q, o, m, l);
+      attend_tile<PREFILL_NQ, true>(tile, kb, valid_end, qpos, qlo, a.keep, sc, q, o, m, l);
   };
-  if (lo >= hi) return;   // (cannot happen: a wave with a query sees at least that query's key)
-  fetch(t0, lo);
-  fetch(t1, lo + 32);
-  for (int kb = lo; kb < hi; kb += 64) {
-    attend(t0, kb);
-    fetch(t0, kb + 64);
-    if (kb + 32 < hi) attend(t1, kb + 32);
-    fetch(t1, kb + 96);
+  if (places <= 0) return;   // (cannot happen: a wave with a query sees at least that query's key)
+  fetch(t0, 0);
+  fetch(t1, 32);
+  for (int place = 0; place < places; place += 64) {
+    attend(t0, place);
+    fetch(t0, place + 64);
+    if (place + 32 < places) attend(t1, place + 32);
+    fetch(t1, place + 96);
   }
 #pragma unroll
   for (int nq = 0; nq < PREFILL_NQ; ++nq) {
@@ -463,7 +463,7 @@ attention_prefill_kernel(AttnArgs a) {
 //   excluded scores, so the compiler keeps every running sum in one place.
 //   `Operands` hands out the block's operands: k(t, ks) keys 16 t .. + 15 and channels 32 ks .. + 31,
 //   v(dt, half) channels 16 dt .. + 15 and positions 32 half .. + 31.  BOUNDED: a query may also have a
-//   first key that it sees (qlo).  RAGGED: positions from valid_end on may lie in the block.
+//   first key that it sees (qlo) beside the positions below `keep`.  RAGGED: positions from valid_end on may lie in the block.
 struct BlockOperands {
   bf16x8 keys[4][NKS];
   bf16x8 values[ND][2];   // [block of 16 channels][half of the block's positions]: see SHARED_V_BYTES
@@ -473,7 +473,7 @@ struct BlockOperands {
 
 template <int NQ, bool BOUNDED, bool RAGGED, typename Operands>
 __device__ __forceinline__ void attend_block(const Operands& blk, int kb, int valid_end, bool masked,
-                                             const int (&qpos)[NQ], const int (&qlo)[NQ], const Scoring& sc,
+                                             const int (&qpos)[NQ], const int (&qlo)[NQ], int keep, const Scoring& sc,
                                              const bf16x8 (&q)[NQ][NKS], floatx4 (&o)[NQ][ND], float (&m)[NQ],
                                              floatx4 (&rows)[NQ]) {
   const int lane = threadIdx.x & 63, g = lane >> 4;
@@ -504,12 +504,13 @@ __device__ __forceinline__ void attend_block(const Operands& blk, int kb, int va
 #pragma unroll
     for (int nq = 0; nq < NQ; ++nq) {
       const int qp = qpos[nq];
+      const SeenKeys seen = bt_seen_keys(qp, qlo[nq], keep);
 #pragma unroll
       for (int t = 0; t < 4; ++t)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int kp = kb + 16 * t + 4 * g + r;
-          s[nq][t][r] = kp <= qp && (!BOUNDED || kp >= qlo[nq]) ? s[nq][t][r] : -INFINITY;
+          s[nq][t][r] = (BOUNDED ? seen(kp) : kp <= qp) ? s[nq][t][r] : -INFINITY;
         }
     }
   }
@@ -868,7 +869,7 @@ attention_prefill_split_kernel(AttnArgs a) {
         for (int half = 0; half < 2; ++half)
           blk.values[dt][half] = *reinterpret_cast<const bf16x8*>(stage + SHARED_K_BYTES +
                                                              ((4 * half + g) * 64 + dt * 16 + i16) * 16);
-      attend_block<PREFILL_NQ, false, true>(blk, kb, valid_end, kb + 64 > whole_until, qpos, qpos, sc, q, o, m, rows);
+      attend_block<PREFILL_NQ, false, true>(blk, kb, valid_end, kb + 64 > whole_until, qpos, qpos, 0, sc, q, o, m, rows);
     }
     __syncthreads();   // turn t + 1 is in place, and everyone is done with turn t before it is overwritten
   }
@@ -951,7 +952,9 @@ attention_prefill_wide_kernel(AttnArgs a) {
   const int reach = (q_tile + 1) * PREFILL_QUERIES < count ? (q_tile + 1) * PREFILL_QUERIES : count;
   const int first_block = bt_first_seen(start + q_tile * PREFILL_QUERIES, a.window, a.chunk) / BT_KV_BLOCK;
   const int last_block = (start + reach - 1) / BT_KV_BLOCK;
-  const int n_turns = (last_block - first_block + 2) / 2;
+  const KeyWalk walk = bt_key_walk(first_block, (a.keep + BT_KV_BLOCK - 1) / BT_KV_BLOCK, 1);      // (in blocks)
+  const int last_place = walk.places(last_block);
+  const int n_turns = (last_place + 2) / 2;
   const int per_run = (n_turns + runs - 1) / runs;
   const int t_begin = run * per_run;
   const int t_end = t_begin + per_run < n_turns ? t_begin + per_run : n_turns;
@@ -969,8 +972,8 @@ attention_prefill_wide_kernel(AttnArgs a) {
   const unsigned char* planes = static_cast<const unsigned char*>(bring_values ? a.kv.values : a.kv.keys);
   const int* block_row = a.kv.blocks + (int64_t)seq * a.kv.max_blocks;
   auto block_of = [&](int turn) {                           // where the wave's block of a turn lies
-    const int block = first_block + 2 * turn + bring_block;
-    return block_row[block < last_block ? block : last_block];                // (one too many: brought again, never multiplied)
+    const int place = 2 * turn + bring_block;
+    return block_row[walk.at(place < last_place ? place : last_place)];       // (one too many: brought again, never multiplied)
   };
   auto bring = [&](int physical, int stage) {
     const unsigned char* src = planes + kv_plane(a.kv, __builtin_amdgcn_readfirstlane(physical), kv_head) * 2;
@@ -1056,19 +1059,19 @@ attention_prefill_wide_kernel(AttnArgs a) {
     // values of positions that hold no token (they may be anything, and 0 * NaN is NaN) become zero where they lie, once,
     // in the turn that holds the sequence's last block: a test before every operand would keep their reads from flying together
     const int beyond = valid_end - last_block * BT_KV_BLOCK;
-    if (beyond < BT_KV_BLOCK && first_block + 2 * t + 1 >= last_block) {      // (the same for the whole work-group)
+    if (beyond < BT_KV_BLOCK && 2 * t + 1 >= last_place) {                    // (the same for the whole work-group)
       unsigned short* v = reinterpret_cast<unsigned short*>(wide_lds + ((t - t_begin) & 1) * WIDE_TURN +
-                                                            ((last_block - first_block) & 1) * WIDE_STAGE + WIDE_PLANE);
+                                                            (last_place & 1) * WIDE_STAGE + WIDE_PLANE);
       for (int e = (beyond >> 2) * 4 * HD + tid; e < BT_KV_BLOCK * HD; e += WIDE_THREADS)
         if (e / (4 * HD) * 4 + (e & 3) >= beyond) v[e] = 0;
       __syncthreads();
     }
-    const int block = first_block + 2 * t + set;
-    const int kb = block * BT_KV_BLOCK;
-    if (block <= last_block && kb < hi && kb + BT_KV_BLOCK > lo) {           // (the same for the whole wave)
+    const int place = 2 * t + set;
+    const int kb = walk.at(place) * BT_KV_BLOCK;
+    if (place <= last_place && kb < hi && (kb + BT_KV_BLOCK > lo || kb < a.keep)) {      // (the same for the whole wave)
       ops.stage = wide_lds + ((t - t_begin) & 1) * WIDE_TURN + set * WIDE_STAGE;
-      attend_block<PREFILL_NQ, true, false>(ops, kb, valid_end, kb + BT_KV_BLOCK > start + q0 + 1 || kb < lo_last, qpos, qlo, sc, q,
-                                            o, m, rows);
+      attend_block<PREFILL_NQ, true, false>(ops, kb, valid_end, kb + BT_KV_BLOCK > start + q0 + 1 || kb < lo_last, qpos, qlo, a.keep, sc,
+                                            q, o, m, rows);
     }
   }
   __syncthreads();                                          // everyone is done with the last turn
@@ -1131,36 +1134,37 @@ attention_decode_kernel(AttnArgs a) {
 #pragma unroll
   for (int dt = 0; dt < ND; ++dt) o[0][dt] = floatx4{0.f, 0.f, 0.f, 0.f};
 
-  const int lo = qlo[0] & ~31;
+  const KeyWalk walk = bt_key_walk(qlo[0] & ~31, a.keep, 32);
   const bf16_t* keys = static_cast<const bf16_t*>(a.kv.keys);
   const bf16_t* values = static_cast<const bf16_t*>(a.kv.values);
-  // the tiles of 32 keys from `lo` through the query's own position, cut into `splits` runs
-  const int tiles = (pos - lo) / 32 + 1, per_split = (tiles + splits - 1) / splits;
+  // the tiles of 32 keys that are kept or lie from `qlo` through the query's own position, cut into `splits` runs
+  const int tiles = walk.places(pos) / 32 + 1, per_split = (tiles + splits - 1) / splits;
   const int tile_begin = split * per_split;
   const int tile_end = tile_begin + per_split < tiles ? tile_begin + per_split : tiles;
-  const int first = lo + 32 * (tile_begin + wave), end = lo + 32 * tile_end;
+  const int first = 32 * (tile_begin + wave), end = 32 * tile_end;      // (places of the walk)
   // plane of the tile at kb: from the blocks fetched early where they apply, else from the table
   auto plane_of = [&](int kb, int j) {
     int block = (early && j < 2) ? (j == 0 ? early_block0 : early_block1) : block_row[kb / BT_KV_BLOCK];
     return kv_plane(a.kv, block, kv_head);
   };
   const Scoring sc = scoring_of(a, head);
-  auto fetch = [&](TileOperands& into, int kb, int j) {
-    if (kb < end) {
+  auto fetch = [&](TileOperands& into, int place, int j) {
+    if (place < end) {
+      const int kb = walk.at(place);
       int64_t plane = plane_of(kb, j);
       load_tile(into, keys + plane, values + plane, kb);
     }
   };
   auto attend = [&](const TileOperands& tile, int kb) {   // one form: this kernel waits for memory, not for the ALU
-    attend_tile<1, true>(tile, kb, pos + 1, qpos, qlo, sc, q, o, m, l);
+    attend_tile<1, true>(tile, kb, pos + 1, qpos, qlo, a.keep, sc, q, o, m, l);
   };
   TileOperands current, next;
   fetch(next, first, 0);
   int j = 0;
-  for (int kb = first; kb < end; kb += stride, ++j) {
+  for (int place = first; place < end; place += stride, ++j) {
     current = next;
-    fetch(next, kb + stride, j + 1);
-    attend(current, kb);
+    fetch(next, place + stride, j + 1);
+    attend(current, walk.at(place));
   }
   float total = l[0];
   total += __shfl_xor(total, 16, 64);
@@ -1263,7 +1267,8 @@ static int check_args(const AttnArgs& a, const char* who) {
   if (a.kv.head_dim != HD) BT_REFUSE("%s: built for head size %d, asked for %d", who, HD, a.kv.head_dim);
   if (a.kv.kv_heads <= 0 || a.q_heads <= 0 || a.q_heads % a.kv.kv_heads != 0)
     BT_REFUSE("%s: %d query heads cannot share %d key/value heads", who, a.q_heads, a.kv.kv_heads);
-  if (a.window < 0 || a.chunk < 0) BT_REFUSE("%s: window %d and chunk %d must not be negative", who, a.window, a.chunk);
+  if (a.window < 0 || a.chunk < 0 || a.keep < 0)
+    BT_REFUSE("%s: window %d, chunk %d and %d kept positions must not be negative", who, a.window, a.chunk, a.keep);
   if (!(a.scale > 0.f)) BT_REFUSE("%s: the score scale %g must be positive (the maximum is taken before scaling)", who, a.scale);
   if (!a.q || !a.out || !a.seq_off || !a.seq_start || !a.kv.blocks || !a.kv.keys || !a.kv.values)
     BT_REFUSE("%s: missing operand", who);

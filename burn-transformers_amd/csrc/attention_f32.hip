@@ -79,7 +79,9 @@ attention_f32_mfma_kernel(AttnArgs a) {
   const int n_queries = count - q0 < F32M_QUERIES ? count - q0 : F32M_QUERIES;
   const int first_pos = start + q0, last_pos = first_pos + n_queries - 1;
   const int lo_pos = bt_first_seen(first_pos, a.window, a.chunk);
-  const int first_block = lo_pos / BT_KV_BLOCK, last_block = last_pos / BT_KV_BLOCK;
+  const int last_block = last_pos / BT_KV_BLOCK;
+  const KeyWalk walk = bt_key_walk(lo_pos / BT_KV_BLOCK, (a.keep + BT_KV_BLOCK - 1) / BT_KV_BLOCK, 1);      // (in blocks)
+  const int last_place = walk.places(last_block);
   const bool wave_active = wave * 16 < n_queries;
   // what the wave's queries can see at all: positions wave_lo .. wave_hi
   const int wave_first = first_pos + wave * 16;
@@ -89,7 +91,7 @@ attention_f32_mfma_kernel(AttnArgs a) {
   const int mine = wave * 16 + i16;                          // the lane's query within the tile
   const bool exists = wave_active && mine < n_queries;
   const int qpos = exists ? first_pos + mine : -1;           // (a column without a query sees no key and is never stored)
-  const int qlo = exists ? bt_first_seen(qpos, a.window, a.chunk) : 0;
+  const SeenKeys seen = bt_seen_keys(qpos, bt_first_seen(qpos, a.window, a.chunk), a.keep);
 
   const float* q = static_cast<const float*>(a.q);
   floatx4 qreg[KS];
@@ -139,14 +141,15 @@ attention_f32_mfma_kernel(AttnArgs a) {
 #pragma unroll
   for (int dt = 0; dt < KS; ++dt) o[dt] = floatx4{0.f, 0.f, 0.f, 0.f};
 
-  fetch(first_block);
-  for (int block = first_block; block <= last_block; ++block) {
+  fetch(walk.at(0));
+  for (int place = 0; place <= last_place; ++place) {
+    const int block = walk.at(place);
     __syncthreads();                                         // the previous block's LDS is no longer read
     stage(block);
-    if (block < last_block) fetch(block + 1);                // in flight while this block is worked on
+    if (place < last_place) fetch(walk.at(place + 1));       // in flight while this block is worked on
     __syncthreads();
     const int kb = block * BT_KV_BLOCK;
-    if (!wave_active || kb > wave_hi || kb + BT_KV_BLOCK <= wave_lo) continue;   // (the same for the whole wave)
+    if (!wave_active || kb > wave_hi || (kb + BT_KV_BLOCK <= wave_lo && kb >= a.keep)) continue;   // (the same for the whole wave)
     // Operands are asked for a step before they are multiplied (two sets of registers, named at
     // compile time), and the four tiles' sums (then the blocks of output channels) take turns, so
     // that neither an LDS read nor a matrix instruction waits for the one before it.
@@ -184,11 +187,7 @@ attention_f32_mfma_kernel(AttnArgs a) {
 #pragma unroll
       for (int t = 0; t < 4; ++t)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int key_pos = kb + 16 * t + 4 * g + r;
-          const bool seen = key_pos <= qpos && key_pos >= qlo;
-          s[t][r] = seen ? s[t][r] : -INFINITY;
-        }
+        for (int r = 0; r < 4; ++r) s[t][r] = seen(kb + 16 * t + 4 * g + r) ? s[t][r] : -INFINITY;
     }
     if constexpr (FORM == 2) {           // every key's weight by itself; an excluded key's -inf gives exactly zero
 #pragma unroll
@@ -276,12 +275,14 @@ attention_f32_decode_kernel(AttnArgs a) {
   if (tid < hd) qs[tid] = q[tid];
   __syncthreads();
   const int lo = bt_first_seen(pos, a.window, a.chunk);
-  int first_block = lo / BT_KV_BLOCK, last_block = pos / BT_KV_BLOCK;
+  const KeyWalk walk = bt_key_walk(lo / BT_KV_BLOCK, (a.keep + BT_KV_BLOCK - 1) / BT_KV_BLOCK, 1);      // (in blocks)
+  const SeenKeys sees = bt_seen_keys(pos, lo, a.keep);
+  int first_place = 0, last_place = walk.places(pos / BT_KV_BLOCK);
   const int splits = a.splits > 1 ? a.splits : 1, split = blockIdx.z;
   if (splits > 1) {       // this work-group's run of the blocks (it may be empty)
-    const int per_split = (last_block - first_block + splits) / splits;
-    first_block += split * per_split;
-    last_block = first_block + per_split - 1 < last_block ? first_block + per_split - 1 : last_block;
+    const int per_split = (last_place + splits) / splits;
+    first_place += split * per_split;
+    last_place = first_place + per_split - 1 < last_place ? first_place + per_split - 1 : last_place;
   }
   const float* keys = static_cast<const float*>(a.kv.keys);
   const float* values = static_cast<const float*>(a.kv.values);
@@ -289,7 +290,8 @@ attention_f32_decode_kernel(AttnArgs a) {
   float run_max = FIRST_MAXIMUM, run_sum = 0.f, acc[CPT];
 #pragma unroll
   for (int j = 0; j < CPT; ++j) acc[j] = 0.f;
-  for (int block = first_block + wave; block <= last_block; block += 4) {
+  for (int place = first_place + wave; place <= last_place; place += 4) {
+    const int block = walk.at(place);
     int physical = a.kv.blocks[(int64_t)seq * a.kv.max_blocks + block];
     int64_t base = kv_plane(a.kv, physical, kv_head);
     // this lane's key: row `lane` of the block
@@ -309,8 +311,7 @@ attention_f32_decode_kernel(AttnArgs a) {
         s = fmaf(q4.w, kreg[c4].w, s);
       }
     }
-    const int key_pos = block * BT_KV_BLOCK + lane;
-    const bool seen = key_pos <= pos && key_pos >= lo;
+    const bool seen = sees(block * BT_KV_BLOCK + lane);
     float p, rescale = 1.f;
     if constexpr (FORM == 2) {
       p = seen ? bt_sigmoid(fmaf(s, a.scale, bias)) : 0.f;
@@ -436,7 +437,8 @@ BT_EXPORT int bt_attention_f32(void* stream, const AttnArgs* args) {
   if (hd <= 0 || hd % 16 != 0 || hd > 128) BT_REFUSE("attention_f32: head size %d must be a multiple of 16 up to 128", hd);
   if (a.kv.kv_heads <= 0 || a.q_heads <= 0 || a.q_heads % a.kv.kv_heads != 0)
     BT_REFUSE("attention_f32: %d query heads cannot share %d key/value heads", a.q_heads, a.kv.kv_heads);
-  if (a.window < 0 || a.chunk < 0) BT_REFUSE("attention_f32: window %d and chunk %d must not be negative", a.window, a.chunk);
+  if (a.window < 0 || a.chunk < 0 || a.keep < 0)
+    BT_REFUSE("attention_f32: window %d, chunk %d and %d kept positions must not be negative", a.window, a.chunk, a.keep);
   if (a.max_count <= 0) BT_REFUSE("attention_f32: max_count %d must be positive", a.max_count);
   if (!(a.scale > 0.f)) BT_REFUSE("attention_f32: scale %g must be positive", (double)a.scale);
   if (!a.q || !a.out || !a.seq_off || !a.seq_start || !a.kv.blocks || !a.kv.keys || !a.kv.values)

@@ -461,7 +461,7 @@ BT_EXPORT int bt_gemm_plain(void* stream, int dtype, const void* A, int64_t lda,
 // ---------------------------------------------------------------------------------------------
 // Plain attention over the paged cache.  One work-group per (token, query head).
 //   scores s_k = scale * (q . key_k) for keys lo <= k <= pos, lo = max(0, pos - window + 1), or the
-//   first position of pos's chunk if that is later (bt_first_seen)
+//   first position of pos's chunk if that is later (bt_first_seen), and for the kept first positions
 //   out = sum_k softmax(s)_k value_k, softmax in 32-bit with a running maximum over chunks; the other forms of
 //   the scores and the output stage (AttnArgs) as in the tiled kernels, decided as the kernel runs.
 // Keys beyond the token's own position are never read.
@@ -485,7 +485,8 @@ attention_plain_kernel(AttnArgs a) {
   const T* q = static_cast<const T*>(a.q) + (int64_t)t * a.ldq + head * hd;
   for (int c = threadIdx.x; c < hd; c += blockDim.x) qs[c] = to_float(q[c]);
   __syncthreads();
-  int lo = bt_first_seen(pos, a.window, a.chunk);
+  const KeyWalk walk = bt_key_walk(bt_first_seen(pos, a.window, a.chunk), a.keep, 1);      // (every position of it is seen)
+  const int places = walk.places(pos + 1);
   float run_max = a.form == 2 ? 0.f : -INFINITY, run_sum = 0.f;
   const float bias = a.form == 2 && a.score_bias ? a.score_bias[head] : 0.f;
   float acc[PLAIN_PER_THREAD];                          // channels threadIdx.x, threadIdx.x + 256, ... (< hd)
@@ -493,11 +494,11 @@ attention_plain_kernel(AttnArgs a) {
   for (int j = 0; j < PLAIN_PER_THREAD; ++j) acc[j] = 0.f;
   const T* keys = static_cast<const T*>(a.kv.keys);
   const T* values = static_cast<const T*>(a.kv.values);
-  for (int c0 = lo; c0 <= pos; c0 += PLAIN_CHUNK) {
-    int n = pos + 1 - c0 < PLAIN_CHUNK ? pos + 1 - c0 : PLAIN_CHUNK;
+  for (int c0 = 0; c0 < places; c0 += PLAIN_CHUNK) {
+    int n = places - c0 < PLAIN_CHUNK ? places - c0 : PLAIN_CHUNK;
     float local_max = -INFINITY;
     for (int i = threadIdx.x; i < n; i += blockDim.x) {
-      int k = c0 + i;
+      int k = walk.at(c0 + i);
       const T* kr = keys + kv_block_base(a.kv, seq, k, kv_head) + key_offset(hd, k, 0);
       float s = 0.f;
       for (int c = 0; c < hd; ++c) s = fmaf(qs[c], to_float(kr[c]), s);
@@ -526,7 +527,7 @@ attention_plain_kernel(AttnArgs a) {
       if (channel >= hd) break;
       acc[j] *= rescale;
       for (int i = 0; i < n; ++i) {
-        int k = c0 + i;
+        int k = walk.at(c0 + i);
         const T* vr = values + kv_block_base(a.kv, seq, k, kv_head);
         acc[j] = fmaf(ps[i], to_float(vr[value_offset(hd, k, channel)]), acc[j]);
       }
@@ -554,7 +555,8 @@ int bt_check_attention(const AttnArgs& a, const char* who) {
               PLAIN_MAX_HEAD, PLAIN_PER_THREAD);
   if (a.kv.kv_heads <= 0 || a.q_heads <= 0 || a.q_heads % a.kv.kv_heads != 0)
     BT_REFUSE("%s: %d query heads cannot share %d key/value heads", who, a.q_heads, a.kv.kv_heads);
-  if (a.window < 0 || a.chunk < 0) BT_REFUSE("%s: window %d and chunk %d must not be negative", who, a.window, a.chunk);
+  if (a.window < 0 || a.chunk < 0 || a.keep < 0)
+    BT_REFUSE("%s: window %d, chunk %d and %d kept positions must not be negative", who, a.window, a.chunk, a.keep);
   if (!a.q || !a.out || !a.tok_seq || !a.tok_pos || !a.seq_off || !a.seq_start || !a.kv.blocks ||
       !a.kv.keys || !a.kv.values)
     BT_REFUSE("%s: missing operand", who);

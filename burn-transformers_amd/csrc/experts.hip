@@ -14,6 +14,8 @@
 // instead of its best, and weights that are the chosen experts' scores as they are instead of over
 // their sum.  The experts' activation (`act`) is silu(g) * u, or with a `limit`:
 // g' = min(g, limit), u' = clamp(u, -limit, limit), g' * sigmoid(alpha * g') * (u' + 1).
+// A third kind of score makes the choice by the logits themselves (with the correction) and weighs the chosen
+// experts by the softmax over THEIR logits alone.  `bias` is added to the logits first.
 // Ties between equal scores go to the lower index.
 #include "host.h"
 
@@ -33,9 +35,10 @@ struct RouteCall {
   const float* gate_w;      // [width] float32 or null
   float* weights;           // [tokens][experts]
   float* gate;              // [tokens]: sigmoid(gate_w . h), or null
-  int score;                // 0: softmax over all experts; 1: each logit's sigmoid
+  int score;                // 0: softmax over all experts; 1: each logit's sigmoid; 2: the logits, softmax over the chosen
   int group_rank;           // a group's score is the sum of its so many best (corrected) scores; 0 or 1: its best
   int normalize;            // 1: the chosen experts' scores over their sum; 0: the scores as they are
+  const float* bias;        // [experts] or null: added to the logits
 };
 
 // The best (value, index) of a wave; among equal values the lowest index.  Every lane gets it.
@@ -74,6 +77,11 @@ __global__ void __launch_bounds__(ROUTE_THREADS) route_kernel(RouteCall c) {
 #pragma unroll
     for (int j = 0; j < 4; ++j)
       if (lane + 64 * j < c.experts) early_correction[j] = c.correction[lane + 64 * j];
+  float early_bias[4] = {0.f, 0.f, 0.f, 0.f};
+  if (wave == 0 && c.bias)
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (lane + 64 * j < c.experts) early_bias[j] = c.bias[lane + 64 * j];
   for (int first = wave; first < outputs; first += waves * ROUTE_OUTPUTS) {
     float sums[ROUTE_OUTPUTS];
     const float* rows[ROUTE_OUTPUTS];               // an output beyond the last reads the last one's row and is dropped
@@ -116,6 +124,8 @@ __global__ void __launch_bounds__(ROUTE_THREADS) route_kernel(RouteCall c) {
   }
   __syncthreads();
   if (wave != 0) return;
+  if (c.bias)                                       // a lane keeps to its own experts
+    for (int e = lane, j = 0; e < c.experts; e += 64, ++j) score[e] += j < 4 ? early_bias[j < 4 ? j : 0] : c.bias[e];
   float top_logit = -INFINITY;
   for (int e = lane; e < c.experts; e += 64) top_logit = fmaxf(top_logit, score[e]);
   top_logit = wave_max(top_logit);
@@ -124,9 +134,10 @@ __global__ void __launch_bounds__(ROUTE_THREADS) route_kernel(RouteCall c) {
   total = wave_sum(total);
   float* weights = c.weights + (int64_t)t * c.experts;
   for (int e = lane, j = 0; e < c.experts; e += 64, ++j) {     // a lane keeps to its own experts: no other lane reads them yet
-    const float s = c.score == 1 ? 1.0f / (1.0f + expf(-score[e])) : expf(score[e] - top_logit) / total;
+    const float z = score[e];
+    const float s = c.score == 1 ? 1.0f / (1.0f + expf(-z)) : c.score == 2 ? expf(z - top_logit) : expf(z - top_logit) / total;
     score[e] = s;
-    choice[e] = s + (c.correction ? (j < 4 ? early_correction[j < 4 ? j : 0] : c.correction[e]) : 0.f);
+    choice[e] = (c.score == 2 ? z : s) + (c.correction ? (j < 4 ? early_correction[j < 4 ? j : 0] : c.correction[e]) : 0.f);
   }
   __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
   __builtin_amdgcn_wave_barrier();
@@ -209,7 +220,7 @@ BT_EXPORT int bt_route_call(void* stream, const RouteCall* c) {
       BT_REFUSE("route: %d open groups of %d experts cannot give %d experts", c->keep, c->experts / c->groups, c->top);
   }
   if (c->width <= 0) BT_REFUSE("route: width %d must be positive", c->width);
-  if ((c->score != 0 && c->score != 1) || c->group_rank < 0 || (c->normalize != 0 && c->normalize != 1))
+  if (c->score < 0 || c->score > 2 || (c->score == 2 && c->normalize != 1) || c->group_rank < 0 || (c->normalize != 0 && c->normalize != 1))
     BT_REFUSE("route: score %d, group_rank %d, normalize %d: not a router this kernel knows", c->score, c->group_rank, c->normalize);
   if (!c->h || !c->W || !c->weights || (c->gate_w && !c->gate)) BT_REFUSE("route: missing operand");
   // (measured at 2,048 tokens of width 2,048: 32 us with sixteen waves a token, 18 with four)
@@ -240,13 +251,14 @@ struct GatedExpertsCall {
   int64_t ldh;
   float* identity_out;      // [tokens][width] float32: (sum of the identity experts' weights) * h; or null
   int act;                  // 0: silu(g) * u; 1: min(g, limit) * sigmoid(alpha * min(g, limit)) * (clamp(u, -limit, limit) + 1);
-                            // 2, 3: units WITHOUT a gate, gelu(u) in its exact (erf) form and silu(u): `gu` then holds per
-                            // expert its ff up rows only, the shared expert's behind them
+                            // 2, 3, 4: units WITHOUT a gate, gelu(u) in its exact (erf) form, silu(u) and max(u, 0)^2: `gu`
+                            // then holds per expert its ff up rows only, the shared expert's behind them
   float limit;
   float alpha;
 };
 
 __device__ __forceinline__ float plain_unit(const GatedExpertsCall& c, float u) {
+  if (c.act == 4) return u > 0.f ? u * u : 0.f;
   return c.act == 2 ? 0.5f * u * (1.0f + erff(u * 0.70710678118654752f)) : u / (1.0f + expf(-u));
 }
 
@@ -305,7 +317,7 @@ BT_EXPORT int bt_gated_experts_call(void* stream, const GatedExpertsCall* c) {
   if (c->experts < 0 || c->ff <= 0 || c->shared_ff < 0 || c->identity < 0)
     BT_REFUSE("gated_experts: %d experts of %d, a shared one of %d and %d identity experts", c->experts, c->ff, c->shared_ff, c->identity);
   const int64_t columns = (int64_t)c->experts * c->ff + c->shared_ff;
-  if (c->act < 0 || c->act > 3) BT_REFUSE("gated_experts: unknown activation %d", c->act);
+  if (c->act < 0 || c->act > 4) BT_REFUSE("gated_experts: unknown activation %d", c->act);
   if (c->hidden_cols < columns || c->ld_hidden < c->hidden_cols || c->ld_gu < (c->act < 2 ? 2 : 1) * columns)
     BT_REFUSE("gated_experts: the rows do not hold the experts");
   if (!c->gu || (!c->weights && c->experts + c->identity > 0) || !c->hidden || (c->identity_out && (!c->h || c->width <= 0)))

@@ -2,7 +2,8 @@
 // latents; only the key/value latent is cached, and attention runs on it directly).
 //   * latent norms: the two RMS norms behind the fused down-projection; the query latent goes to a
 //     buffer for the next product, the key/value latent straight into the paged cache, where it is
-//     the one shared "head" whose keys and values are the same vector.  With `rot_dim` > 0 the down-projection
+//     the one shared "head" whose keys and values are the same vector (or only the query latent, for a layer that
+//     attends over another layer's cached latent: `kv_rank` 0).  With `rot_dim` > 0 the down-projection
 //     has that many more rows behind the key/value latent: one key part that all heads share, not normalised,
 //     turned by the token's position (channel 2 i with channel 2 i + 1, or i with i + rot_dim / 2), kept behind
 //     the latent in the cached head's KEYS (its values have zeros there)
@@ -17,7 +18,7 @@ struct LatentNormCall {
   int dtype;              // element type of `q_out` and of the cache: 0 float32, 1 bfloat16
   int tokens;
   int q_rank, q_cols;     // the query latent's length; columns of q_out written (latent, then zeros)
-  int kv_rank;            // the key/value latent's length (the cache's head size may be larger: zeros)
+  int kv_rank;            // the key/value latent's length (the cache's head size may be larger: zeros); 0: none, nothing is cached
   int kv_offset;          // its first column in `in`
   float eps;
   const float* in;        // [tokens][ld] float32: the fused down-projection
@@ -76,18 +77,20 @@ __global__ void __launch_bounds__(256) latent_norm_kernel(LatentNormCall c) {
 
 BT_EXPORT int bt_latent_norm_call(void* stream, const LatentNormCall* c) {
   if (c->tokens <= 0) return BT_OK;
-  if (c->q_rank <= 0 || c->kv_rank <= 0) BT_REFUSE("latent_norm: ranks %d and %d must be positive", c->q_rank, c->kv_rank);
+  if (c->q_rank <= 0 || c->kv_rank < 0) BT_REFUSE("latent_norm: ranks %d and %d must be positive", c->q_rank, c->kv_rank);
+  const bool caches = c->kv_rank > 0;
   if (c->rot_dim < 0 || c->rot_dim % 2 != 0 || (c->pairing != 0 && c->pairing != 1) || (c->rot_dim > 0 && !c->inv_freq))
     BT_REFUSE("latent_norm: a turned key part of %d channels (even, with frequencies), pairing %d (0 or 1)", c->rot_dim, c->pairing);
-  if (c->kv.kv_heads != 1 || c->kv.head_dim < c->kv_rank + c->rot_dim)
+  if (caches && (c->kv.kv_heads != 1 || c->kv.head_dim < c->kv_rank + c->rot_dim))
     BT_REFUSE("latent_norm: the cache keeps %d heads of %d, expected one of at least %d", c->kv.kv_heads,
               c->kv.head_dim, c->kv_rank + c->rot_dim);
-  if (c->q_cols < c->q_rank || c->ld_q < c->q_cols || c->ld < c->kv_offset + c->kv_rank + c->rot_dim || c->kv_offset < c->q_rank)
+  if (c->q_cols < c->q_rank || c->ld_q < c->q_cols || c->ld < c->q_rank ||
+      (caches && (c->ld < c->kv_offset + c->kv_rank + c->rot_dim || c->kv_offset < c->q_rank)))
     BT_REFUSE("latent_norm: the rows do not hold the latents");
-  if (!c->in || !c->q_gamma || !c->kv_gamma || !c->q_out || !c->tok_seq || !c->tok_pos || !c->kv.blocks ||
-      !c->kv.keys || !c->kv.values)
+  if (!c->in || !c->q_gamma || !c->q_out ||
+      (caches && (!c->kv_gamma || !c->tok_seq || !c->tok_pos || !c->kv.blocks || !c->kv.keys || !c->kv.values)))
     BT_REFUSE("latent_norm: missing operand");
-  dim3 grid(c->tokens, 2), block(256);
+  dim3 grid(c->tokens, caches ? 2 : 1), block(256);
   if (c->dtype == 0)
     hipLaunchKernelGGL(latent_norm_kernel<float>, grid, block, 0, (hipStream_t)stream, *c);
   else
@@ -153,6 +156,7 @@ BT_EXPORT int bt_latent_query_call(void* stream, const LatentQueryCall* c) {
   return bt_check_launch("latent_query");
 }
 
+// (gate_span 1: one gate a head, sigmoid(gate[t][h]), instead of one per output)
 // out[t][h * vdim + v] = sigmoid(gate[t][h * vdim + v]) * sum_r W[h * vdim + v][r] * ctx[t][h * ld_head + r]
 // One work-group per (tile of HP_TOKENS tokens, head, run of up to HP_VCHUNK outputs); the rank is
 // walked in steps of HP_RSTEP through LDS (the weights transposed, so that threads with consecutive
@@ -175,6 +179,7 @@ struct HeadProjectCall {
   int64_t ld_gate;
   void* out;              // [tokens][ld_out]
   int64_t ld_out;
+  int gate_span;          // 0: a gate per output; 1: a gate per head
 };
 
 template <typename T>
@@ -218,7 +223,7 @@ __global__ void __launch_bounds__(256) head_project_kernel(HeadProjectCall c) {
     if (t0 + i >= c.tokens || v >= vc) continue;
     const int col = head * c.vdim + v0 + v;
     float y = acc[k];
-    if (c.gate) y *= 1.0f / (1.0f + expf(-c.gate[(int64_t)(t0 + i) * c.ld_gate + col]));
+    if (c.gate) y *= 1.0f / (1.0f + expf(-c.gate[(int64_t)(t0 + i) * c.ld_gate + (c.gate_span == 1 ? head : col)]));
     out[(int64_t)(t0 + i) * c.ld_out + col] = from_float<T>(y);
   }
   // the columns behind the last head's, which the next product reads as zeros
@@ -249,7 +254,7 @@ __global__ void __launch_bounds__(256) head_project_small_kernel(HeadProjectCall
   acc += __shfl_xor(acc, 1, 64);
   T* out = static_cast<T*>(c.out) + (int64_t)t * c.ld_out;
   if (live && part == 0) {
-    if (c.gate) acc *= 1.0f / (1.0f + expf(-c.gate[(int64_t)t * c.ld_gate + col]));
+    if (c.gate) acc *= 1.0f / (1.0f + expf(-c.gate[(int64_t)t * c.ld_gate + (c.gate_span == 1 ? head : col)]));
     out[col] = from_float<T>(acc);
   }
   if (head == c.heads - 1 && blockIdx.z == gridDim.z - 1)
@@ -262,8 +267,9 @@ BT_EXPORT int bt_head_project_call(void* stream, const HeadProjectCall* c) {
     BT_REFUSE("head_project: %d heads of %d from rank %d: all must be positive", c->heads, c->vdim, c->rank);
   if (c->head_pitch < c->rank || c->ld_ctx < (int64_t)c->heads * c->head_pitch ||
       c->out_cols < c->heads * c->vdim || c->ld_out < c->out_cols ||
-      (c->gate && c->ld_gate < (int64_t)c->heads * c->vdim))
+      (c->gate && c->ld_gate < (c->gate_span == 1 ? (int64_t)c->heads : (int64_t)c->heads * c->vdim)))
     BT_REFUSE("head_project: the rows do not hold %d heads", c->heads);
+  if (c->gate_span != 0 && c->gate_span != 1) BT_REFUSE("head_project: gate_span %d must be 0 or 1", c->gate_span);
   if (!c->ctx || !c->W || !c->out) BT_REFUSE("head_project: missing operand");
   if (c->tokens <= HP_SMALL_TOKENS) {
     dim3 small(c->tokens, c->heads, (c->vdim + 63) / 64);

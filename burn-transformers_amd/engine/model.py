@@ -48,8 +48,8 @@ class CausalLM:
         K.prepare(self.dtype, sorted({name for part in parts for name in part.kernel_modules(self.dtype)}))
 
     def _check_schedule(self):
-        """Every cache entry has exactly one writer, which runs before any reader, and readers keep
-        what the writer keeps."""
+        """Every cache entry has exactly one writer, which runs before any reader, and readers read heads of
+        the size the writer keeps; the entry keeps every position that one of them still reads."""
         writers = {}
         for position, entry in enumerate(self.schedule):
             if not (0 <= entry.layer < len(self.blocks)):
@@ -64,9 +64,13 @@ class CausalLM:
                 writers[entry.cache] = specs
             elif entry.cache not in writers:
                 raise ValueError(f"schedule entry {position} reads cache entry {entry.cache} before it is written")
-            elif writers[entry.cache] != specs:
-                raise ValueError(f"schedule entry {position} reads cache entry {entry.cache}, "
-                                 f"whose keys and values have another shape")
+            else:
+                kv, state = writers[entry.cache]
+                if state != specs[1] or (kv is None) != (specs[0] is None) or \
+                        (kv is not None and (kv.kv_heads, kv.head_dim) != (specs[0].kv_heads, specs[0].head_dim)):
+                    raise ValueError(f"schedule entry {position} reads cache entry {entry.cache}, "
+                                     f"whose keys and values have another shape")
+                writers[entry.cache] = (kv.joined(specs[0]) if kv is not None else None, state)
         self.cache_entries = max(writers) + 1 if writers else 0
         self.kv_specs = [writers.get(i, (None, None))[0] for i in range(self.cache_entries)]
         self.state_specs = [writers.get(i, (None, None))[1] for i in range(self.cache_entries)]

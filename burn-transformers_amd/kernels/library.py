@@ -51,7 +51,7 @@ class AttnArgs(ctypes.Structure):
                 ("max_count", _c_int), ("window", _c_int), ("scale", _c_float), ("splits", _c_int),
                 ("partial", _c_ptr), ("out_rows", _c_int), ("chunk", _c_int), ("sink", _c_ptr), ("form", _c_int),
                 ("cap", _c_float), ("score_bias", _c_ptr), ("gate", _c_ptr), ("ld_gate", _c_i64), ("gate_span", _c_int),
-                ("gate_dim", _c_int), ("out_f32", _c_int)]
+                ("gate_dim", _c_int), ("out_f32", _c_int), ("keep", _c_int)]
 
 
 class NormOperand(ctypes.Structure):
@@ -132,7 +132,7 @@ class LatentQueryCall(ctypes.Structure):
 class HeadProjectCall(ctypes.Structure):
     _fields_ = [("dtype", _c_int), ("tokens", _c_int), ("heads", _c_int), ("vdim", _c_int), ("rank", _c_int),
                 ("head_pitch", _c_int), ("out_cols", _c_int), ("ctx", _c_ptr), ("ld_ctx", _c_i64), ("W", _c_ptr),
-                ("gate", _c_ptr), ("ld_gate", _c_i64), ("out", _c_ptr), ("ld_out", _c_i64)]
+                ("gate", _c_ptr), ("ld_gate", _c_i64), ("out", _c_ptr), ("ld_out", _c_i64), ("gate_span", _c_int)]
     _step_fields_ = {"tokens": "tokens"}
 
 
@@ -196,7 +196,7 @@ class RouteCall(ctypes.Structure):
     _fields_ = [("dtype", _c_int), ("tokens", _c_int), ("width", _c_int), ("experts", _c_int), ("top", _c_int),
                 ("groups", _c_int), ("keep", _c_int), ("h", _c_ptr), ("ldh", _c_i64), ("W", _c_ptr),
                 ("correction", _c_ptr), ("gate_w", _c_ptr), ("weights", _c_ptr), ("gate", _c_ptr), ("score", _c_int),
-                ("group_rank", _c_int), ("normalize", _c_int)]
+                ("group_rank", _c_int), ("normalize", _c_int), ("bias", _c_ptr)]
     _step_fields_ = {"tokens": "tokens"}
 
 
@@ -953,20 +953,22 @@ def _library_has_algorithm(lda, m, n, k, epilogue):
 
 def attention_args(q, out, kv_view, tok_seq, tok_pos, seq_off, seq_start, q_heads, n_seqs, max_count,
                    scale, window=0, partial=None, runs=None, chunk=0, sink=None, softcap=0.0, sigmoid=False, score_bias=None,
-                   gate=None, gate_dim=0):
+                   gate=None, gate_dim=0, keep=0):
     """``partial``: float32 [rows * q_heads * runs, head_dim + 2] for a step whose keys are cut into
     runs that separate work-groups take.  Decode steps (long contexts in small batches): rows are
     the sequences, and ``runs`` follows from the shape.  Prompt steps (few query tiles behind a long
     context): rows are the step's tokens, the buffer may be longer than this step needs, and
     ``runs`` is given.  ``out`` may be a :class:`Chunked` for the bfloat16 decode kernels.
     ``chunk`` > 0: a query at position p sees only the keys from p - p % chunk on (chunks are counted
-    from position 0 of its sequence); ``window`` > 0: only the last ``window`` positions.  ``sink``: float32
+    from position 0 of its sequence); ``window`` > 0: only the last ``window`` positions; the first ``keep`` positions of a
+    sequence are seen whatever these say.  ``sink``: float32
     [q_heads], a logit per head whose exponential stands in every softmax's denominator beside the keys'
     (no key, no value, not scaled).  ``softcap`` > 0: scores become softcap * tanh(score / softcap) before the
     softmax.  ``sigmoid``: no softmax; a visible key weighs sigmoid(score + ``score_bias``[head]) (float32 [q_heads]).
     ``gate``: float32 logits whose sigmoid multiplies the output, [tokens, >= q_heads] a logit per head, or with
     ``gate_dim`` [tokens, >= q_heads * gate_dim] one per channel.  A float32 ``out`` of bfloat16 queries keeps the
     output's digits."""
+    keep = min(keep or 0, 1 << 30)
     if score_bias is not None and (score_bias.dtype != torch.float32 or score_bias.numel() != q_heads or not score_bias.is_contiguous()):
         raise KernelError(f"attention: the scores' bias is one float32 number per query head, got {tuple(score_bias.shape)} {score_bias.dtype}")
     if gate is not None and (gate.dtype != torch.float32 or gate.shape[0] < q.shape[0] or gate.stride(1) != 1):
@@ -988,7 +990,8 @@ def attention_args(q, out, kv_view, tok_seq, tok_pos, seq_off, seq_start, q_head
                     n_seqs=n_seqs, max_count=max_count, window=window or 0, scale=scale, chunk=chunk or 0, sink=_ptr(sink),
                     form=2 if sigmoid else 1 if softcap else 0, cap=softcap or 0.0, score_bias=_ptr(score_bias),
                     gate=_ptr(gate), ld_gate=gate.stride(0) if gate is not None else 0, gate_span=1 if gate_dim else 0,
-                    gate_dim=gate_dim, out_f32=1 if out.dtype == torch.float32 and q.dtype != torch.float32 else 0)
+                    gate_dim=gate_dim, out_f32=1 if out.dtype == torch.float32 and q.dtype != torch.float32 else 0,
+                    keep=keep)
 
 
 def attention_variant(args):
@@ -1186,11 +1189,12 @@ def latent_norm(fused, q_rank, kv_offset, kv_rank, q_gamma, kv_gamma, eps, q_out
     paged cache at each token's position, as the keys AND the values of its one head.  With ``rot_dim`` the
     next so many columns are a key part that is not normalised but turned by the token's position (angles
     position * ``inv_freq[i]``, sine and cosine times ``amplitude``; channel 2 i with 2 i + 1, or with
-    ``neighbours`` False i with i + rot_dim / 2) and kept behind the latent in the head's keys."""
+    ``neighbours`` False i with i + rot_dim / 2) and kept behind the latent in the head's keys.  ``kv_rank`` 0:
+    only the first of the two norms, nothing goes to the cache."""
     _launch(_module("latent"), "bt_latent_norm_call",
             LatentNormCall(dtype=DTYPE_CODES[dtype], tokens=fused.shape[0], q_rank=q_rank, q_cols=q_out.shape[1],
                            kv_rank=kv_rank, kv_offset=kv_offset, eps=eps, input=fused.data_ptr(), ld=fused.stride(0),
-                           q_gamma=q_gamma.data_ptr(), kv_gamma=kv_gamma.data_ptr(), q_out=q_out.data_ptr(),
+                           q_gamma=q_gamma.data_ptr(), kv_gamma=_ptr(kv_gamma), q_out=q_out.data_ptr(),
                            ld_q=q_out.stride(0), tok_seq=tok_seq.data_ptr(), tok_pos=tok_pos.data_ptr(), kv=kv_view,
                            rot_dim=rot_dim, pairing=1 if neighbours else 0, amplitude=amplitude, inv_freq=_ptr(inv_freq)))
 
@@ -1205,9 +1209,9 @@ def latent_query(sums, heads, pitch, rot_at, rot_dim, inv_freq, tok_pos, out, ne
                             tok_pos=tok_pos.data_ptr()))
 
 
-def head_project(ctx, weight, heads, vdim, rank, head_pitch, out, gate=None):
+def head_project(ctx, weight, heads, vdim, rank, head_pitch, out, gate=None, gate_span="channel"):
     """out[t, h * vdim + v] = sigmoid(gate[t, h * vdim + v]) * sum_r weight[h * vdim + v, r] * ctx[t, h * head_pitch + r]
-    (without ``gate``: no factor); the columns of ``out`` behind heads * vdim are set to zero."""
+    (without ``gate``: no factor; ``gate_span`` "head": one gate a head, gate[t, h]); the columns of ``out`` behind heads * vdim are set to zero."""
     if ctx.dtype != weight.dtype or out.dtype != weight.dtype or not weight.is_contiguous() or \
             tuple(weight.shape) != (heads * vdim, rank):
         raise KernelError(f"head_project: weights {tuple(weight.shape)} {weight.dtype} do not fit {heads} heads of {vdim} from rank {rank}")
@@ -1215,7 +1219,7 @@ def head_project(ctx, weight, heads, vdim, rank, head_pitch, out, gate=None):
             HeadProjectCall(dtype=DTYPE_CODES[weight.dtype], tokens=ctx.shape[0], heads=heads, vdim=vdim, rank=rank,
                             head_pitch=head_pitch, out_cols=out.shape[1], ctx=ctx.data_ptr(), ld_ctx=ctx.stride(0),
                             W=weight.data_ptr(), gate=_ptr(gate), ld_gate=gate.stride(0) if gate is not None else 0,
-                            out=out.data_ptr(), ld_out=out.stride(0)))
+                            out=out.data_ptr(), ld_out=out.stride(0), gate_span={"channel": 0, "head": 1}[gate_span]))
 
 
 # --- recurrent mixers ------------------------------------------------------------------------
@@ -1344,21 +1348,24 @@ def differential(rows, heads, vdim, pitch, weight, post, eps, out):
 # --- routed feed-forward ----------------------------------------------------------------------
 
 def route(h, router, correction, top, groups, keep, weights, gate_weight=None, gate=None, score="softmax",
-          group_rank=1, normalize=True):
+          group_rank=1, normalize=True, bias=None):
     """Per row of ``h``: softmax of the float32 router's logits over all experts, the ``top`` experts
     with the largest score + ``correction`` among the best ``keep`` of ``groups`` equal groups (groups
     <= 1: among all), and into ``weights`` [rows, experts] the chosen experts' scores divided by their
     sum, zero elsewhere.  With ``gate_weight`` [width]: ``gate`` [rows] = sigmoid(gate_weight . h).
     ``score`` "sigmoid": each logit's sigmoid instead of the softmax; ``group_rank`` n: a group's score is the
-    sum of its n best; ``normalize`` False: the chosen experts' scores as they are."""
+    sum of its n best; ``normalize`` False: the chosen experts' scores as they are.  ``score`` "chosen": the choice is made
+    by logit + ``correction``, the weights are the softmax over the chosen logits alone.  ``bias`` ([experts] float32):
+    added to the logits."""
     _launch(_module("experts"), "bt_route_call",
             RouteCall(dtype=DTYPE_CODES[h.dtype], tokens=h.shape[0], width=router.shape[1], experts=router.shape[0],
                       top=top, groups=groups, keep=keep, h=h.data_ptr(), ldh=h.stride(0), W=router.data_ptr(),
                       correction=_ptr(correction), gate_w=_ptr(gate_weight), weights=weights.data_ptr(), gate=_ptr(gate),
-                      score={"softmax": 0, "sigmoid": 1}[score], group_rank=group_rank, normalize=1 if normalize else 0))
+                      score={"softmax": 0, "sigmoid": 1, "chosen": 2}[score], group_rank=group_rank, normalize=1 if normalize else 0,
+                      bias=_ptr(bias)))
 
 
-EXPERT_UNITS = {"gated_silu": 0, "gated_clamped": 1, "gelu_erf": 2, "silu": 3}
+EXPERT_UNITS = {"gated_silu": 0, "gated_clamped": 1, "gelu_erf": 2, "silu": 3, "squared_relu": 4}
 
 
 def gated_experts(gu, weights, gate, experts, ff, shared_ff, identity, hidden, h=None, identity_out=None, limit=None,
@@ -1368,7 +1375,7 @@ def gated_experts(gu, weights, gate, experts, ff, shared_ff, identity, hidden, h
     token uses, weighted by ``gate[t]``); columns behind them are set to zero.  ``identity_out`` (float32
     [rows, width]) receives (the sum of the identity experts' weights) * h.  With ``limit`` the unit is
     g' * sigmoid(alpha * g') * (u' + 1), g' = min(gate, limit), u' = clamp(up, -limit, limit), instead of silu(gate) * up.
-    ``unit`` "gelu_erf" or "silu": units without a gate, act(up_e,i); ``gu`` then holds only the up rows (ff per
+    ``unit`` "gelu_erf", "silu" or "squared_relu": units without a gate, act(up_e,i); ``gu`` then holds only the up rows (ff per
     expert, the shared expert's behind them)."""
     act = EXPERT_UNITS[unit] if unit is not None else (0 if limit is None else 1)
     _launch(_module("experts"), "bt_gated_experts_call",

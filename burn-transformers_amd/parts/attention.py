@@ -2,7 +2,8 @@
 
 Parameters (all from the plan): width, heads, kv_heads, head_dim, scale (multiplies q.k),
 window (0 = every earlier key), chunk (0, or a query sees only the keys of its own chunk of that many
-positions, counted from position 0 of the sequence), causal.  Tensors: a fused projection ``qkv_weight`` held
+positions, counted from position 0 of the sequence), keep (default 0: the first so many positions of a sequence are
+seen whatever window and chunk say), causal.  Tensors: a fused projection ``qkv_weight`` held
 [heads*head_dim + 2*kv_heads*head_dim, width] with its bias, and ``out_weight`` [width,
 heads*head_dim] with its bias.
 
@@ -40,6 +41,14 @@ PROMPT_RUN_BLOCKS = 8
 PROMPT_RUN_MIN_CONTEXT = 1024      # no runs in steps whose class of context is this or less: they gain from some 2,000 keys on
 
 
+def keys_in_reach(context, window, chunk, keep):
+    """The most keys a query of a step sees whose longest context is ``context``, a tile's slack added."""
+    for reach in (window, chunk):
+        if reach:
+            context = min(context, reach + 32 + (keep + 31) // 32 * 32)
+    return context
+
+
 @register("mixer", "attention")
 class CausalSelfAttention(Mixer):
     takes_deferred_norm = True
@@ -50,7 +59,7 @@ class CausalSelfAttention(Mixer):
         p = params
         self.width, self.heads, self.kv_heads = p["width"], p["heads"], p["kv_heads"]
         self.head_dim, self.scale, self.window = p["head_dim"], float(p["scale"]), int(p.get("window") or 0)
-        self.chunk = int(p.get("chunk") or 0)
+        self.chunk, self.keep = int(p.get("chunk") or 0), int(p.get("keep") or 0)
         if not p.get("causal", True):
             raise ValueError("attention: only causal attention runs from a cache")
         if self.head_dim <= 0:
@@ -86,7 +95,7 @@ class CausalSelfAttention(Mixer):
         self.out_packed = packed_for_stream(self.out_weight) if self.out_weight.is_cuda else None
 
     def kv_spec(self):
-        return KVSpec(self.kv_heads, self.head_dim, self.window, self.chunk)
+        return KVSpec(self.kv_heads, self.head_dim, self.window, self.chunk, self.keep)
 
     def kernel_modules(self, dtype):
         if self.plain_only:
@@ -100,10 +109,7 @@ class CausalSelfAttention(Mixer):
         context, not its exact lengths, so that every step of a class runs the same kernels."""
         if not step.decode:
             return 1
-        keys = step.context_limit
-        for reach in (self.window, self.chunk):           # the most keys a query sees, a tile's slack added
-            if reach:
-                keys = min(keys, reach + 32)
+        keys = keys_in_reach(step.context_limit, self.window, self.chunk, self.keep)
         pair_bytes = keys * self.head_dim * 2 * (2 if step.dtype_is_bf16 else 4)     # one head's keys and values
         if pair_bytes <= SPLIT_BYTES:
             return 1
@@ -162,6 +168,6 @@ class CausalSelfAttention(Mixer):
             partial = step.buffer("attention.partial", tokens * self.heads * prompt_runs, self.head_dim + 2, "float32")
         args = K.attention_args(q, mixed, kv, step.tok_seq, step.tok_pos, step.seq_off, step.seq_start,
                                 self.heads, step.n_seqs, step.max_count, self.scale, self.window, partial,
-                                runs=prompt_runs if prompt_runs > 1 else None, chunk=self.chunk)
+                                runs=prompt_runs if prompt_runs > 1 else None, chunk=self.chunk, keep=self.keep)
         K.attention(args, step.dtype, step.decode, impl="plain" if self.plain_only else "auto")
         stream.add_product(step, mixed, self.out_weight, self.out_bias, packed=self.out_packed)

@@ -6,13 +6,15 @@ without tensors whose output is their input; they are the LAST router outputs), 
 token uses), groups / keep (the experts, identity experts included, form ``groups`` equal groups of
 neighbours, and only experts of the ``keep`` groups with the best score can be chosen; groups <= 1:
 all can), shared_ff (inner width of the expert every token uses; 0: none), score ("softmax", the default,
-or "sigmoid": each router logit's own sigmoid), group_rank (a group's score is the sum of its so many best
+"sigmoid": each router logit's own sigmoid, or "chosen": the choice is made by the logits themselves and the weights
+are the softmax over the chosen logits alone), group_rank (a group's score is the sum of its so many best
 scores; default 1, its best), normalize (default true; false: the weights are the chosen experts' scores as
 they are), limit and alpha (with a limit an expert's unit is g' * sigmoid(alpha g') * (u' + 1) with
 g' = min(gate h, limit), u' = clamp(up h, -limit, limit), instead of silu(gate h) * (up h)), unit ("gated", the
-default; "gelu_erf" or "silu": experts WITHOUT a gate, down(act(up h)), act the exact (erf) GELU or the SiLU; such
+default; "gelu_erf", "silu" or "squared_relu": experts WITHOUT a gate, down(act(up h)), act the exact (erf) GELU, the SiLU or
+max(u, 0)^2; such
 experts have no ``gate_<e>`` / ``shared_gate`` tensors).
-Tensors: router [experts + identity, width] and correction [experts + identity] in float32, per
+Tensors: router [experts + identity, width], optional router_bias [experts + identity] (added to the logits) and optional correction [experts + identity] in float32, per
 expert gate / up [ff, width] and down [width, ff] (``gate_<e>``, ``up_<e>``, ``down_<e>``), and for the
 shared expert shared_gate / shared_up / shared_down and, optionally, shared_mix [1, width] (without it the shared
 expert's output is added as it is).
@@ -59,12 +61,12 @@ class RoutedExperts(FeedForward):
         self.limit = float(p["limit"]) if p.get("limit") is not None else None
         self.alpha = float(p.get("alpha", 1.0))
         self.unit = p.get("unit", "gated")
-        if self.unit not in ("gated", "gelu_erf", "silu"):
+        if self.unit not in ("gated", "gelu_erf", "silu", "squared_relu"):
             raise ValueError(f"routed experts: unknown unit {self.unit!r}")
         if self.unit != "gated" and self.limit is not None:
             raise ValueError("routed experts: the clamped unit has a gate")
         self.gated = self.unit == "gated"
-        if self.score not in ("softmax", "sigmoid"):
+        if self.score not in ("softmax", "sigmoid", "chosen") or (self.score == "chosen" and not self.normalize):
             raise ValueError(f"routed experts: unknown score {self.score!r}")
         if self.limit is not None and not self.limit > 0.0:
             raise ValueError(f"routed experts: the limit {self.limit} must be positive")
@@ -75,7 +77,10 @@ class RoutedExperts(FeedForward):
                                 or self.keep * (self.outputs // self.groups) < self.top):
             raise ValueError(f"routed experts: {self.groups} groups of which {self.keep} stay open do not fit "
                              f"{self.outputs} experts of which a token uses {self.top}")
-        self.router, self.correction = tensors["router"], tensors.get("correction")
+        self.router, self.correction, self.router_bias = tensors["router"], tensors.get("correction"), tensors.get("router_bias")
+        if self.router_bias is not None and (tuple(self.router_bias.shape) != (self.outputs,) or self.router_bias.dtype != torch.float32):
+            raise ValueError(f"routed experts: the router's bias is {tuple(self.router_bias.shape)} {self.router_bias.dtype}, "
+                             f"expected {(self.outputs,)} in float32")
         if tuple(self.router.shape) != (self.outputs, self.width) or self.router.dtype != torch.float32:
             raise ValueError(f"routed experts: the router is {tuple(self.router.shape)} {self.router.dtype}, expected "
                              f"{(self.outputs, self.width)} in float32")
@@ -122,7 +127,7 @@ class RoutedExperts(FeedForward):
         weights = step.buffer("experts.weights", tokens, self.outputs, "float32")
         mix = step.buffer("experts.mix", tokens, 1, "float32") if self.shared_mix is not None else None
         K.route(h, self.router, self.correction, self.top, self.groups, self.keep, weights, self.shared_mix, mix,
-                score=self.score, group_rank=self.group_rank, normalize=self.normalize)
+                score=self.score, group_rank=self.group_rank, normalize=self.normalize, bias=self.router_bias)
         fused = step.buffer("experts.fused", tokens, self.fused_cols, step.dtype)
         K.gemm(h, self.in_weight, K.epilogue_store(fused), packed=self.in_packed)
         hidden = step.buffer("experts.hidden", tokens, self.hidden_cols, step.dtype)

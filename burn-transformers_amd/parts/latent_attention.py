@@ -3,12 +3,15 @@ turned by position and shared by all heads.
 
 Parameters: width, heads, dim (query/key size per head), vdim (value size per head), q_rank,
 kv_rank, scale (multiplies q.k), eps (of the two latent norms), window (default 0: every earlier key; else the
-latest so many positions), rot_dim (default 0), rot_base, rot_scaling, rot_pairing ("neighbours", the default, or
+latest so many positions), keep (default 0: the first so many positions are seen beside the window), gate (how an
+optional tensor ``gate`` acts: "channel", the default, or "head"), borrows (default false; true: the mixer has no
+down_kv and kv_norm and attends over the latent and the turned key part that ANOTHER layer keeps, of the same kv_rank,
+rot_dim and rotation; its run's schedule entry reads that layer's cache entry), rot_dim (default 0), rot_base, rot_scaling, rot_pairing ("neighbours", the default, or
 "halves"; frequencies and pairing as in ``parts/rotary_attention.py``).  Tensors, all [out, in]:
 down_q [q_rank, width], q_norm [q_rank], up_q [heads*(dim + rot_dim), q_rank] (per head its dim plain rows, then
 its rot_dim turned rows), down_kv [kv_rank + rot_dim, width] (the latent's rows, then the shared turned key part's,
 which is not normalised), kv_norm [kv_rank], up_k [heads*dim, kv_rank], up_v [heads*vdim, kv_rank], optional
-gate [heads*vdim, width], out_weight [width, heads*vdim].
+gate [heads*vdim, width] ([heads, width]: one gate a head), out_weight [width, heads*vdim].
 
 With rot_dim > 0 a head's score is q_plain . k_plain + turn(q_turned) . turn(k_shared): the cached head is
 [c; turn(k_shared)], its values c with zeros behind, and the absorbed query of head i is
@@ -23,7 +26,7 @@ of the attention kernels (all heads of a token read each cached vector once).  T
 up_k_i^T up_q_i is formed once when the part is built (in float64, rounded to the products' type).
 
 One step: a fused product [down_q; down_kv; gate] h (32-bit sums) -> the two norms, c straight into
-the paged cache -> absorbed queries (one product) -> attention over the cache -> per head up_v and
+the paged cache (a borrowing mixer: [down_q; gate] h and the one norm) -> absorbed queries (one product) -> attention over the cache -> per head up_v and
 sigmoid gate -> output projection (the sublayer's output).
 """
 
@@ -31,7 +34,7 @@ import torch
 
 from ..cache.storage import KVSpec
 from ..kernels import library as K
-from .attention import CausalSelfAttention
+from .attention import CausalSelfAttention, keys_in_reach
 from .base import Mixer, compute_units, operand_columns, packed_for_stream, pad_columns, pad_rows
 from .registry import register
 from .rotary_attention import rotary_amplitude, rotary_frequencies
@@ -48,17 +51,21 @@ class LatentAttention(Mixer):
         self.q_rank, self.kv_rank = p["q_rank"], p["kv_rank"]
         self.scale, self.eps = float(p["scale"]), float(p["eps"])
         self.window, self.rot_dim = int(p.get("window") or 0), int(p.get("rot_dim") or 0)
+        self.keep, self.borrows = int(p.get("keep") or 0), bool(p.get("borrows"))
         self.neighbours = {"halves": False, "neighbours": True}[p.get("rot_pairing", "neighbours")]
         if self.rot_dim % 2 != 0:
             raise ValueError(f"latent attention: {self.rot_dim} turned channels must be even")
-        self.gated = "gate" in tensors
+        self.gated, self.gate_span = "gate" in tensors, p.get("gate", "channel")
+        gate_rows = {"channel": self.heads * self.vdim, "head": self.heads}[self.gate_span] if self.gated else 0
         shapes = {"down_q": (self.q_rank, self.width), "q_norm": (self.q_rank,),
                   "up_q": (self.heads * (self.dim + self.rot_dim), self.q_rank),
                   "down_kv": (self.kv_rank + self.rot_dim, self.width),
                   "kv_norm": (self.kv_rank,), "up_k": (self.heads * self.dim, self.kv_rank),
                   "up_v": (self.heads * self.vdim, self.kv_rank), "out_weight": (self.width, self.heads * self.vdim)}
         if self.gated:
-            shapes["gate"] = (self.heads * self.vdim, self.width)
+            shapes["gate"] = (gate_rows, self.width)
+        if self.borrows:
+            del shapes["down_kv"], shapes["kv_norm"]
         for role, shape in shapes.items():
             if tuple(tensors[role].shape) != shape:
                 raise ValueError(f"latent attention: {role} is {tuple(tensors[role].shape)}, expected {shape}")
@@ -75,14 +82,14 @@ class LatentAttention(Mixer):
         # segments of the fused first product, each padded so that the next starts where 16-byte loads may
         self.q_cols = operand_columns(self.q_rank, dtype)
         self.kv_offset = (self.q_rank + 3) // 4 * 4
-        self.gate_offset = self.kv_offset + (self.kv_rank + self.rot_dim + 3) // 4 * 4
-        self.fused_cols = self.gate_offset + (self.heads * self.vdim if self.gated else 0)
-        self.fused_weight = torch.cat([pad_rows(tensors["down_q"], self.kv_offset),
-                                       pad_rows(tensors["down_kv"], self.gate_offset - self.kv_offset)] +
+        self.gate_offset = self.kv_offset + (0 if self.borrows else (self.kv_rank + self.rot_dim + 3) // 4 * 4)
+        self.fused_cols = self.gate_offset + gate_rows
+        self.fused_weight = torch.cat([pad_rows(tensors["down_q"], self.kv_offset)] +
+                                      ([pad_rows(tensors["down_kv"], self.gate_offset - self.kv_offset)] if not self.borrows else []) +
                                       ([tensors["gate"]] if self.gated else []))
         # (the rows it multiplies carry zero columns where the width is no multiple of what 16-byte loads take)
         self.fused_weight = pad_columns(self.fused_weight, operand_columns(self.width, dtype))
-        self.q_norm, self.kv_norm = tensors["q_norm"], tensors["kv_norm"]
+        self.q_norm, self.kv_norm = tensors["q_norm"], None if self.borrows else tensors["kv_norm"]
         # absorbed queries: rows i * head_dim .. of W are up_k_i^T up_q_i  ([kv_rank, q_rank]), and behind them
         # the head's turned rows of up_q as they are
         up_q = tensors["up_q"].double().view(self.heads, self.dim + self.rot_dim, self.q_rank)
@@ -108,7 +115,7 @@ class LatentAttention(Mixer):
         self.out_packed = packed_for_stream(self.out_weight) if on_gpu else None
 
     def kv_spec(self):
-        return KVSpec(1, self.head_dim, self.window)
+        return KVSpec(1, self.head_dim, self.window, keep=self.keep)
 
     def kernel_modules(self, dtype):
         names = ["latent"]
@@ -132,7 +139,7 @@ class LatentAttention(Mixer):
         compute unit.  Planned for the step's class of context, like the ordinary attention's."""
         if not step.decode:
             return 1
-        keys = min(step.context_limit, self.window + 32) if self.window else step.context_limit
+        keys = keys_in_reach(step.context_limit, self.window, 0, self.keep)
         pair_bytes = keys * self.head_dim * 2 * (2 if step.dtype_is_bf16 else 4)
         if pair_bytes <= self.SPLIT_BYTES:
             return 1
@@ -147,10 +154,10 @@ class LatentAttention(Mixer):
         fused = step.buffer("latent.fused", tokens, self.fused_cols, "float32")
         K.gemm(h, self.fused_weight, K.epilogue_f32(fused), packed=self.fused_packed)
         c_q = step.buffer("latent.query_latent", tokens, self.q_cols, step.dtype)
-        if not memory.writes:
-            raise ValueError("latent attention: every run keeps a cache entry of its own")
-        K.latent_norm(fused, self.q_rank, self.kv_offset, self.kv_rank, self.q_norm, self.kv_norm, self.eps, c_q,
-                      step.tok_seq, step.tok_pos, kv, step.dtype, rot_dim=self.rot_dim, inv_freq=self.inv_freq,
+        if memory.writes == self.borrows:
+            raise ValueError("latent attention: a mixer keeps a cache entry of its own, or borrows and reads another layer's")
+        K.latent_norm(fused, self.q_rank, self.kv_offset, 0 if self.borrows else self.kv_rank, self.q_norm, self.kv_norm, self.eps, c_q,
+                      step.tok_seq, step.tok_pos, kv, step.dtype, rot_dim=0 if self.borrows else self.rot_dim, inv_freq=self.inv_freq,
                       neighbours=self.neighbours, amplitude=self.amplitude)
         q = step.buffer("latent.queries", tokens, self.n_q, step.dtype)
         if self.rot_dim:         # the turned part of every head is rotated from the 32-bit sums
@@ -170,9 +177,9 @@ class LatentAttention(Mixer):
             partial = step.buffer("attention.partial", tokens * self.heads * prompt_runs, self.head_dim + 2, "float32")
         args = K.attention_args(q, ctx, kv, step.tok_seq, step.tok_pos, step.seq_off, step.seq_start, self.heads,
                                 step.n_seqs, step.max_count, self.scale, self.window, partial,
-                                runs=prompt_runs if prompt_runs > 1 else None)
+                                runs=prompt_runs if prompt_runs > 1 else None, keep=self.keep)
         K.attention(args, step.dtype, step.decode, impl="plain" if self.plain_only else "auto")
         mixed = step.buffer("latent.mixed", tokens, self.mixed_cols, step.dtype)
         K.head_project(ctx, self.up_v, self.heads, self.vdim, self.kv_rank, self.head_dim, mixed,
-                       gate=fused[:, self.gate_offset:] if self.gated else None)
+                       gate=fused[:, self.gate_offset:] if self.gated else None, gate_span=self.gate_span)
         stream.add_product(step, mixed, self.out_weight, packed=self.out_packed)

@@ -4,7 +4,7 @@ positions (rotary positions), with grouped heads over the paged cache.
 Parameters (all from the plan): width, heads, kv_heads, dim (a query's and a key's head size), vdim
 (a value's head size, which may differ), scale (multiplies q.k), eps (of the head norms), head_norm
 (whether queries and keys are divided by their root mean square per head, times the scales
-``q_norm`` / ``k_norm`` [dim] that all heads share), rot_dims (the first so many channels of every
+``q_norm`` / ``k_norm`` [dim] that all heads share; norm_scale False: without such scales), rot_dims (the first so many channels of every
 query and key head are turned, channel i with channel i + rot_dims / 2, by the angle position *
 f_i), rot_base (f_i = rot_base^(-2 i / rot_dims)), rot_scaling (None, or factor / low / high /
 original: frequencies whose wavelength is beyond original / low are divided by factor, those whose
@@ -15,7 +15,7 @@ pairs up to turns(fast) are kept, pairs from turns(slow) on are divided by facto
 between, and every sine and cosine is multiplied by 0.1 ln(factor) + 1), rot_pairing ("halves", the default: channel i with channel i + rot_dims / 2;
 "neighbours": channel 2 i with channel 2 i + 1), norm_span ("head", the default; "whole": the root mean square
 is taken over a token's whole query (key) projection before it is split into heads, and the scales ``q_norm`` /
-``k_norm`` are [heads * dim] / [kv_heads * dim]), window and chunk (which earlier keys a query sees, as in
+``k_norm`` are [heads * dim] / [kv_heads * dim]), window, chunk and keep (which earlier keys a query sees, as in
 ``parts/attention.py``), taps (default 0; with taps > 0 every channel of the query, key and value projections
 passes a short causal convolution over its sequence's tokens, tensors ``q_conv`` / ``k_conv`` / ``v_conv``
 [channels, taps], the last tap meeting the current token, no bias, no activation, before norms and rotation;
@@ -91,6 +91,7 @@ class RotaryAttention(CausalSelfAttention):
         self.dim, self.vdim = p["dim"], p["vdim"]
         self.scale, self.eps = float(p["scale"]), float(p.get("eps", 0.0))
         self.window, self.chunk = int(p.get("window") or 0), int(p.get("chunk") or 0)
+        self.keep = int(p.get("keep") or 0)
         self.rot_dims = int(p.get("rot_dims") or 0)
         if self.heads % self.kv_heads != 0:
             raise ValueError(f"rotary attention: {self.heads} query heads cannot share {self.kv_heads} key/value heads")
@@ -120,7 +121,8 @@ class RotaryAttention(CausalSelfAttention):
             shapes["gate_weight"] = (self.gate_cols, self.width)
         self.neighbours = {"halves": False, "neighbours": True}[p.get("rot_pairing", "halves")]
         self.whole_norm = {"head": False, "whole": True}[p.get("norm_span", "head")]
-        if p.get("head_norm", True):
+        scaled = bool(p.get("norm_scale", True))
+        if p.get("head_norm", True) and scaled:
             shapes.update(q_norm=(n_qk[0],), k_norm=(n_qk[1],)) if self.whole_norm else \
                 shapes.update(q_norm=(self.dim,), k_norm=(self.dim,))
         if "sink" in tensors:
@@ -136,6 +138,10 @@ class RotaryAttention(CausalSelfAttention):
             if tuple(tensors[role].shape) != shape:
                 raise ValueError(f"rotary attention: {role} is {tuple(tensors[role].shape)}, expected {shape}")
         self.q_norm, self.k_norm = tensors.get("q_norm"), tensors.get("k_norm")
+        if p.get("head_norm", True) and not scaled:           # the kernel multiplies by ones, which is exact
+            q_scales, k_scales = n_qk if self.whole_norm else (self.dim, self.dim)
+            self.q_norm, self.k_norm = (torch.ones(count, dtype=torch.float32, device=tensors["q_weight"].device)
+                                        for count in (q_scales, k_scales))
         self.sink = tensors["sink"].float().contiguous() if "sink" in tensors else None
         self.score_bias = tensors["score_bias"].float().contiguous() if self.sigmoid else None
         dtype = tensors["q_weight"].dtype
@@ -258,6 +264,6 @@ class RotaryAttention(CausalSelfAttention):
             partial = step.buffer("attention.partial", q.shape[0] * self.q_heads * prompt_runs, self.head_dim + 2, "float32")
         args = K.attention_args(q, out, kv, step.tok_seq, step.tok_pos, step.seq_off, step.seq_start,
                                 self.q_heads, step.n_seqs, step.max_count, self.scale, self.window, partial,
-                                runs=prompt_runs if prompt_runs > 1 else None, chunk=self.chunk, sink=self.sink, softcap=self.softcap, sigmoid=self.sigmoid,
+                                runs=prompt_runs if prompt_runs > 1 else None, chunk=self.chunk, keep=self.keep, sink=self.sink, softcap=self.softcap, sigmoid=self.sigmoid,
                                 score_bias=self.score_bias, gate=gate, gate_dim=self.vdim if self.gate_kind == "channel" else 0)
         K.attention(args, step.dtype, step.decode, impl="plain" if plain else "auto")

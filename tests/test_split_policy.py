@@ -52,11 +52,11 @@ def test_a_folded_norm_is_worth_it_by_rows_and_width():
 
 # --- the runs a decode step's keys are cut into, and the classes of context ---------------------
 
-def _runs(monkeypatch, n_seqs, context_limit, kv_heads=25, head_dim=64, bf16=True, window=0, decode=True, units=256, chunk=0):
+def _runs(monkeypatch, n_seqs, context_limit, kv_heads=25, head_dim=64, bf16=True, window=0, decode=True, units=256, chunk=0, keep=0):
     from types import SimpleNamespace
     from burn_transformers_amd.parts import attention
     monkeypatch.setattr(attention, "compute_units", lambda device: units)
-    mixer = SimpleNamespace(kv_heads=kv_heads, head_dim=head_dim, window=window, chunk=chunk)
+    mixer = SimpleNamespace(kv_heads=kv_heads, head_dim=head_dim, window=window, chunk=chunk, keep=keep)
     step = SimpleNamespace(decode=decode, context_limit=context_limit, dtype_is_bf16=bf16, n_seqs=n_seqs)
     return attention.CausalSelfAttention.decode_runs(mixer, step, "cuda:0")
 
