@@ -1,7 +1,7 @@
 """Throughput of GPT-2 generation on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--layers 48] [--dtype bf16]
-                    [--repetitions 10] [--workload xl|small|medium|sweep|salopel|kodatar|rotutar|gavasun|loselix] [--model xl|medium|small]
+                    [--repetitions 10] [--workload xl|small|medium|sweep|salopel|kodatar|rotutar|gavasun|loselix|rirovik] [--model xl|medium|small]
                     [--kernel-batches 1,64] [--sweep-part all|decode|prompts] [--no-points] [--no-kernels] [--no-own]
 
 The default workload (``xl``) has the layer sizes of GPT-2 XL with random weights: a batch of 8
@@ -58,6 +58,9 @@ the library's closest family, at equal width, layers and vocabulary.
 ``--workload loselix`` runs the sixth family, Loselix (differential attention with capped scores, attention with a gate per
 head, sigmoid attention on its own keys, mixer and feed-forward side by side, a stretch of layers that runs twice), beside
 GPT-2 (whole contexts, dense feed-forwards) at equal width, runs of layers, feed-forward and vocabulary.
+``--workload rirovik`` runs the seventh family, Rirovik (attention in a window that keeps the first tokens, latent attention
+over whole contexts, in a window and on a borrowed latent, a norm before and behind every sublayer, ungated experts), beside
+Gavasun, the library's closest family, at equal width, layers, experts and vocabulary.
 """
 
 import argparse
@@ -665,6 +668,35 @@ def loselix_config(width, layers, vocab):
                        for i in range(layers - third)]}
 
 
+def rirovik_config(width, layers, vocab):
+    """Rirovik at layer sizes that resemble a real model's: groups of four layers (attention in a window of 512 that keeps
+    the first 64 tokens, latent attention over the whole context, latent attention in a window of 512, and one that borrows
+    the latter's latent), all with experts; heads of 128, the attention's on a quarter as many key/value heads; the latent
+    attentions' heads of 128 plain and 32 turned channels on a key/value latent of 96 (a cached head of 128) and a query
+    latent of 3/8 of the width; eight experts of the model's width of which a token uses two, and one every token uses."""
+    heads = max(4, width // 128)
+    attention = {"heads": heads, "kv_heads": heads // 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                 "mask": {"size": 512, "keep_first": 64}}
+    whole = {"heads": min(heads, 16), "dim": 128, "rot_dim": 32, "vdim": 128, "q_rank": 3 * width // 8, "kv_rank": 96,
+             "scale": 160 ** -0.5, "rot": {"dims": 32, "base": 500000.0}}
+    window = dict(whole, mask={"size": 512})
+    experts = {"kind": "moe", "expert": {"ff": width}, "router": {"experts": 8, "top": 2}, "shared": {"ff": width}}
+    group = [("attention", attention), ("latent_attention_2", whole), ("latent_attention", window), ("latent_attention", window)]
+    return {"architecture": "Rirovik", "vocab": vocab, "width": width, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-5},
+            "layers": [{"type": group[i % 4][0], "mixer": dict(group[i % 4][1], **({"kv_from": i - 1} if i % 4 == 3 else {})),
+                        "mlp": experts} for i in range(layers)]}
+
+
+def run_rirovik(args):
+    """Rirovik beside the library's closest family, Gavasun (latent attention with a shared turned key part, attention on
+    grouped heads, ungated experts), at equal width, layers, experts and vocabulary."""
+    def values_and_columns(attention):
+        return 2 * attention.kv.head_dim * attention.kv.kv_heads, attention.q_heads * attention.kv.head_dim
+    heads = lambda width: max(4, width // 128)
+    run_beside_gpt2(args, "rirovik", rirovik_config, None, of_call=values_and_columns,
+                    other=("gavasun", gavasun_config, lambda width: (2 * 128 * (heads(width) // 4), 128 * heads(width))))
+
+
 def run_loselix(args):
     """Loselix beside GPT-2 at equal width, runs of layers, feed-forward and vocabulary."""
     def values_and_columns(attention):
@@ -776,7 +808,7 @@ def main():
     parser.add_argument("--kernel-batches", default="", help="further batch sizes whose decode kernel classes are timed, e.g. 1,64")
     parser.add_argument("--dtype", choices=["bf16", "fp32"], default=None)
     parser.add_argument("--repetitions", type=int, default=10, help="measured repetitions, each on fresh sequences")
-    parser.add_argument("--workload", choices=["xl", "small", "medium", "sweep", "salopel", "kodatar", "rotutar", "gavasun", "loselix"], default="xl")
+    parser.add_argument("--workload", choices=["xl", "small", "medium", "sweep", "salopel", "kodatar", "rotutar", "gavasun", "loselix", "rirovik"], default="xl")
     parser.add_argument("--sweep-part", choices=["all", "decode", "prompts"], default="all",
                         help="which table of --workload sweep to run")
     parser.add_argument("--no-points", action="store_true", help="skip batch 1 and 64")
@@ -789,7 +821,8 @@ def main():
     if args.repetitions < 1:
         parser.error("--repetitions must be at least 1")
     args.kernel_batches = [int(b) for b in args.kernel_batches.split(",") if b]
-    families = {"salopel": run_salopel, "kodatar": run_kodatar, "rotutar": run_rotutar, "gavasun": run_gavasun, "loselix": run_loselix}
+    families = {"salopel": run_salopel, "kodatar": run_kodatar, "rotutar": run_rotutar, "gavasun": run_gavasun, "loselix": run_loselix,
+                "rirovik": run_rirovik}
     if args.workload in families:
         families[args.workload](args)
         return

@@ -14,7 +14,11 @@ enum EpilogueMode {
   EPI_RESIDUAL = 4,  // out[m][n] += acc + bias                  (float: the residual stream itself)
   EPI_F32_ACT = 5,   // columns [0,n_q) -> out as in EPI_F32, those behind -> act(acc + bias) in out2 (element type T), columns
                      //   from 0: two products of the same rows as one (the skinny kernel only)
+  EPI_TURN = 6,      // out[m][n] = acc, of every turn_pitch columns the turn_dim from turn_at on rotated in neighbouring pairs
+                     //   by the row's position (element type T; the skinny kernel only)
 };
+// What the skinny kernel is built for: the common modes, or one of the two that are forms of the kernel of their own.
+enum EpilogueKind { EPILOGUE_COMMON = 0, EPILOGUE_TWO = 1, EPILOGUE_TURN = 2 };
 
 enum Activation {
   ACT_GELU_TANH = 0,
@@ -38,6 +42,11 @@ struct Epilogue {
   int out_rows;          // EPI_STORE, EPI_ACT (EPI_F32_ACT: `out2`): 0, or `out` is chunk-major with that many rows (activation_offset)
   void* out2;            // EPI_F32_ACT only
   int64_t ldo2;
+  // EPI_TURN: columns turn_at + 2 i and turn_at + 2 i + 1 of a head of turn_pitch (a multiple of four; turn_at and turn_dim
+  // even) turn by the angle tok_pos[m] * inv_freq[i], sine and cosine times `amplitude`
+  int turn_pitch, turn_at, turn_dim;
+  float amplitude;
+  const float* inv_freq;
 };
 
 // 32-bit activations.  The float32 path (T = float) uses the library's tanhf / erff; the
@@ -88,6 +97,7 @@ __device__ __forceinline__ void store4<bf16_t>(bf16_t* dst, const float* v, int 
 // value of the residual stream in EPI_RESIDUAL) and, for the key/value scatter, where the row's
 // token lives in the paged cache.
 struct EpiloguePrefetch {
+  float freq[2];     // EPI_TURN: the frequencies of the two pairs (0: not turned)
   float add[4];
   int64_t kv_base;   // start of the (block, head) plane of the token; valid for key/value columns
   int pos;
@@ -132,18 +142,44 @@ __device__ __forceinline__ EpiloguePrefetch epilogue_prefetch(const Epilogue& e,
   return p;
 }
 
-// The epilogue with everything but the accumulators already in registers.  TWO: the mode is EPI_F32_ACT (a form of the
-// kernel of its own, so that the others carry none of it).
-template <typename T, bool TWO = false>
+// The same for EPI_TURN: the row's position and the frequencies of the two pairs.
+__device__ __forceinline__ EpiloguePrefetch epilogue_prefetch_turn(const Epilogue& e, int M, int m, int n0) {
+  EpiloguePrefetch p = {};
+  p.pos = e.tok_pos[m < M ? m : M - 1];
+  const int j = n0 % e.turn_pitch - e.turn_at;       // (even: the pairs of four columns are 0, 1 and 2, 3)
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const bool turned = j + 2 * i >= 0 && j + 2 * i < e.turn_dim;
+    const float f = e.inv_freq[turned ? (j + 2 * i) >> 1 : 0];
+    p.freq[i] = turned ? f : 0.f;
+    p.add[i] = turned ? e.amplitude : 1.f;
+  }
+  return p;
+}
+
+// The epilogue with everything but the accumulators already in registers.  KIND: EPI_F32_ACT and EPI_TURN are forms of
+// the kernel of their own, so that the others carry none of them.
+template <typename T, int KIND = EPILOGUE_COMMON>
 __device__ __forceinline__ void epilogue4_prefetched(const Epilogue& e, int N, int m, int n0, const float* acc,
                                                      int split, const EpiloguePrefetch& p) {
   int count = N - n0 < 4 ? N - n0 : 4;
   if (count <= 0) return;
   float v[4];
+  bool aligned = (e.ldo & 3) == 0;
+  if constexpr (KIND == EPILOGUE_TURN) {
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      float sn = 0.f, cs = 1.f;
+      if (p.freq[i] != 0.f) sincosf((float)p.pos * p.freq[i], &sn, &cs);
+      v[2 * i] = p.add[i] * (acc[2 * i] * cs - acc[2 * i + 1] * sn);
+      v[2 * i + 1] = p.add[i] * (acc[2 * i + 1] * cs + acc[2 * i] * sn);
+    }
+    store4<T>(static_cast<T*>(e.out) + (int64_t)m * e.ldo + n0, v, count, aligned);
+    return;
+  }
 #pragma unroll
   for (int i = 0; i < 4; ++i) v[i] = acc[i] + p.add[i];
-  bool aligned = (e.ldo & 3) == 0;
-  if constexpr (TWO) {
+  if constexpr (KIND == EPILOGUE_TWO) {
     if (n0 < e.n_q) {
       store4<float>(static_cast<float*>(e.out) + (int64_t)m * e.ldo + n0, v, count, aligned);
     } else {

@@ -17,6 +17,8 @@
 // A third kind of score makes the choice by the logits themselves (with the correction) and weighs the chosen
 // experts by the softmax over THEIR logits alone.  `bias` is added to the logits first.
 // Ties between equal scores go to the lower index.
+//   * weighed experts, for small steps: the router's logits come from the product that makes the experts' units (rows of
+//     the same matrix, 32-bit results), and ONE kernel makes the choice and multiplies the units by their weights.
 #include "host.h"
 
 #define ROUTE_THREADS 1024
@@ -51,93 +53,37 @@ __device__ __forceinline__ void wave_best(float& value, int& index) {
   }
 }
 
-// One work-group of sixteen waves per token.  Logits: a wave takes whole outputs (two at a time, the
-// outputs dealt round the waves), its lanes the columns, sixteen a turn; nothing of a turn's loads stands
-// behind a branch of its own, so all of them are in flight together, every wave's at once: the
-// logits cost one round trip to memory and a wave reduction, and no sum crosses waves.  (Columns
-// dealt to the threads and sixteen outputs' sums met through LDS, batch after batch, took 6 us a batch
-// of sixteen outputs: a decode step has few tokens, and a kernel's time is the chain of its waits.)
-// Everything after the logits is the first wave's alone, the experts dealt to its lanes, maxima and
-// choices as wave reductions: no barrier, no serial scan.
-#define ROUTE_OUTPUTS 2         // outputs whose sums a wave carries at once
-#define ROUTE_COLUMNS 16        // columns of a lane and turn
-
-template <typename T>
-__global__ void __launch_bounds__(ROUTE_THREADS) route_kernel(RouteCall c) {
-  __shared__ float score[ROUTE_MAX_EXPERTS];      // logits, then softmax scores
-  __shared__ float choice[ROUTE_MAX_EXPERTS];     // scores with the correction; +inf once taken, -inf where shut out
-  __shared__ float gate_sum;
-  const int t = blockIdx.x, lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const T* h = static_cast<const T*>(c.h) + (int64_t)t * c.ldh;
-  const int outputs = c.experts + (c.gate_w ? 1 : 0);
-  const int waves = blockDim.x >> 6;              // sixteen in steps of few tokens, four where tokens fill the chip anyway
-  // the corrections of this lane's first experts are asked for now, with the first loads
-  float early_correction[4] = {0.f, 0.f, 0.f, 0.f};
-  if (wave == 0 && c.correction)
+// Corrections and biases of a lane's first four experts.
+struct RouteEarly {
+  float correction[4], bias[4];
+  __device__ __forceinline__ void load(const RouteCall& c) {
+    const int lane = threadIdx.x & 63;
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
-      if (lane + 64 * j < c.experts) early_correction[j] = c.correction[lane + 64 * j];
-  float early_bias[4] = {0.f, 0.f, 0.f, 0.f};
-  if (wave == 0 && c.bias)
-#pragma unroll
-    for (int j = 0; j < 4; ++j)
-      if (lane + 64 * j < c.experts) early_bias[j] = c.bias[lane + 64 * j];
-  for (int first = wave; first < outputs; first += waves * ROUTE_OUTPUTS) {
-    float sums[ROUTE_OUTPUTS];
-    const float* rows[ROUTE_OUTPUTS];               // an output beyond the last reads the last one's row and is dropped
-#pragma unroll
-    for (int j = 0; j < ROUTE_OUTPUTS; ++j) {
-      sums[j] = 0.f;
-      const int e = first + waves * j < outputs ? first + waves * j : outputs - 1;
-      rows[j] = e < c.experts ? c.W + (int64_t)e * c.width : c.gate_w;
-    }
-    for (int col0 = lane; col0 < c.width; col0 += 64 * ROUTE_COLUMNS) {
-      int cc[ROUTE_COLUMNS];
-      float xs[ROUTE_COLUMNS];
-#pragma unroll
-      for (int u = 0; u < ROUTE_COLUMNS; ++u) {
-        const int col = col0 + 64 * u;
-        cc[u] = col < c.width ? col : 0;
-        xs[u] = to_float(h[cc[u]]);
-      }
-      float ws[ROUTE_OUTPUTS][ROUTE_COLUMNS];
-#pragma unroll
-      for (int j = 0; j < ROUTE_OUTPUTS; ++j)
-#pragma unroll
-        for (int u = 0; u < ROUTE_COLUMNS; ++u) ws[j][u] = rows[j][cc[u]];
-#pragma unroll
-      for (int u = 0; u < ROUTE_COLUMNS; ++u) xs[u] = col0 + 64 * u < c.width ? xs[u] : 0.f;
-#pragma unroll
-      for (int j = 0; j < ROUTE_OUTPUTS; ++j)
-#pragma unroll
-        for (int u = 0; u < ROUTE_COLUMNS; ++u) sums[j] = fmaf(ws[j][u], xs[u], sums[j]);
-    }
-#pragma unroll
-    for (int j = 0; j < ROUTE_OUTPUTS; ++j) {
-      const float sum = wave_sum(sums[j]);
-      const int e = first + waves * j;
-      if (lane == 0 && e < outputs) {
-        if (e < c.experts) score[e] = sum;
-        else gate_sum = sum;                         // (stored at the end: nothing waits for a store meanwhile)
-      }
+    for (int j = 0; j < 4; ++j) {
+      correction[j] = c.correction && lane + 64 * j < c.experts ? c.correction[lane + 64 * j] : 0.f;
+      bias[j] = c.bias && lane + 64 * j < c.experts ? c.bias[lane + 64 * j] : 0.f;
     }
   }
-  __syncthreads();
-  if (wave != 0) return;
+};
+
+// From a token's logits to its experts, by ONE wave: the experts dealt to its lanes, maxima and choices as wave
+// reductions.  `score` holds the logits and afterwards the scores, `choice` afterwards +inf where an expert was chosen
+// (both in LDS).  Returns the factor on the chosen experts' scores.
+__device__ __forceinline__ float route_choice(const RouteCall& c, const RouteEarly& early, float* score, float* choice) {
+  const int lane = threadIdx.x & 63;
   if (c.bias)                                       // a lane keeps to its own experts
-    for (int e = lane, j = 0; e < c.experts; e += 64, ++j) score[e] += j < 4 ? early_bias[j < 4 ? j : 0] : c.bias[e];
+    for (int e = lane, j = 0; e < c.experts; e += 64, ++j) score[e] += j < 4 ? early.bias[j < 4 ? j : 0] : c.bias[e];
   float top_logit = -INFINITY;
   for (int e = lane; e < c.experts; e += 64) top_logit = fmaxf(top_logit, score[e]);
   top_logit = wave_max(top_logit);
   float total = 0.f;
   for (int e = lane; e < c.experts; e += 64) total += expf(score[e] - top_logit);
   total = wave_sum(total);
-  float* weights = c.weights + (int64_t)t * c.experts;
   for (int e = lane, j = 0; e < c.experts; e += 64, ++j) {     // a lane keeps to its own experts: no other lane reads them yet
     const float z = score[e];
     const float s = c.score == 1 ? 1.0f / (1.0f + expf(-z)) : c.score == 2 ? expf(z - top_logit) : expf(z - top_logit) / total;
     score[e] = s;
-    choice[e] = (c.score == 2 ? z : s) + (c.correction ? (j < 4 ? early_correction[j < 4 ? j : 0] : c.correction[e]) : 0.f);
+    choice[e] = (c.score == 2 ? z : s) + (c.correction ? (j < 4 ? early.correction[j < 4 ? j : 0] : c.correction[e]) : 0.f);
   }
   __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
   __builtin_amdgcn_wave_barrier();
@@ -203,25 +149,99 @@ __global__ void __launch_bounds__(ROUTE_THREADS) route_kernel(RouteCall c) {
     __builtin_amdgcn_wave_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
   }
+  return c.normalize ? 1.0f / (sum + 1e-20f) : 1.0f;
+}
+
+// One work-group of sixteen waves per token.  Logits: a wave takes whole outputs (two at a time, the
+// outputs dealt round the waves), its lanes the columns, sixteen a turn; nothing of a turn's loads stands
+// behind a branch of its own, so all of them are in flight together, every wave's at once: the
+// logits cost one round trip to memory and a wave reduction, and no sum crosses waves.  (Columns
+// dealt to the threads and sixteen outputs' sums met through LDS, batch after batch, took 6 us a batch
+// of sixteen outputs: a decode step has few tokens, and a kernel's time is the chain of its waits.)
+// Everything after the logits is the first wave's alone, the experts dealt to its lanes, maxima and
+// choices as wave reductions: no barrier, no serial scan.
+#define ROUTE_OUTPUTS 2         // outputs whose sums a wave carries at once
+#define ROUTE_COLUMNS 16        // columns of a lane and turn
+
+template <typename T>
+__global__ void __launch_bounds__(ROUTE_THREADS) route_kernel(RouteCall c) {
+  __shared__ float score[ROUTE_MAX_EXPERTS];      // logits, then softmax scores
+  __shared__ float choice[ROUTE_MAX_EXPERTS];     // scores with the correction; +inf once taken, -inf where shut out
+  __shared__ float gate_sum;
+  const int t = blockIdx.x, lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const T* h = static_cast<const T*>(c.h) + (int64_t)t * c.ldh;
+  const int outputs = c.experts + (c.gate_w ? 1 : 0);
+  const int waves = blockDim.x >> 6;              // sixteen in steps of few tokens, four where tokens fill the chip anyway
+  // the corrections and biases of this lane's first experts are asked for now, with the first loads
+  RouteEarly early;
+  if (wave == 0) early.load(c);
+  for (int first = wave; first < outputs; first += waves * ROUTE_OUTPUTS) {
+    float sums[ROUTE_OUTPUTS];
+    const float* rows[ROUTE_OUTPUTS];               // an output beyond the last reads the last one's row and is dropped
+#pragma unroll
+    for (int j = 0; j < ROUTE_OUTPUTS; ++j) {
+      sums[j] = 0.f;
+      const int e = first + waves * j < outputs ? first + waves * j : outputs - 1;
+      rows[j] = e < c.experts ? c.W + (int64_t)e * c.width : c.gate_w;
+    }
+    for (int col0 = lane; col0 < c.width; col0 += 64 * ROUTE_COLUMNS) {
+      int cc[ROUTE_COLUMNS];
+      float xs[ROUTE_COLUMNS];
+#pragma unroll
+      for (int u = 0; u < ROUTE_COLUMNS; ++u) {
+        const int col = col0 + 64 * u;
+        cc[u] = col < c.width ? col : 0;
+        xs[u] = to_float(h[cc[u]]);
+      }
+      float ws[ROUTE_OUTPUTS][ROUTE_COLUMNS];
+#pragma unroll
+      for (int j = 0; j < ROUTE_OUTPUTS; ++j)
+#pragma unroll
+        for (int u = 0; u < ROUTE_COLUMNS; ++u) ws[j][u] = rows[j][cc[u]];
+#pragma unroll
+      for (int u = 0; u < ROUTE_COLUMNS; ++u) xs[u] = col0 + 64 * u < c.width ? xs[u] : 0.f;
+#pragma unroll
+      for (int j = 0; j < ROUTE_OUTPUTS; ++j)
+#pragma unroll
+        for (int u = 0; u < ROUTE_COLUMNS; ++u) sums[j] = fmaf(ws[j][u], xs[u], sums[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < ROUTE_OUTPUTS; ++j) {
+      const float sum = wave_sum(sums[j]);
+      const int e = first + waves * j;
+      if (lane == 0 && e < outputs) {
+        if (e < c.experts) score[e] = sum;
+        else gate_sum = sum;                         // (stored at the end: nothing waits for a store meanwhile)
+      }
+    }
+  }
+  __syncthreads();
+  if (wave != 0) return;
+  const float inverse = route_choice(c, early, score, choice);
   // the one store of a lane's experts: the chosen ones' scores over their sum, zero elsewhere
-  const float inverse = c.normalize ? 1.0f / (sum + 1e-20f) : 1.0f;
+  float* weights = c.weights + (int64_t)t * c.experts;
   for (int e = lane; e < c.experts; e += 64) weights[e] = choice[e] == INFINITY ? score[e] * inverse : 0.f;
   if (c.gate_w && lane == 0) c.gate[t] = 1.0f / (1.0f + expf(-gate_sum));
 }
 
-BT_EXPORT int bt_route_call(void* stream, const RouteCall* c) {
-  if (c->tokens <= 0) return BT_OK;
-  if (c->experts <= 0 || c->experts > ROUTE_MAX_EXPERTS) BT_REFUSE("route: %d experts outside 1..%d", c->experts, ROUTE_MAX_EXPERTS);
-  if (c->top <= 0 || c->top > c->experts || c->top > 64) BT_REFUSE("route: %d of %d experts a token (at most 64)", c->top, c->experts);
+static const char* route_refusal(const RouteCall* c) {
+  if (c->experts <= 0 || c->experts > ROUTE_MAX_EXPERTS) return "1 to 1024 experts are possible";
+  if (c->top <= 0 || c->top > c->experts || c->top > 64) return "a token uses 1 to 64 of the experts";
   if (c->groups > 1) {
     if (c->groups > 64 || c->experts % c->groups != 0 || c->keep <= 0 || c->keep > c->groups)
-      BT_REFUSE("route: %d groups (at most 64) must divide %d experts, and 1..groups of them stay open, not %d", c->groups, c->experts, c->keep);
-    if (c->keep * (c->experts / c->groups) < c->top)
-      BT_REFUSE("route: %d open groups of %d experts cannot give %d experts", c->keep, c->experts / c->groups, c->top);
+      return "the groups (at most 64) must divide the experts, and 1 to all of them stay open";
+    if (c->keep * (c->experts / c->groups) < c->top) return "the open groups hold fewer experts than a token uses";
   }
-  if (c->width <= 0) BT_REFUSE("route: width %d must be positive", c->width);
   if (c->score < 0 || c->score > 2 || (c->score == 2 && c->normalize != 1) || c->group_rank < 0 || (c->normalize != 0 && c->normalize != 1))
-    BT_REFUSE("route: score %d, group_rank %d, normalize %d: not a router this kernel knows", c->score, c->group_rank, c->normalize);
+    return "not a router these kernels know";
+  return nullptr;
+}
+
+BT_EXPORT int bt_route_call(void* stream, const RouteCall* c) {
+  if (c->tokens <= 0) return BT_OK;
+  if (const char* wrong = route_refusal(c))
+    BT_REFUSE("route: %d of %d experts a token, %d of %d groups, score %d: %s", c->top, c->experts, c->keep, c->groups, c->score, wrong);
+  if (c->width <= 0) BT_REFUSE("route: width %d must be positive", c->width);
   if (!c->h || !c->W || !c->weights || (c->gate_w && !c->gate)) BT_REFUSE("route: missing operand");
   // (measured at 2,048 tokens of width 2,048: 32 us with sixteen waves a token, 18 with four)
   dim3 grid(c->tokens), block(c->tokens <= 256 ? ROUTE_THREADS : 256);
@@ -312,6 +332,30 @@ __global__ void __launch_bounds__(256) gated_experts_kernel(GatedExpertsCall c) 
   }
 }
 
+// The same for units without a gate whose columns can be taken 16 bytes at a time: no piece lies in two experts.
+template <typename T>
+__global__ void __launch_bounds__(256) plain_experts_kernel(GatedExpertsCall c) {
+  typedef __attribute__((__vector_size__(4 * sizeof(int)))) int int4v;
+  constexpr int PER = 16 / sizeof(T);
+  const int t = blockIdx.x, routed = c.experts * c.ff / PER, pieces = c.hidden_cols / PER;
+  const int4v* up = reinterpret_cast<const int4v*>(static_cast<const T*>(c.gu) + (int64_t)t * c.ld_gu);
+  int4v* hidden = reinterpret_cast<int4v*>(static_cast<T*>(c.hidden) + (int64_t)t * c.ld_hidden);
+  const float* weights = c.weights + (int64_t)t * (c.experts + c.identity);
+  const float share = c.gate ? c.gate[t] : 1.0f;
+  const int all = (c.experts * c.ff + c.shared_ff) / PER;
+  for (int piece = blockIdx.y * blockDim.x + threadIdx.x; piece < pieces; piece += gridDim.y * blockDim.x) {
+    const float w = piece < routed ? weights[piece * PER / c.ff] : piece < all ? share : 0.f;
+    int4v v = {0, 0, 0, 0};
+    if (w != 0.f) {
+      v = up[piece];
+      T* values = reinterpret_cast<T*>(&v);
+#pragma unroll
+      for (int i = 0; i < PER; ++i) values[i] = from_float<T>(w * plain_unit(c, to_float(values[i])));
+    }
+    hidden[piece] = v;
+  }
+}
+
 BT_EXPORT int bt_gated_experts_call(void* stream, const GatedExpertsCall* c) {
   if (c->tokens <= 0) return BT_OK;
   if (c->experts < 0 || c->ff <= 0 || c->shared_ff < 0 || c->identity < 0)
@@ -326,9 +370,96 @@ BT_EXPORT int bt_gated_experts_call(void* stream, const GatedExpertsCall* c) {
   int per_token = (c->hidden_cols + 1023) / 1024;
   if (per_token > 64) per_token = 64;
   dim3 grid(c->tokens, per_token), block(256);
+  const int per = c->dtype == 0 ? 4 : 8;
+  if (c->act >= 2 && !c->identity_out && c->ff % per == 0 && c->shared_ff % per == 0 && c->hidden_cols % per == 0 && c->ld_gu % per == 0 &&
+      c->ld_hidden % per == 0 && ((uintptr_t)c->gu & 15) == 0 && ((uintptr_t)c->hidden & 15) == 0 && c->ld_gu >= c->hidden_cols) {
+    grid.y = (c->hidden_cols / per + 255) / 256;
+    if (grid.y > 64) grid.y = 64;
+    if (c->dtype == 0)
+      hipLaunchKernelGGL(plain_experts_kernel<float>, grid, block, 0, (hipStream_t)stream, *c);
+    else
+      hipLaunchKernelGGL(plain_experts_kernel<bf16_t>, grid, block, 0, (hipStream_t)stream, *c);
+    return bt_check_launch("gated_experts");
+  }
   if (c->dtype == 0)
     hipLaunchKernelGGL(gated_experts_kernel<float>, grid, block, 0, (hipStream_t)stream, *c);
   else
     hipLaunchKernelGGL(gated_experts_kernel<bf16_t>, grid, block, 0, (hipStream_t)stream, *c);
   return bt_check_launch("gated_experts");
+}
+
+// hidden[t][e * ff + i] *= the token's weight of expert e, for `experts` experts side by side, from the router's logits of
+// the token; columns behind them (an expert every token uses) stay.  A work-group makes the token's whole choice (its
+// first wave, a few reductions over the experts) and multiplies its share of the columns.
+struct WeighExpertsCall {
+  RouteCall route;          // dtype: element type of `hidden`; tokens, experts, top, groups, keep, correction, score, group_rank,
+                            // normalize, bias; nothing else is looked at
+  int ff;
+  const float* logits;      // [tokens][ld_logits]
+  int64_t ld_logits;
+  void* hidden;             // [tokens][ld_hidden]
+  int64_t ld_hidden;
+};
+
+template <typename T>
+__global__ void __launch_bounds__(256) weigh_experts_kernel(WeighExpertsCall w) {
+  __shared__ float score[ROUTE_MAX_EXPERTS], choice[ROUTE_MAX_EXPERTS];
+  __shared__ float factor;
+  typedef __attribute__((__vector_size__(4 * sizeof(int)))) int int4v;
+  constexpr int PER = 16 / sizeof(T);
+  const RouteCall& c = w.route;
+  const int t = blockIdx.x, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
+  T* hidden = static_cast<T*>(w.hidden) + (int64_t)t * w.ld_hidden;
+  const int columns = c.experts * w.ff;
+  const int pieces = (columns + PER - 1) / PER;
+  // (16 bytes at a time where no piece lies in two experts)
+  const bool whole = w.ff % PER == 0 && (w.ld_hidden % PER) == 0 && ((uintptr_t)w.hidden & 15) == 0;
+  int piece = blockIdx.y * blockDim.x + threadIdx.x;
+  int4v held = {0, 0, 0, 0};
+  if (whole && piece < pieces) held = *reinterpret_cast<const int4v*>(hidden + (int64_t)piece * PER);      // on its way during the choice
+  if (wave == 0) {
+    const float* logits = w.logits + (int64_t)t * w.ld_logits;
+    RouteEarly early;
+    early.load(c);
+    for (int e = lane; e < c.experts; e += 64) score[e] = logits[e];
+    const float inverse = route_choice(c, early, score, choice);
+    if (lane == 0) factor = inverse;
+  }
+  __syncthreads();
+  auto weight = [&](int e) { return choice[e] == INFINITY ? score[e] * factor : 0.f; };
+  if (!whole) {
+    for (int col = piece; col < columns; col += gridDim.y * blockDim.x) {
+      const float f = weight(col / w.ff);
+      hidden[col] = from_float<T>(f != 0.f ? f * to_float(hidden[col]) : 0.f);
+    }
+    return;
+  }
+  for (; piece < pieces; piece += gridDim.y * blockDim.x) {
+    const float f = weight(piece * PER / w.ff);
+    T* values = reinterpret_cast<T*>(&held);
+#pragma unroll
+    for (int i = 0; i < PER; ++i) values[i] = from_float<T>(f != 0.f ? f * to_float(values[i]) : 0.f);
+    *reinterpret_cast<int4v*>(hidden + (int64_t)piece * PER) = held;
+    const int next = piece + gridDim.y * blockDim.x;
+    if (next < pieces) held = *reinterpret_cast<const int4v*>(hidden + (int64_t)next * PER);
+  }
+}
+
+BT_EXPORT int bt_weigh_experts_call(void* stream, const WeighExpertsCall* w) {
+  const RouteCall* c = &w->route;
+  if (c->tokens <= 0) return BT_OK;
+  if (const char* wrong = route_refusal(c))
+    BT_REFUSE("weigh_experts: %d of %d experts a token, %d of %d groups, score %d: %s", c->top, c->experts, c->keep, c->groups, c->score, wrong);
+  if (w->ff <= 0 || w->ld_logits < c->experts || w->ld_hidden < (int64_t)c->experts * w->ff || (int64_t)c->experts * w->ff > 0x7fffffff)
+    BT_REFUSE("weigh_experts: the rows do not hold %d experts of %d", c->experts, w->ff);
+  if (!w->logits || !w->hidden) BT_REFUSE("weigh_experts: missing operand");
+  const int per = c->dtype == 0 ? 4 : 8;
+  int per_token = (c->experts * w->ff + 256 * per - 1) / (256 * per);
+  if (per_token > 64) per_token = 64;
+  dim3 grid(c->tokens, per_token), block(256);
+  if (c->dtype == 0)
+    hipLaunchKernelGGL(weigh_experts_kernel<float>, grid, block, 0, (hipStream_t)stream, *w);
+  else
+    hipLaunchKernelGGL(weigh_experts_kernel<bf16_t>, grid, block, 0, (hipStream_t)stream, *w);
+  return bt_check_launch("weigh_experts");
 }

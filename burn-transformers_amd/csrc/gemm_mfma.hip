@@ -636,7 +636,7 @@ gemm_tile_deep_kernel(const bf16_t* __restrict__ A, int64_t lda, const bf16_t* _
 // statistics are computed while the weights are on their way.
 __device__ float bt_norm_zeros[4] = {0.f, 0.f, 0.f, 0.f};
 
-template <typename T, int MT, int NT, int U, int WAVES, int QPL = 0, bool CHUNKED = false, bool TWO = false>
+template <typename T, int MT, int NT, int U, int WAVES, int QPL = 0, bool CHUNKED = false, int KIND = EPILOGUE_COMMON>
 __global__ void __launch_bounds__(WAVES * 64)
 gemm_skinny_kernel(const T* __restrict__ A, int64_t lda, const T* __restrict__ W, int M, int N,
                    int K, Epilogue epi, int tile_columns, NormOperand norm, int packed, int a_rows) {
@@ -811,7 +811,11 @@ gemm_skinny_kernel(const T* __restrict__ A, int64_t lda, const T* __restrict__ W
   const int mine = wave < blocks ? wave : 0;
   const int out_m = (mine / NT) * 16 + i16, out_n0 = n_base + (mine % NT) * 16 + g * 4;
   EpiloguePrefetch pre = {};
-  if (wave < blocks) pre = epilogue_prefetch(epi, M, n_end, out_m, out_n0, split);
+  if constexpr (KIND == EPILOGUE_TURN) {
+    if (wave < blocks) pre = epilogue_prefetch_turn(epi, M, out_m, out_n0);
+  } else {
+    if (wave < blocks) pre = epilogue_prefetch(epi, M, n_end, out_m, out_n0, split);
+  }
   multiply(c0);
   for (c0 += stride * U; c0 < chunks; c0 += stride * U) {
     issue(c0);
@@ -830,7 +834,7 @@ gemm_skinny_kernel(const T* __restrict__ A, int64_t lda, const T* __restrict__ W
     for (int w = 0; w < WAVES; ++w)
 #pragma unroll
       for (int r = 0; r < 4; ++r) v[r] += red[w][wave][lane][r];
-    if (out_m < M) epilogue4_prefetched<T, TWO>(epi, n_end, out_m, out_n0, v, split, pre);   // nothing beyond n_end
+    if (out_m < M) epilogue4_prefetched<T, KIND>(epi, n_end, out_m, out_n0, v, split, pre);   // nothing beyond n_end
   }
 }
 
@@ -840,9 +844,13 @@ static int check_operands(const char* who, int elems, const void* A, int64_t lda
   if (K % elems != 0 || lda % elems != 0)
     BT_REFUSE("%s: K %d and the row pitch %lld must be multiples of %d (16-byte loads)", who, K, (long long)lda, elems);
   if (((uintptr_t)A & 15) || ((uintptr_t)W & 15)) BT_REFUSE("%s: operands must be 16-byte aligned", who);
-  if (e.mode < 0 || e.mode > 5 || e.out == nullptr) BT_REFUSE("%s: bad epilogue", who);
+  if (e.mode < 0 || e.mode > 6 || e.out == nullptr) BT_REFUSE("%s: bad epilogue", who);
   if (e.mode == EPI_F32_ACT && (!e.out2 || e.n_q <= 0 || e.n_q >= N || e.n_q % 4 != 0))
     BT_REFUSE("%s: %d of %d columns in 32-bit, the others activated: a multiple of four, and a place for each", who, e.n_q, N);
+  if (e.mode == EPI_TURN && (e.turn_pitch <= 0 || e.turn_pitch % 4 != 0 || N % e.turn_pitch != 0 || e.turn_at < 0 || e.turn_at % 2 != 0 ||
+                             e.turn_dim <= 0 || e.turn_dim % 2 != 0 || e.turn_at + e.turn_dim > e.turn_pitch || !e.tok_pos || !e.inv_freq || e.bias))
+    BT_REFUSE("%s: heads of %d columns (a multiple of four) in %d, turned in neighbouring pairs from %d on (%d columns, both even), without a bias",
+              who, e.turn_pitch, N, e.turn_at, e.turn_dim);
   if (splits < 1 || (splits > 1 && e.mode != EPI_F32))
     BT_REFUSE("%s: K can be split %d ways only into 32-bit partial sums", who, splits);
   if (e.out_rows != 0 && ((e.mode != EPI_STORE && e.mode != EPI_ACT && e.mode != EPI_F32_ACT) || e.out_rows < M))
@@ -909,6 +917,7 @@ BT_EXPORT int bt_gemm_tile(void* stream, int dtype, const void* A, int64_t lda, 
   if (M <= 0) return BT_OK;
   if (dtype != 0 && dtype != 1) BT_REFUSE("gemm_tile: element type %d is neither float nor bfloat16", dtype);
   if (epi->mode == EPI_F32_ACT) BT_REFUSE("gemm_tile: 32-bit and activated columns of one product are the skinny kernel's");
+  if (epi->mode == EPI_TURN) BT_REFUSE("gemm_tile: turned columns are the skinny kernel's");
   int rc = check_operands("gemm_tile", dtype == 0 ? 4 : 8, A, lda, W, M, N, K, *epi, splits);
   if (rc) return rc;
   hipStream_t s = (hipStream_t)stream;
@@ -953,14 +962,17 @@ static void launch_skinny(hipStream_t s, const T* a, int64_t lda, const T* w, in
                           int splits, int columns, int packed, int a_rows) {
   dim3 grid((N + columns - 1) / columns, splits), block(512);
   const NormOperand none = {};
-  const bool two = epi.mode == EPI_F32_ACT;
+  const bool two = epi.mode == EPI_F32_ACT, turn = epi.mode == EPI_TURN;
 #define LAUNCH_SKINNY(MT, NT, U)                                                                                   \
   do {                                                                                                             \
-    if (two && a_rows > 0)                                                                                         \
-      hipLaunchKernelGGL((gemm_skinny_kernel<T, MT, NT, U, 8, 0, true, true>), grid, block, 0, s, a, lda, w, M, N, K, \
+    if (turn)                                                                                                      \
+      hipLaunchKernelGGL((gemm_skinny_kernel<T, MT, NT, U, 8, 0, false, EPILOGUE_TURN>), grid, block, 0, s, a, lda, w, M, N, K, \
+                         epi, columns, none, packed, 0);                                                           \
+    else if (two && a_rows > 0)                                                                                         \
+      hipLaunchKernelGGL((gemm_skinny_kernel<T, MT, NT, U, 8, 0, true, EPILOGUE_TWO>), grid, block, 0, s, a, lda, w, M, N, K, \
                          epi, columns, none, packed, a_rows);                                                      \
     else if (two)                                                                                                  \
-      hipLaunchKernelGGL((gemm_skinny_kernel<T, MT, NT, U, 8, 0, false, true>), grid, block, 0, s, a, lda, w, M, N, K, \
+      hipLaunchKernelGGL((gemm_skinny_kernel<T, MT, NT, U, 8, 0, false, EPILOGUE_TWO>), grid, block, 0, s, a, lda, w, M, N, K, \
                          epi, columns, none, packed, 0);                                                           \
     else if (a_rows > 0)                                                                                           \
       hipLaunchKernelGGL((gemm_skinny_kernel<T, MT, NT, U, 8, 0, true>), grid, block, 0, s, a, lda, w, M, N, K, epi, \
@@ -996,11 +1008,13 @@ static int launch_skinny_norm(hipStream_t s, const NormOperand& norm, const bf16
   size_t lds = (size_t)16 * (K * 2 + 16);
 #define LAUNCH_NORM(NT, QPL)                                                                                   \
   do {                                                                                                         \
-    if (epi.mode == EPI_F32_ACT) LAUNCH_NORM_FORM(NT, QPL, true); else LAUNCH_NORM_FORM(NT, QPL, false);       \
+    if (epi.mode == EPI_F32_ACT) LAUNCH_NORM_FORM(NT, QPL, EPILOGUE_TWO);                                      \
+    else if (epi.mode == EPI_TURN) LAUNCH_NORM_FORM(NT, QPL, EPILOGUE_TURN);                                   \
+    else LAUNCH_NORM_FORM(NT, QPL, EPILOGUE_COMMON);                                                           \
   } while (0)
-#define LAUNCH_NORM_FORM(NT, QPL, TWO)                                                                         \
+#define LAUNCH_NORM_FORM(NT, QPL, KIND)                                                                        \
   do {                                                                                                         \
-    auto kernel = gemm_skinny_kernel<bf16_t, 1, NT, 8, 8, QPL, false, TWO>;                                                \
+    auto kernel = gemm_skinny_kernel<bf16_t, 1, NT, 8, 8, QPL, false, KIND>;                                                \
     static size_t granted = 0;    /* statically allocated LDS comes on top: ask for room beyond the default */ \
     if (lds > granted) {                                                                                       \
       hipError_t err = hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); \
@@ -1042,6 +1056,7 @@ BT_EXPORT int bt_gemm_skinny(void* stream, int dtype, const void* A, int64_t lda
     A = W;            // (only its alignment is looked at below)
     lda = K;
   }
+  if (epi->mode == EPI_TURN && a_rows != 0) BT_REFUSE("gemm_skinny: turned columns go with row-major activations");
   if (a_rows != 0) lda = K;          // (chunk-major rows have no pitch; K itself is checked)
   int rc = check_operands("gemm_skinny", elems, A, lda, W, M, N, K, *epi, splits);
   if (rc) return rc;

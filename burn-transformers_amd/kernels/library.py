@@ -17,7 +17,7 @@ from . import build
 FLOAT32, BFLOAT16 = 0, 1
 DTYPE_CODES = {torch.float32: FLOAT32, torch.bfloat16: BFLOAT16}
 
-EPI_STORE, EPI_ACT, EPI_F32, EPI_QKV, EPI_RESIDUAL, EPI_F32_ACT = 0, 1, 2, 3, 4, 5
+EPI_STORE, EPI_ACT, EPI_F32, EPI_QKV, EPI_RESIDUAL, EPI_F32_ACT, EPI_TURN = 0, 1, 2, 3, 4, 5, 6
 ACTIVATIONS = {"gelu_tanh": 0, "gelu_erf": 1, "squared_relu": 2}
 NORM_KINDS = {"layer_norm": 0, "rms_norm": 1}
 KV_BLOCK = 64
@@ -41,7 +41,8 @@ class Epilogue(ctypes.Structure):
     _fields_ = [("mode", _c_int), ("act", _c_int), ("bias", _c_ptr), ("out", _c_ptr),
                 ("ldo", _c_i64), ("split_stride", _c_i64), ("n_q", _c_int), ("n_kv", _c_int),
                 ("tok_seq", _c_ptr), ("tok_pos", _c_ptr), ("kv", KvView), ("out_rows", _c_int), ("out2", _c_ptr),
-                ("ldo2", _c_i64)]
+                ("ldo2", _c_i64), ("turn_pitch", _c_int), ("turn_at", _c_int), ("turn_dim", _c_int), ("amplitude", _c_float),
+                ("inv_freq", _c_ptr)]
 
 
 class AttnArgs(ctypes.Structure):
@@ -198,6 +199,11 @@ class RouteCall(ctypes.Structure):
                 ("correction", _c_ptr), ("gate_w", _c_ptr), ("weights", _c_ptr), ("gate", _c_ptr), ("score", _c_int),
                 ("group_rank", _c_int), ("normalize", _c_int), ("bias", _c_ptr)]
     _step_fields_ = {"tokens": "tokens"}
+
+
+class WeighExpertsCall(ctypes.Structure):
+    _fields_ = [("route", RouteCall), ("ff", _c_int), ("logits", _c_ptr), ("ld_logits", _c_i64), ("hidden", _c_ptr), ("ld_hidden", _c_i64)]
+    _step_fields_ = {"route.tokens": "tokens"}
 
 
 class GatedExpertsCall(ctypes.Structure):
@@ -686,6 +692,14 @@ def epilogue_f32_act(sums, columns, out, activation):
                     out2=out.data_ptr(), ldo2=out.stride(0), out_rows=_out_rows(out))
 
 
+def epilogue_turn(out, pitch, turn_at, turn_dim, inv_freq, tok_pos, amplitude=1.0):
+    """``out`` [M, N] in the products' type; of every head of ``pitch`` columns (a multiple of four) the ``turn_dim`` from
+    ``turn_at`` on (both even) are turned in neighbouring pairs by the row's position, as ``latent_query`` does with
+    ``neighbours``: a product of up to 64 rows (the skinny kernel)."""
+    return Epilogue(mode=EPI_TURN, out=out.data_ptr(), ldo=out.stride(0), tok_pos=tok_pos.data_ptr(), turn_pitch=pitch,
+                    turn_at=turn_at, turn_dim=turn_dim, amplitude=amplitude, inv_freq=inv_freq.data_ptr())
+
+
 def epilogue_residual(x, bias=None):
     """x[m][n] += acc + bias, with x the float32 residual stream [M, N] itself."""
     return Epilogue(mode=EPI_RESIDUAL, bias=_ptr(bias), out=x.data_ptr(), ldo=x.stride(0))
@@ -796,8 +810,8 @@ class PackedWeight:
 
 
 def takes_two_kinds(a):
-    """Whether a product of the rows ``a`` can leave some columns in 32-bit and others activated (``epilogue_f32_act``):
-    the skinny kernel's steps."""
+    """Whether a product of the rows ``a`` can leave some columns in 32-bit and others activated (``epilogue_f32_act``), or
+    turn columns (``epilogue_turn``; not of chunk-major rows): the skinny kernel's steps."""
     if a.shape[0] > 64:
         return False
     return isinstance(a, Normalized) or a.dtype == torch.bfloat16 or (a.shape[1] % 4 == 0 and a.stride(0) % 4 == 0)
@@ -1363,6 +1377,19 @@ def route(h, router, correction, top, groups, keep, weights, gate_weight=None, g
                       correction=_ptr(correction), gate_w=_ptr(gate_weight), weights=weights.data_ptr(), gate=_ptr(gate),
                       score={"softmax": 0, "sigmoid": 1, "chosen": 2}[score], group_rank=group_rank, normalize=1 if normalize else 0,
                       bias=_ptr(bias)))
+
+
+def weigh_experts(logits, bias, correction, top, groups, keep, hidden, experts, ff, score="softmax", group_rank=1, normalize=True):
+    """hidden[t, e * ff + i] *= the weight of expert e for token t, the choice made as in ``route`` from the float32 router
+    ``logits`` [rows, >= experts]; columns of ``hidden`` behind the experts stay."""
+    if logits.dtype != torch.float32 or logits.stride(1) != 1 or hidden.stride(1) != 1:
+        raise KernelError(f"weigh_experts: float32 logits and plain rows, got {logits.dtype}")
+    call = RouteCall(dtype=DTYPE_CODES[hidden.dtype], tokens=hidden.shape[0], experts=experts, top=top, groups=groups, keep=keep,
+                     correction=_ptr(correction), score={"softmax": 0, "sigmoid": 1, "chosen": 2}[score], group_rank=group_rank,
+                     normalize=1 if normalize else 0, bias=_ptr(bias))
+    _launch(_module("experts"), "bt_weigh_experts_call",
+            WeighExpertsCall(route=call, ff=ff, logits=logits.data_ptr(), ld_logits=logits.stride(0), hidden=hidden.data_ptr(),
+                             ld_hidden=hidden.stride(0)))
 
 
 EXPERT_UNITS = {"gated_silu": 0, "gated_clamped": 1, "gelu_erf": 2, "silu": 3, "squared_relu": 4}

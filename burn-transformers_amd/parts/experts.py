@@ -35,6 +35,10 @@ every other; the price is that every expert multiplies every token.  In decode s
 little once tokens * top reaches the number of experts (all matrices are read anyway); a prompt does
 experts / top times the routed arithmetic, which a grouped product over tokens sorted by expert
 would save.
+
+In small steps the router's logits come from the same product (``rides``: units without a gate whose activation the product
+has, a router that the products' type holds exactly, nothing else beside the experts): its rows lie before the up matrices,
+the product leaves 32-bit logits and activated units, and one kernel makes the choice and weighs the units.
 """
 
 import torch
@@ -116,7 +120,15 @@ class RoutedExperts(FeedForward):
         self.in_weight = pad_columns(pad_rows(torch.cat(rows), self.fused_cols), operand_columns(self.width, dtype))
         self.down_weight = pad_columns(torch.cat(columns, dim=1), self.hidden_cols)           # [width, inner (+ zeros)]
         on_gpu = self.in_weight.is_cuda
-        self.in_packed = K.PackedWeight(self.in_weight) if on_gpu else None
+        self.rides = self.unit in K.ACTIVATIONS and not self.identity and self.shared_mix is None and \
+            torch.equal(self.router.to(dtype).float(), self.router)
+        if self.rides:
+            self.logit_cols = (self.outputs + 3) // 4 * 4             # (the product's epilogue works on four columns at a time)
+            router = pad_columns(pad_rows(self.router.to(dtype), self.logit_cols), self.in_weight.shape[1])
+            self.first_weight = torch.cat([router, self.in_weight]).contiguous()
+            self.in_weight = self.first_weight[self.logit_cols:]
+            self.first_packed = K.PackedWeight(self.first_weight) if on_gpu else None
+        self.in_packed = K.PackedWeight(self.in_weight) if on_gpu and not self.rides else None
         self.down_packed = packed_for_stream(self.down_weight) if on_gpu else None
 
     def kernel_modules(self, dtype):
@@ -124,6 +136,16 @@ class RoutedExperts(FeedForward):
 
     def forward(self, h, step, stream):
         tokens = h.shape[0]
+        if self.rides and K.takes_two_kinds(h):
+            logits = step.buffer("experts.logits", tokens, self.logit_cols, "float32")
+            hidden = step.buffer("experts.hidden", tokens, self.hidden_cols, step.dtype)
+            K.gemm(h, self.first_weight, K.epilogue_f32_act(logits, self.logit_cols, hidden, self.unit), packed=self.first_packed)
+            K.weigh_experts(logits, self.router_bias, self.correction, self.top, self.groups, self.keep, hidden, self.experts, self.ff,
+                            score=self.score, group_rank=self.group_rank, normalize=self.normalize)
+            splits = stream_product_splits(step, hidden, self.down_weight)
+            partials = step.partial_sums("experts.partials", splits, tokens, self.width)
+            K.gemm(hidden, self.down_weight, K.epilogue_f32(partials), splits=splits, packed=self.down_packed)
+            return Delta(partials, None)
         weights = step.buffer("experts.weights", tokens, self.outputs, "float32")
         mix = step.buffer("experts.mix", tokens, 1, "float32") if self.shared_mix is not None else None
         K.route(h, self.router, self.correction, self.top, self.groups, self.keep, weights, self.shared_mix, mix,

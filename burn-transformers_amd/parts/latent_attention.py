@@ -25,9 +25,14 @@ keys and values are the same vector, and the heads' queries against it are the g
 of the attention kernels (all heads of a token read each cached vector once).  The matrix
 up_k_i^T up_q_i is formed once when the part is built (in float64, rounded to the products' type).
 
+The same on the way out: out_weight_i up_v_i is formed once as well (``absorbs_values``: no gate, or one per head, and
+a matrix that is not much larger for it), so that the output projection reads the attention's own result, gated head by
+head where there is a gate.  A gate per channel stands between the two products and keeps them apart.
+
 One step: a fused product [down_q; down_kv; gate] h (32-bit sums) -> the two norms, c straight into
-the paged cache (a borrowing mixer: [down_q; gate] h and the one norm) -> absorbed queries (one product) -> attention over the cache -> per head up_v and
-sigmoid gate -> output projection (the sublayer's output).
+the paged cache (a borrowing mixer: [down_q; gate] h and the one norm) -> absorbed queries (one product; in small steps
+their turned parts are rotated in its epilogue, and a borrowing mixer's norm is folded into it) -> attention over the
+cache -> per head up_v and sigmoid gate, where they are not absorbed -> output projection (the sublayer's output).
 """
 
 import torch
@@ -83,10 +88,10 @@ class LatentAttention(Mixer):
         self.q_cols = operand_columns(self.q_rank, dtype)
         self.kv_offset = (self.q_rank + 3) // 4 * 4
         self.gate_offset = self.kv_offset + (0 if self.borrows else (self.kv_rank + self.rot_dim + 3) // 4 * 4)
-        self.fused_cols = self.gate_offset + gate_rows
+        self.fused_cols = (self.gate_offset + gate_rows + 3) // 4 * 4
         self.fused_weight = torch.cat([pad_rows(tensors["down_q"], self.kv_offset)] +
                                       ([pad_rows(tensors["down_kv"], self.gate_offset - self.kv_offset)] if not self.borrows else []) +
-                                      ([tensors["gate"]] if self.gated else []))
+                                      ([pad_rows(tensors["gate"], self.fused_cols - self.gate_offset)] if self.gated else []))
         # (the rows it multiplies carry zero columns where the width is no multiple of what 16-byte loads take)
         self.fused_weight = pad_columns(self.fused_weight, operand_columns(self.width, dtype))
         self.q_norm, self.kv_norm = tensors["q_norm"], None if self.borrows else tensors["kv_norm"]
@@ -104,10 +109,21 @@ class LatentAttention(Mixer):
             self.inv_freq = rotary_frequencies(self.rot_dim, p["rot_base"], p.get("rot_scaling")).to(torch.float32).to(device)
             self.amplitude = rotary_amplitude(p.get("rot_scaling"))
         self.query_weight = full.view(self.heads * self.head_dim, self.q_cols).to(dtype).contiguous()
-        self.up_v = tensors["up_v"].contiguous()
-        self.mixed_cols = operand_columns(self.heads * self.vdim, dtype)
-        self.out_weight = pad_columns(tensors["out_weight"], self.mixed_cols)
         self.n_q = self.heads * self.head_dim
+        extra = self.heads * (self.head_dim - self.vdim) * self.width * tensors["out_weight"].element_size()
+        self.absorbs_values = extra <= self.ABSORBED_BYTES and not (self.gated and self.gate_span == "channel")
+        if self.absorbs_values:
+            out = tensors["out_weight"].double().view(self.width, self.heads, self.vdim)
+            up_v = tensors["up_v"].double().view(self.heads, self.vdim, self.kv_rank)
+            full = out.new_zeros(self.width, self.heads, self.head_dim)
+            full[:, :, :self.kv_rank] = torch.einsum("whv,hvr->whr", out, up_v)
+            self.out_weight = full.view(self.width, self.n_q).to(dtype).contiguous()
+        else:
+            self.up_v = tensors["up_v"].contiguous()
+            self.mixed_cols = operand_columns(self.heads * self.vdim, dtype)
+            self.out_weight = pad_columns(tensors["out_weight"], self.mixed_cols)
+        # what the query product's epilogue in small steps takes: neighbouring pairs within four columns
+        self.turns_in_product = self.rot_dim > 0 and self.neighbours and self.kv_rank % 2 == 0
         # second copies for decode steps, which read the weights and little else
         on_gpu = self.fused_weight.is_cuda
         self.fused_packed = K.PackedWeight(self.fused_weight) if on_gpu else None
@@ -119,11 +135,12 @@ class LatentAttention(Mixer):
 
     def kernel_modules(self, dtype):
         names = ["latent"]
+        variant = "_softmax" if self.gated and self.absorbs_values else ""        # (the form with an output stage)
         if not self.plain_only:
             if dtype == torch.bfloat16:
-                names.append(f"attention_bf16_hd{self.head_dim}")
+                names.append(f"attention_bf16_hd{self.head_dim}{variant}")
             elif self.head_dim <= 128:
-                names.append("attention_f32")
+                names.append("attention_f32" + variant)
         return tuple(names)
 
     # the planning of a prompt's runs of keys is the ordinary attention's: one cached head, ``heads`` query heads
@@ -147,28 +164,51 @@ class LatentAttention(Mixer):
 
     SPLIT_BYTES = 128 << 10
     RUN_BYTES = 64 << 10
+    # How much larger than out_weight the matrix with up_v absorbed may be: a decode step reads so much in less time than
+    # the kernel takes that it saves (4 us), and a prompt of 2,048 tokens multiplies by it in less (23 us at 8 heads)
+    ABSORBED_BYTES = 8 << 20
 
     def forward(self, h, step, memory, stream):
         tokens = h.shape[0]
         kv = memory.kv()
         fused = step.buffer("latent.fused", tokens, self.fused_cols, "float32")
         K.gemm(h, self.fused_weight, K.epilogue_f32(fused), packed=self.fused_packed)
-        c_q = step.buffer("latent.query_latent", tokens, self.q_cols, step.dtype)
         if memory.writes == self.borrows:
             raise ValueError("latent attention: a mixer keeps a cache entry of its own, or borrows and reads another layer's")
-        K.latent_norm(fused, self.q_rank, self.kv_offset, 0 if self.borrows else self.kv_rank, self.q_norm, self.kv_norm, self.eps, c_q,
-                      step.tok_seq, step.tok_pos, kv, step.dtype, rot_dim=0 if self.borrows else self.rot_dim, inv_freq=self.inv_freq,
-                      neighbours=self.neighbours, amplitude=self.amplitude)
         q = step.buffer("latent.queries", tokens, self.n_q, step.dtype)
-        if self.rot_dim:         # the turned part of every head is rotated from the 32-bit sums
+        self.make_queries(fused, q, kv, step)
+        self.attend(fused, q, kv, step, stream)
+
+    def make_queries(self, fused, q, kv, step):
+        """The absorbed and turned queries into ``q``, and the latent of a mixer that keeps one into the cache."""
+        tokens = q.shape[0]
+        small = tokens <= 64 and (not self.rot_dim or self.turns_in_product)
+        if self.borrows and small and step.dtype_is_bf16 and self.q_cols == self.q_rank and K.Normalized.worth_it(tokens, self.q_rank):
+            c_q = K.Normalized(fused[:, :self.q_rank], self.q_norm, None, self.eps, "rms_norm")
+        else:
+            c_q = step.buffer("latent.query_latent", tokens, self.q_cols, step.dtype)
+            K.latent_norm(fused, self.q_rank, self.kv_offset, 0 if self.borrows else self.kv_rank, self.q_norm, self.kv_norm, self.eps,
+                          c_q, step.tok_seq, step.tok_pos, kv, step.dtype, rot_dim=0 if self.borrows else self.rot_dim,
+                          inv_freq=self.inv_freq, neighbours=self.neighbours, amplitude=self.amplitude)
+        if not self.rot_dim:
+            K.gemm(c_q, self.query_weight, K.epilogue_store(q), packed=self.query_packed)
+        elif self.turns_in_product and K.takes_two_kinds(c_q):
+            K.gemm(c_q, self.query_weight, K.epilogue_turn(q, self.head_dim, self.kv_rank, self.rot_dim, self.inv_freq, step.tok_pos,
+                                                           self.amplitude), packed=self.query_packed)
+        else:                    # the turned part of every head is rotated from the 32-bit sums
             sums = step.buffer("latent.query_sums", tokens, self.n_q, "float32")
             K.gemm(c_q, self.query_weight, K.epilogue_f32(sums), packed=self.query_packed)
             K.latent_query(sums, self.heads, self.head_dim, self.kv_rank, self.rot_dim, self.inv_freq, step.tok_pos, q,
                            neighbours=self.neighbours, amplitude=self.amplitude)
+
+    def attend(self, fused, q, kv, step, stream):
+        tokens = q.shape[0]
+        gate = fused[:, self.gate_offset:] if self.gated else None
+        if self.absorbs_values and step.decode and step.dtype_is_bf16 and not self.plain_only and K.Chunked.wanted(tokens):
+            ctx = K.Chunked.take(step, "latent.context", tokens, self.n_q, step.dtype)       # read by the next product only
         else:
-            K.gemm(c_q, self.query_weight, K.epilogue_store(q), packed=self.query_packed)
-        ctx = step.buffer("latent.context", tokens, self.n_q, step.dtype)
-        partial, runs, prompt_runs = None, self.decode_runs(step, h.device), self.prompt_runs(step, h.device)
+            ctx = step.buffer("latent.context", tokens, self.n_q, step.dtype)
+        partial, runs, prompt_runs = None, self.decode_runs(step, q.device), self.prompt_runs(step, q.device)
         if self.plain_only:
             runs = prompt_runs = 1
         if runs > 1:
@@ -177,9 +217,11 @@ class LatentAttention(Mixer):
             partial = step.buffer("attention.partial", tokens * self.heads * prompt_runs, self.head_dim + 2, "float32")
         args = K.attention_args(q, ctx, kv, step.tok_seq, step.tok_pos, step.seq_off, step.seq_start, self.heads,
                                 step.n_seqs, step.max_count, self.scale, self.window, partial,
-                                runs=prompt_runs if prompt_runs > 1 else None, keep=self.keep)
+                                runs=prompt_runs if prompt_runs > 1 else None, keep=self.keep, gate=gate if self.absorbs_values else None)
         K.attention(args, step.dtype, step.decode, impl="plain" if self.plain_only else "auto")
+        if self.absorbs_values:
+            stream.add_product(step, ctx, self.out_weight, packed=self.out_packed)
+            return
         mixed = step.buffer("latent.mixed", tokens, self.mixed_cols, step.dtype)
-        K.head_project(ctx, self.up_v, self.heads, self.vdim, self.kv_rank, self.head_dim, mixed,
-                       gate=fused[:, self.gate_offset:] if self.gated else None, gate_span=self.gate_span)
+        K.head_project(ctx, self.up_v, self.heads, self.vdim, self.kv_rank, self.head_dim, mixed, gate=gate, gate_span=self.gate_span)
         stream.add_product(step, mixed, self.out_weight, packed=self.out_packed)

@@ -219,3 +219,100 @@ def test_squared_relu_as_an_experts_unit(dtype, experts, ff, shared):
     want[:, :experts * ff] *= weights.double().repeat_interleave(ff, dim=1)
     assert rel_err(hidden[:, :inner], want) < (1e-6 if dtype == "float32" else 1e-2)
     assert float(hidden[:, inner:].float().abs().max()) == 0.0
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("m", [1, 8, 16, 17, 33, 64])
+@pytest.mark.parametrize("heads,pitch,at,dims,k", [(3, 48, 32, 16, 40), (5, 16, 10, 6, 96), (2, 128, 0, 128, 24), (1, 4, 2, 2, 8), (16, 128, 96, 32, 384)])
+def test_a_product_that_turns_columns_by_the_rows_positions(dtype, m, heads, pitch, at, dims, k):
+    """Plain and packed weights; turned ranges that begin inside four columns; positions up to some thousands."""
+    gen = torch.Generator().manual_seed(m + pitch)
+    n, amplitude = heads * pitch, 1.25
+    a, w = torch.randn(m, k, generator=gen).to(DTYPES[dtype]), (torch.randn(n, k, generator=gen) / math.sqrt(k)).to(DTYPES[dtype])
+    positions = torch.randint(0, 3000, (m,), generator=gen)
+    positions[0] = 0
+    rot = {"dims": dims, "base": 700.0}
+    want = (a.double() @ w.double().T).view(m, heads, pitch)
+    want[..., at:at + dims] = amplitude * plain.turn(want[..., at:at + dims], positions, rot)
+    freq = torch.tensor([700.0 ** (-2.0 * i / dims) for i in range(dims // 2)]).to(DEV)
+    bound = 1e-3 if dtype == "float32" else 1e-2        # (angles are 32-bit products: at position 3,000 they are off by 2e-4)
+    out = torch.full((m, n + 4), float("nan"), dtype=DTYPES[dtype], device=DEV)[:, :n]
+    on_gpu = positions.to(torch.int32).to(DEV)          # (an epilogue holds addresses: what they name stays here)
+    epilogue = K.epilogue_turn(out, pitch, at, dims, freq, on_gpu, amplitude)
+    K.gemm(a.to(DEV), w.to(DEV), epilogue)
+    assert rel_err(out, want.reshape(m, n)) < bound
+    first = out.clone()
+    K.gemm(a.to(DEV), w.to(DEV), epilogue, packed=(K.pack_columns(w.to(DEV), 16), 16))
+    assert torch.equal(first, out)
+
+
+@pytest.mark.parametrize("m", [1, 7, 16])
+def test_a_turning_product_that_normalises_its_rows_itself(m):
+    gen = torch.Generator().manual_seed(m)
+    k, heads, pitch, at, dims, eps = 72, 4, 32, 20, 12, 1e-4
+    fused, gamma = torch.randn(m, k + 8, generator=gen), torch.randn(k, generator=gen)
+    w = (torch.randn(heads * pitch, k, generator=gen) / 8).to(torch.bfloat16)
+    positions = torch.arange(m) * 5 + 3
+    c = (plain.unit_rms(fused[:, :k].double(), eps) * gamma.double()).to(torch.bfloat16).double()
+    want = (c @ w.double().T).view(m, heads, pitch)
+    want[..., at:at + dims] = plain.turn(want[..., at:at + dims], positions, {"dims": dims, "base": 50.0})
+    freq = torch.tensor([50.0 ** (-2.0 * i / dims) for i in range(dims // 2)]).to(DEV)
+    out = torch.zeros(m, heads * pitch, dtype=torch.bfloat16, device=DEV)
+    held = fused.to(DEV), gamma.to(DEV), positions.to(torch.int32).to(DEV)
+    K.gemm(K.Normalized(held[0][:, :k], held[1], None, eps, "rms_norm"), w.to(DEV), K.epilogue_turn(out, pitch, at, dims, freq, held[2]))
+    assert rel_err(out, want.reshape(m, -1)) < 1.5e-2
+
+
+def test_what_a_turning_product_refuses():
+    a, w, out = torch.zeros(4, 16, device=DEV), torch.zeros(32, 16, device=DEV), torch.zeros(4, 32, device=DEV)
+    freq, pos = torch.ones(8, device=DEV), torch.zeros(4, dtype=torch.int32, device=DEV)
+    for pitch, at, dims in ((16, 1, 4), (16, 0, 3), (16, 14, 4), (6, 0, 2), (20, 0, 4)):
+        with pytest.raises(K.KernelError):
+            K.gemm(a, w, K.epilogue_turn(out, pitch, at, dims, freq, pos))
+    with pytest.raises(K.KernelError):
+        K.gemm(a, w, K.epilogue_turn(out, 16, 0, 4, freq, pos), impl="tile")
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("experts,ff,shared,top,tokens", [(8, 1024, 64, 2, 8), (5, 7, 0, 3, 64), (3, 16, 9, 1, 1), (130, 8, 8, 6, 20), (1, 1, 1, 1, 2)])
+@pytest.mark.parametrize("score", ["chosen", "softmax", "sigmoid"])
+def test_units_weighed_by_logits_that_came_with_them(dtype, experts, ff, shared, top, tokens, score):
+    """The same weights as the router kernel's, on the units in place; columns behind the experts stay; an unchosen
+    expert's units are zero whatever they were."""
+    gen = torch.Generator().manual_seed(experts + tokens)
+    logits = torch.randn(tokens, experts + 3, generator=gen) * 3.0
+    bias = torch.randn(experts, generator=gen)
+    z = (logits[:, :experts] + bias).double()
+    weights = torch.zeros(tokens, experts, dtype=F64)
+    s = {"chosen": torch.exp(z - z.max(1, keepdim=True).values), "softmax": torch.softmax(z, 1), "sigmoid": plain.sigmoid(z)}[score]
+    for t in range(tokens):
+        chosen = z[t].argsort(descending=True)[:top]
+        weights[t, chosen] = s[t, chosen] / s[t, chosen].sum()
+    hidden = torch.randn(tokens, experts * ff + shared + 5, generator=gen).to(DTYPES[dtype])
+    want = hidden.double()
+    want[:, :experts * ff] *= weights.repeat_interleave(ff, dim=1)
+    if top < experts:
+        hidden[0, int(z[0].argmin()) * ff] = float("inf")
+    rows = hidden.to(DEV)
+    K.weigh_experts(logits.to(DEV), bias.to(DEV), None, top, 1, 1, rows, experts, ff, score=score)
+    assert rel_err(rows, want) < (1e-5 if dtype == "float32" else 1e-2)
+    assert torch.equal(rows[:, experts * ff:].cpu(), hidden[:, experts * ff:])
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("unit", ["squared_relu", "gelu_erf", "silu"])
+def test_units_taken_sixteen_bytes_at_a_time(dtype, unit):
+    gen = torch.Generator().manual_seed(2)
+    tokens, experts, ff, shared = 70, 3, 1032, 24
+    inner = experts * ff + shared
+    up = torch.randn(tokens, inner + 8, generator=gen).to(DTYPES[dtype])
+    weights = torch.rand(tokens, experts, generator=gen)
+    weights[weights < 0.4] = 0.0
+    hidden = torch.full((tokens, inner + 8), float("nan"), dtype=DTYPES[dtype], device=DEV)
+    K.gated_experts(up.to(DEV), weights.to(DEV), None, experts, ff, shared, 0, hidden, unit=unit)
+    act = {"squared_relu": plain.squared_relu, "silu": lambda z: z * plain.sigmoid(z),
+           "gelu_erf": lambda z: 0.5 * z * (1.0 + torch.erf(z / math.sqrt(2.0)))}[unit]
+    want = act(up.double()[:, :inner])
+    want[:, :experts * ff] *= weights.double().repeat_interleave(ff, dim=1)
+    assert rel_err(hidden[:, :inner], want) < (1e-6 if dtype == "float32" else 1e-2)
+    assert float(hidden[:, inner:].float().abs().max()) == 0.0
