@@ -55,6 +55,8 @@ struct AttnArgs {
   int out_f32;
   // The first `keep` positions of a sequence are seen by every later query of it, whatever window and chunk say.
   int keep;
+  // attention_shared.hip only: the value channels from here on are zero (0: none is).
+  int value_dim;
 };
 
 // What a sink adds to a softmax's denominator that is kept relative to the maximum `top`.  The plain and

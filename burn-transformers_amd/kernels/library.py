@@ -52,7 +52,7 @@ class AttnArgs(ctypes.Structure):
                 ("max_count", _c_int), ("window", _c_int), ("scale", _c_float), ("splits", _c_int),
                 ("partial", _c_ptr), ("out_rows", _c_int), ("chunk", _c_int), ("sink", _c_ptr), ("form", _c_int),
                 ("cap", _c_float), ("score_bias", _c_ptr), ("gate", _c_ptr), ("ld_gate", _c_i64), ("gate_span", _c_int),
-                ("gate_dim", _c_int), ("out_f32", _c_int), ("keep", _c_int)]
+                ("gate_dim", _c_int), ("out_f32", _c_int), ("keep", _c_int), ("value_dim", _c_int)]
 
 
 class NormOperand(ctypes.Structure):
@@ -967,7 +967,7 @@ def _library_has_algorithm(lda, m, n, k, epilogue):
 
 def attention_args(q, out, kv_view, tok_seq, tok_pos, seq_off, seq_start, q_heads, n_seqs, max_count,
                    scale, window=0, partial=None, runs=None, chunk=0, sink=None, softcap=0.0, sigmoid=False, score_bias=None,
-                   gate=None, gate_dim=0, keep=0):
+                   gate=None, gate_dim=0, keep=0, value_dim=0):
     """``partial``: float32 [rows * q_heads * runs, head_dim + 2] for a step whose keys are cut into
     runs that separate work-groups take.  Decode steps (long contexts in small batches): rows are
     the sequences, and ``runs`` follows from the shape.  Prompt steps (few query tiles behind a long
@@ -981,7 +981,8 @@ def attention_args(q, out, kv_view, tok_seq, tok_pos, seq_off, seq_start, q_head
     softmax.  ``sigmoid``: no softmax; a visible key weighs sigmoid(score + ``score_bias``[head]) (float32 [q_heads]).
     ``gate``: float32 logits whose sigmoid multiplies the output, [tokens, >= q_heads] a logit per head, or with
     ``gate_dim`` [tokens, >= q_heads * gate_dim] one per channel.  A float32 ``out`` of bfloat16 queries keeps the
-    output's digits."""
+    output's digits.  ``value_dim``: channels of the values that are not zero, rounded up to four (0: all), which the
+    "shared" kernel need not read behind."""
     keep = min(keep or 0, 1 << 30)
     if score_bias is not None and (score_bias.dtype != torch.float32 or score_bias.numel() != q_heads or not score_bias.is_contiguous()):
         raise KernelError(f"attention: the scores' bias is one float32 number per query head, got {tuple(score_bias.shape)} {score_bias.dtype}")
@@ -1005,7 +1006,7 @@ def attention_args(q, out, kv_view, tok_seq, tok_pos, seq_off, seq_start, q_head
                     form=2 if sigmoid else 1 if softcap else 0, cap=softcap or 0.0, score_bias=_ptr(score_bias),
                     gate=_ptr(gate), ld_gate=gate.stride(0) if gate is not None else 0, gate_span=1 if gate_dim else 0,
                     gate_dim=gate_dim, out_f32=1 if out.dtype == torch.float32 and q.dtype != torch.float32 else 0,
-                    keep=keep)
+                    keep=keep, value_dim=value_dim)
 
 
 def attention_variant(args):
@@ -1016,7 +1017,8 @@ def attention_variant(args):
 def attention(args, dtype, decode, impl="auto"):
     """Attention of the step's tokens over the cache.  impl: "auto" (bfloat16: the MFMA kernels;
     float32: the tiled kernel for head sizes up to 128, else the plain one), "plain", "tiled"
-    (float32) or "mfma" (bfloat16)."""
+    (float32), "mfma" (bfloat16) or "shared" (bfloat16: one cached head of up to 768 for all query heads, prompts and decode
+    steps)."""
     code = DTYPE_CODES[dtype]
     if impl == "auto":
         if code == BFLOAT16:
@@ -1035,6 +1037,9 @@ def attention(args, dtype, decode, impl="auto"):
         return
     if code != BFLOAT16:
         raise KernelError("attention: the MFMA kernels take bfloat16 only")
+    if impl == "shared":
+        _launch(_module("attention_shared"), "bt_attention_shared_call", call)
+        return
     _launch(_module(f"attention_bf16_hd{args.kv.head_dim}{attention_variant(args)}"),
             "bt_attention_decode_bf16_call" if decode else "bt_attention_prefill_bf16_call", call)
 

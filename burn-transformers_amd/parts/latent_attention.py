@@ -81,9 +81,10 @@ class LatentAttention(Mixer):
         if self.head_dim > 768:
             raise ValueError(f"latent attention: a cached head of {self.kv_rank} + {self.rot_dim} is beyond 768, the most any "
                              f"attention kernel here takes")
-        # the MFMA kernels take heads of up to 128 (bfloat16) and up to 16 query heads per cached head
-        # in decode steps; everything else runs on the plain attention kernel
-        self.plain_only = self.bf16 and (self.head_dim > 128 or self.heads > 16)
+        # bfloat16: the ordinary kernels take heads of up to 128 and up to 16 query heads per cached head in decode steps, the
+        # kernel for one shared head the others.  (float32: the tiled kernel up to 128, the plain one beyond)
+        self.shared_only = self.bf16 and self.head_dim > 128
+        self.shared_decode = self.bf16 and (self.shared_only or self.heads > 16)
         # segments of the fused first product, each padded so that the next starts where 16-byte loads may
         self.q_cols = operand_columns(self.q_rank, dtype)
         self.kv_offset = (self.q_rank + 3) // 4 * 4
@@ -136,17 +137,29 @@ class LatentAttention(Mixer):
     def kernel_modules(self, dtype):
         names = ["latent"]
         variant = "_softmax" if self.gated and self.absorbs_values else ""        # (the form with an output stage)
-        if not self.plain_only:
-            if dtype == torch.bfloat16:
+        if dtype == torch.bfloat16:
+            if self.shared_decode:
+                names.append("attention_shared")
+            if not self.shared_only:
                 names.append(f"attention_bf16_hd{self.head_dim}{variant}")
-            elif self.head_dim <= 128:
-                names.append("attention_f32" + variant)
+        elif self.head_dim <= 128:
+            names.append("attention_f32" + variant)
         return tuple(names)
 
     # the planning of a prompt's runs of keys is the ordinary attention's: one cached head, ``heads`` query heads
     kv_heads = 1
     chunk = 0
-    prompt_runs = CausalSelfAttention.prompt_runs
+    plain_only = False
+
+    def prompt_runs(self, step, device):
+        if not self.shared_only:
+            return CausalSelfAttention.prompt_runs(self, step, device)
+        if step.decode:
+            return 1
+        # tiles of 32 (token, head) rows, a work-group each; a run keeps at least four blocks of keys
+        tiles = -(-step.token_capacity * self.heads // 32) + step.n_seqs - 1
+        keys = keys_in_reach(step.context_limit, self.window, 0, self.keep)
+        return max(1, min(compute_units(device) // tiles, keys // 256, 16))
 
     def decode_runs(self, step, device):
         """Into how many runs a decode step's keys are cut.  All heads share one cached head, so a
@@ -160,7 +173,11 @@ class LatentAttention(Mixer):
         pair_bytes = keys * self.head_dim * 2 * (2 if step.dtype_is_bf16 else 4)
         if pair_bytes <= self.SPLIT_BYTES:
             return 1
-        return max(1, min(compute_units(device) // step.n_seqs, pair_bytes // self.RUN_BYTES, 64))
+        tiles = 1
+        if self.shared_decode:           # (rows of 32 heads a work-group, 16 where there are no more or heads are widest)
+            tiles = -(-self.heads // (16 if self.heads <= 16 or self.head_dim > 576 else 32))
+        runs = min(compute_units(device) // (step.n_seqs * tiles), pair_bytes // self.RUN_BYTES, 64)
+        return max(1, min(runs, -(-keys // 64) if self.shared_decode else runs))
 
     SPLIT_BYTES = 128 << 10
     RUN_BYTES = 64 << 10
@@ -204,21 +221,21 @@ class LatentAttention(Mixer):
     def attend(self, fused, q, kv, step, stream):
         tokens = q.shape[0]
         gate = fused[:, self.gate_offset:] if self.gated else None
-        if self.absorbs_values and step.decode and step.dtype_is_bf16 and not self.plain_only and K.Chunked.wanted(tokens):
+        if self.absorbs_values and step.decode and step.dtype_is_bf16 and K.Chunked.wanted(tokens):
             ctx = K.Chunked.take(step, "latent.context", tokens, self.n_q, step.dtype)       # read by the next product only
         else:
             ctx = step.buffer("latent.context", tokens, self.n_q, step.dtype)
         partial, runs, prompt_runs = None, self.decode_runs(step, q.device), self.prompt_runs(step, q.device)
-        if self.plain_only:
-            runs = prompt_runs = 1
         if runs > 1:
             partial = step.buffer("attention.partial", step.n_seqs * self.heads * runs, self.head_dim + 2, "float32")
         elif prompt_runs > 1:
             partial = step.buffer("attention.partial", tokens * self.heads * prompt_runs, self.head_dim + 2, "float32")
         args = K.attention_args(q, ctx, kv, step.tok_seq, step.tok_pos, step.seq_off, step.seq_start, self.heads,
                                 step.n_seqs, step.max_count, self.scale, self.window, partial,
-                                runs=prompt_runs if prompt_runs > 1 else None, keep=self.keep, gate=gate if self.absorbs_values else None)
-        K.attention(args, step.dtype, step.decode, impl="plain" if self.plain_only else "auto")
+                                runs=prompt_runs if prompt_runs > 1 else None, keep=self.keep, gate=gate if self.absorbs_values else None,
+                                value_dim=(self.kv_rank + 3) // 4 * 4)
+        shared = self.shared_only or (self.shared_decode and step.decode)
+        K.attention(args, step.dtype, step.decode, impl="shared" if shared else "auto")
         if self.absorbs_values:
             stream.add_product(step, ctx, self.out_weight, packed=self.out_packed)
             return

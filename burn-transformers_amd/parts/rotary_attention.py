@@ -154,6 +154,10 @@ class RotaryAttention(CausalSelfAttention):
         self.plain_only = bf16 and self.head_dim > 128
         self.q_heads = self.heads * self.maps                   # queries the attention kernels see
         self.plain_decode = bf16 and self.q_heads // self.kv_heads > 16
+        # ... but where all query heads share one cached head and the scores are an ordinary softmax's, both run on the
+        # kernel for that
+        self.shared_head = (self.plain_only or self.plain_decode) and self.kv_heads == 1 and not self.softcap and not self.sigmoid \
+            and not self.wide_output(dtype)
         self.n_q, self.n_kv = self.q_heads * self.head_dim, self.kv_heads * self.head_dim
         self.fused_cols = n_qk[0] + n_qk[1] + n_v               # what a convolution passes over
         self.first_cols = self.fused_cols + self.gate_cols
@@ -195,6 +199,8 @@ class RotaryAttention(CausalSelfAttention):
         if self.softcap or self.sigmoid or self.gate_cols or self.wide_output(dtype):
             variant = "_sigmoid" if self.sigmoid else "_capped" if self.softcap else "_softmax"
             modules = tuple(name + variant for name in modules)
+        if dtype == torch.bfloat16 and self.shared_head:
+            modules += ("attention_shared",)
         return ("rotary",) + (("state_space",) if self.taps else ()) + modules
 
     def carry(self, weight, activation):
@@ -216,7 +222,7 @@ class RotaryAttention(CausalSelfAttention):
 
     def runs_plain(self, step):
         """(the bfloat16 decode kernel takes up to 16 query heads on a cached head; beyond, the plain kernel)"""
-        return self.plain_only or (self.plain_decode and step.decode)
+        return (self.plain_only or (self.plain_decode and step.decode)) and not self.shared_head
 
     def state_spec(self):
         return StateSpec((self.conv_state,), "float32") if self.conv_state else None
@@ -266,4 +272,5 @@ class RotaryAttention(CausalSelfAttention):
                                 self.q_heads, step.n_seqs, step.max_count, self.scale, self.window, partial,
                                 runs=prompt_runs if prompt_runs > 1 else None, chunk=self.chunk, keep=self.keep, sink=self.sink, softcap=self.softcap, sigmoid=self.sigmoid,
                                 score_bias=self.score_bias, gate=gate, gate_dim=self.vdim if self.gate_kind == "channel" else 0)
-        K.attention(args, step.dtype, step.decode, impl="plain" if plain else "auto")
+        shared = self.shared_head and step.dtype_is_bf16 and (self.plain_only or step.decode)
+        K.attention(args, step.dtype, step.decode, impl="plain" if plain else "shared" if shared else "auto")

@@ -316,3 +316,89 @@ def test_units_taken_sixteen_bytes_at_a_time(dtype, unit):
     want[:, :experts * ff] *= weights.double().repeat_interleave(ff, dim=1)
     assert rel_err(hidden[:, :inner], want) < (1e-6 if dtype == "float32" else 1e-2)
     assert float(hidden[:, inner:].float().abs().max()) == 0.0
+
+
+SHARED = [(1, 144), (3, 64), (16, 128), (16, 576), (20, 96), (33, 320), (5, 512), (128, 192), (2, 640), (17, 768)]
+
+
+@pytest.mark.parametrize("heads,hd", SHARED)
+@pytest.mark.parametrize("window,keep", [(0, 0), (70, 0), (100, 66), (1, 1)])
+def test_attention_on_one_shared_head(heads, hd, window, keep):
+    """Prompts behind contexts, portions of a few tokens and decode steps, whole and in runs (more of them than some
+    sequences have blocks), with and without a last part of the value that is not read, on a cache of NaN wherever no token
+    lies."""
+    gen = torch.Generator().manual_seed(hd + heads)
+    for totals, counts in (([200, 9, 131], [40, 9, 3]), ([330, 70, 1, 129], [1, 1, 1, 1])):
+        case = PagedCase(totals, counts, 1, hd, torch.bfloat16, DEV, seed=hd, poison=True)
+        q = (torch.randn(case.n_tokens, heads * hd, generator=gen) * 2.0 / math.sqrt(hd)).to(torch.bfloat16)
+        whole = reference(case, q, heads, 1.0, window, 0, keep).view(case.n_tokens, heads, hd)
+        for value_dim, runs in ((0, 1), (hd - hd // 5 // 4 * 4, 1), (hd - 16, 3), (0, 8)):
+            out = torch.full((case.n_tokens, heads * hd), float("nan"), dtype=torch.bfloat16, device=DEV)
+            partial = torch.full((case.n_tokens * heads * runs, hd + 2), float("nan"), device=DEV) if runs > 1 else None
+            args = K.attention_args(q.to(DEV), out, case.view(), case.tok_seq, case.tok_pos, case.seq_off, case.seq_start, heads,
+                                    len(totals), max(counts), 1.0, window, partial, runs=runs if runs > 1 else None, keep=keep, value_dim=value_dim)
+            K.attention(args, torch.bfloat16, max(counts) == 1, impl="shared")
+            want = whole.clone()
+            if value_dim:
+                want[..., value_dim:] = 0.0
+            assert rel_err(out, want.reshape(case.n_tokens, -1)) < 1.5e-2, (totals, value_dim, runs)
+            assert not value_dim or float(out.view(case.n_tokens, heads, hd)[..., value_dim:].float().abs().max()) == 0.0
+
+
+@pytest.mark.parametrize("hd", [96, 320, 576])
+@pytest.mark.parametrize("runs", [1, 4])
+@pytest.mark.parametrize("span", ["head", "channel", None])
+def test_shared_head_with_a_gate_a_sink_and_chunk_major_rows(hd, runs, span):
+    totals, heads = [150, 300, 7, 64, 65, 1, 129, 200, 30, 90], 18
+    case = PagedCase(totals, [1] * len(totals), 1, hd, torch.bfloat16, DEV, seed=hd, poison=True)
+    gen = torch.Generator().manual_seed(hd)
+    q = (torch.randn(case.n_tokens, heads * hd, generator=gen) / math.sqrt(hd)).to(torch.bfloat16)
+    sink = torch.randn(heads, generator=gen) + 2.0
+    gate = {"head": torch.randn(case.n_tokens, heads + 2, generator=gen), "channel": torch.randn(case.n_tokens, heads * hd, generator=gen), None: None}[span]
+    want = torch.zeros(case.n_tokens, heads, hd, dtype=F64)
+    for s, total in enumerate(totals):
+        k, v = case.k_rows[s].double(), case.v_rows[s].double()
+        for h in range(heads):
+            scores = torch.cat([k @ q[s, h * hd:(h + 1) * hd].double() * 2.0, sink[h:h + 1].double()])
+            want[s, h] = torch.softmax(scores, 0)[:-1] @ v
+    if span == "head":
+        want *= plain.sigmoid(gate.double())[:, :heads, None]
+    want = want.reshape(case.n_tokens, -1) * (plain.sigmoid(gate.double()) if span == "channel" else 1.0)
+    columns = heads * hd
+    chunked = K.Chunked(torch.zeros(case.n_tokens, (columns + 31) // 32 * 32, dtype=torch.bfloat16, device=DEV), case.n_tokens, columns)
+    row_major = torch.zeros(case.n_tokens, columns, dtype=torch.bfloat16, device=DEV)
+    partial = torch.full((case.n_tokens * heads * runs, hd + 2), float("nan"), device=DEV) if runs > 1 else None
+    held = q.to(DEV), sink.to(DEV), gate.to(DEV) if gate is not None else None
+    for out in (chunked, row_major):
+        args = K.attention_args(held[0], out, case.view(), case.tok_seq, case.tok_pos, case.seq_off, case.seq_start, heads, len(totals), 1,
+                                2.0, 0, partial, sink=held[1], gate=held[2], gate_dim=hd if span == "channel" else 0)
+        K.attention(args, torch.bfloat16, True, impl="shared")
+    assert rel_err(row_major, want) < 1.5e-2
+    assert torch.equal(chunked.to_rows(), row_major)
+
+
+@pytest.mark.parametrize("decode", [False, True])
+@pytest.mark.parametrize("window,keep", [(70, 10), (64, 64), (100, 65)])
+def test_one_key_that_stands_out_on_a_shared_head(decode, window, keep):
+    hd, total, heads = 320, 321, 3
+    edge = total - window
+    for place in sorted({0, keep - 1, keep, 63, 64, 127, 128, edge - 1, edge, 255, 256, total - 1}):
+        case = PagedCase([total], [1 if decode else 60], 1, hd, torch.bfloat16, DEV, seed=place)
+        q = torch.zeros(case.n_tokens, heads * hd)
+        q[-1] = case.k_rows[0][place].float().repeat(heads) * 0.5
+        q = q.to(torch.bfloat16)
+        want = reference(case, q, heads, 0.5, window, 0, keep)[-1:]
+        value = case.v_rows[0][place].double().repeat(heads)
+        assert (float((want[0] - value).abs().max()) < 0.2 * float(value.abs().max())) == (place >= edge or place < keep), f"the premise for the key at {place}"
+        got = run(case, q, heads, 0.5, window, 0, keep, "bfloat16", decode, "shared")[-1:]
+        assert rel_err(got, want) < 1.5e-2, f"the key at {place}"
+
+
+def test_what_the_shared_head_refuses():
+    case = PagedCase([8], [8], 2, 64, torch.bfloat16, DEV)
+    one = PagedCase([8], [8], 1, 64, torch.bfloat16, DEV)
+    q, out = torch.zeros(8, 128, device=DEV, dtype=torch.bfloat16), torch.zeros(8, 128, device=DEV, dtype=torch.bfloat16)
+    for c, options in ((case, {}), (one, {"softcap": 1.0}), (one, {"value_dim": 66}), (one, {"value_dim": 80})):
+        args = K.attention_args(q, out, c.view(), c.tok_seq, c.tok_pos, c.seq_off, c.seq_start, 2, 1, 8, 0.1, **options)
+        with pytest.raises(K.KernelError):
+            K.attention(args, torch.bfloat16, False, impl="shared")
