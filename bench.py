@@ -689,12 +689,32 @@ def rirovik_config(width, layers, vocab):
 
 def run_rirovik(args):
     """Rirovik beside the library's closest family, Gavasun (latent attention with a shared turned key part, attention on
-    grouped heads, ungated experts), at equal width, layers, experts and vocabulary."""
+    grouped heads, ungated experts), at equal width, layers, experts and vocabulary; then both with latents of 512 beside
+    64 turned channels (a cached head of 576)."""
+    def seen(attention, position):
+        first = max(position - attention.window + 1 if attention.window else 0, position - position % attention.chunk if attention.chunk else 0, 0)
+        return position + 1 - max(0, first - attention.keep)
+
     def values_and_columns(attention):
-        return 2 * attention.kv.head_dim * attention.kv.kv_heads, attention.q_heads * attention.kv.head_dim
-    heads = lambda width: max(4, width // 128)
-    run_beside_gpt2(args, "rirovik", rirovik_config, None, of_call=values_and_columns,
-                    other=("gavasun", gavasun_config, lambda width: (2 * 128 * (heads(width) // 4), 128 * heads(width))))
+        # cached values a token, and channels its queries meet on average over keys and values, both times the share of the
+        # context that windows and chunks leave
+        size = attention.kv.head_dim
+        values = attention.value_dim if attention.value_dim and size > 128 else size
+        positions = [512 + min(args.steps, 64) // 2 - 1] if attention.max_count == 1 else range(PREFILL_LEN)
+        share = sum(seen(attention, p) for p in positions) / sum(p + 1 for p in positions)
+        return share * (size + values) * attention.kv.kv_heads, share * attention.q_heads * (size + values) / 2
+    run_beside_gpt2(args, "rirovik", rirovik_config, None, of_call=values_and_columns, other=("gavasun", gavasun_config, values_and_columns))
+
+    def wide(config_of):
+        def config(width, layers, vocab):
+            made = config_of(width, layers, vocab)
+            for layer in made["layers"]:
+                if "latent" in layer["type"]:
+                    layer["mixer"] = dict(layer["mixer"], kv_rank=512, rot_dim=64, rot=dict(layer["mixer"]["rot"], dims=64), scale=192 ** -0.5)
+            return made
+        return config
+    run_beside_gpt2(args, "rirovik", wide(rirovik_config), None, of_call=values_and_columns,
+                    other=("gavasun", wide(gavasun_config), values_and_columns), widths=(2048,), note="latents of 512 + 64")
 
 
 def run_loselix(args):
@@ -735,31 +755,34 @@ def run_kodatar(args):
                     lambda width: (2 * 128 * (max(4, width // 128) // 4), 128 * max(4, width // 128)))
 
 
-def run_beside_gpt2(args, family, config_of, attention_sizes, other=None, of_call=None):
+def run_beside_gpt2(args, family, config_of, attention_sizes, other=None, of_call=None, widths=(1024, 2048), note=None):
     """``attention_sizes(width)``: (cached values a token and layer, columns of a token's queries), for
     the attention kernels' bytes and flops; ``of_call``: the same as a function of an attention call's arguments, for a
-    family whose attention layers differ.  ``other``: (family, its configuration, its attention sizes) of the
-    model that runs beside, GPT-2 without."""
+    family whose attention layers differ.  ``other``: (family, its configuration, its attention sizes, or with ``of_call`` a
+    function like that) of the model that runs beside, GPT-2 without.  ``note``: what the line says of its sizes."""
     import torch
 
     import burn_transformers_amd as bt
     dtype = args.dtype or "bf16"
     layers, batch, prompt_len, steps = args.layers or 12, args.batch, 512, min(args.steps, 64)
     vocab = 32000
-    for width in (1024, 2048):
+    for width in widths:
         beside = other[0] if other else "gpt2"
         line = {"workload": f"{family} beside {beside}", "width": width, "layers": layers, "dtype": dtype, "batch": batch,
                 "prompt_len": prompt_len, "decode_steps": steps, "data": "synthetic token ids, random weights"}
+        if note:
+            line["sizes"] = note
         for name in (family, beside):
             if name == family or other:
                 config = (config_of if name == family else other[1])(width, layers, vocab)
                 model = build_salopel(config, dtype)
                 sizes = attention_sizes if name == family else other[2]
-                cached, columns = sizes(width) if sizes else (None, None)
+                counts = of_call if name == family else sizes if of_call and other else None      # (by call)
+                cached, columns = sizes(width) if sizes and not counts else (None, None)
             else:
                 config = dict(XL, n_layer=layers, n_embd=width, n_head=width // 64, n_inner=4 * width, vocab_size=vocab,
                               n_positions=2048)
-                model = build_model(config, dtype)
+                model, counts = build_model(config, dtype), None
             engine = bt.Engine(model, max_tokens=max(batch, 8) * 2048)
             times, done, _ = decode_run(engine, batch, 8, steps, vocab, max(3, args.repetitions // 2), 1, prompt_len=prompt_len)
             decode_seconds = statistics.median(times) / done
@@ -775,18 +798,18 @@ def run_beside_gpt2(args, family, config_of, attention_sizes, other=None, of_cal
                 engine.step(list(zip(slots, prompts)))
                 if name == "gpt2":
                     cached, columns = 2 * width, width
-                element, per_call = ELEMENT_BYTES[dtype], name == family and of_call
-                kv = (lambda a: batch * context * of_call(a)[0] * element) if per_call else batch * context * cached * element
-                flops = (lambda a: 4.0 * batch * context * of_call(a)[1]) if per_call else 4.0 * batch * context * columns
+                element = ELEMENT_BYTES[dtype]
+                kv = (lambda a: batch * context * counts(a)[0] * element) if counts else batch * context * cached * element
+                flops = (lambda a: 4.0 * batch * context * counts(a)[1]) if counts else 4.0 * batch * context * columns
                 result["decode_kernels"] = kernel_classes(engine, [(slot, [5]) for slot in slots], kv, flops, PEAK_FLOPS[dtype])
                 for slot in slots:
                     engine.close(slot)
                 prompts = synthetic_prompts(PREFILL_SEQS, PREFILL_LEN, vocab, seed=8)
                 slots = [engine.open() for _ in prompts]
                 tokens = PREFILL_SEQS * PREFILL_LEN
-                kv = (lambda a: 4 * tokens * of_call(a)[1] * element) if per_call else 4 * tokens * columns * element
+                kv = (lambda a: 4 * tokens * counts(a)[1] * element) if counts else 4 * tokens * columns * element
                 pairs = PREFILL_SEQS * 2.0 * PREFILL_LEN * (PREFILL_LEN + 1)
-                flops = (lambda a: pairs * of_call(a)[1]) if per_call else pairs * columns
+                flops = (lambda a: pairs * counts(a)[1]) if counts else pairs * columns
                 result["prefill_kernels"] = kernel_classes(engine, list(zip(slots, prompts)), kv, flops, PEAK_FLOPS[dtype], replays=10)
                 for slot in slots:
                     engine.close(slot)

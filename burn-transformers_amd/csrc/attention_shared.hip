@@ -3,7 +3,7 @@
 // ordinary decode kernel takes.  Prompts and decode steps.
 //
 // A row is one (token, query head) pair; a sequence's rows lie one behind the other, token by token, and since all of them
-// meet the same cached vectors a work-group takes 16 or 32 of them whatever tokens they belong to.  Its eight waves divide
+// meet the same cached vectors a work-group takes 16, 32 or 64 of them whatever tokens they belong to.  Its eight waves divide
 // every block of 64 keys between them so that each cached byte is read once a work-group, straight into the registers it
 // is multiplied from:
 //   scores   wave w multiplies 16 of the keys (w % 4) by one half of the channels (w / 4); the two halves' sums meet in LDS.
@@ -25,6 +25,7 @@
 #include "calls.h"
 
 #define SHARED_WAVES 8
+#define SHARED_MANY 128       // work-groups of 64 rows from which on they are that large
 #define LOG2_E 1.4426950408889634f
 
 __device__ __forceinline__ bf16x8 load_bf16x8(const bf16_t* p) { return *reinterpret_cast<const bf16x8*>(p); }
@@ -37,10 +38,15 @@ __device__ __forceinline__ void lds_barrier() {
   asm volatile("" ::: "memory");
 }
 
-// HS: steps of 32 channels in half of a head; NV: blocks of 16 value channels a wave owns; NQ: blocks of 16 rows.
+// HS: steps of 32 channels in half of a head; NV: blocks of 16 value channels a wave owns; NQ: blocks of 16 rows.  The time of
+// a block is the time its keys and values take to arrive, so the more rows share them the better: four blocks of rows keep
+// their queries in LDS (QUERIES_IN_LDS), in the order of the operand, where the registers do not hold them.
 template <int HS, int NV, int NQ>
 __global__ void __launch_bounds__(SHARED_WAVES * 64)
 attention_shared_kernel(AttnArgs a, int tiles_max) {
+  constexpr bool QUERIES_IN_LDS = NQ > 2;
+  constexpr int QREG = QUERIES_IN_LDS ? 1 : NQ;
+  extern __shared__ bf16x8 s_queries[];                    // QUERIES_IN_LDS: [half of the channels][step][rows][lane]
   __shared__ floatx4 s_scores[2][NQ][4][64];               // [half of the channels][rows][16 keys][lane]
   __shared__ bf16x8 s_probs[NQ][2][64];                    // [rows][half of the keys][lane]
   __shared__ float s_alpha[NQ][16], s_max[NQ][16], s_sum[NQ][2][16];
@@ -64,16 +70,24 @@ attention_shared_kernel(AttnArgs a, int tiles_max) {
 
   const bf16_t* Q = static_cast<const bf16_t*>(a.q);
   const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
-  bf16x8 q[NQ][HS];
+  bf16x8 q[QREG][HS];
 #pragma unroll
   for (int nq = 0; nq < NQ; ++nq) {
+    if (QUERIES_IN_LDS && nq != kt) continue;              // (a wave brings one block of rows for its half of the channels)
     const int r = row0 + 16 * nq + i16, rr = r < rows ? r : rows - 1;
     const bf16_t* row = Q + (int64_t)(off + rr / heads) * a.ldq + rr % heads * HD;
 #pragma unroll
     for (int s = 0; s < HS; ++s) {
       const int channel = (half * HS + s) * 32 + g * 8;
-      q[nq][s] = channel < HD ? load_bf16x8(row + channel) : zero8;
+      q[QUERIES_IN_LDS ? 0 : nq][s] = channel < HD ? load_bf16x8(row + channel) : zero8;
     }
+  }
+  bf16x8* my_queries = s_queries + half * HS * NQ * 64 + lane;
+  if constexpr (QUERIES_IN_LDS) {
+    static_assert(NQ == 4, "four waves, four blocks of rows");
+#pragma unroll
+    for (int s = 0; s < HS; ++s) my_queries[(s * NQ + kt) * 64] = q[0][s];
+    lds_barrier();
   }
   // what this wave does in the softmax: rows 16 * sq + i16, keys 32 * sh .. + 31 of a block
   const bool weighs = wave < 2 * NQ;
@@ -134,7 +148,10 @@ attention_shared_kernel(AttnArgs a, int tiles_max) {
 #pragma unroll
     for (int s = 0; s < HS; ++s)
 #pragma unroll
-      for (int nq = 0; nq < NQ; ++nq) acc[nq] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k[s], q[nq][s], acc[nq], 0, 0, 0);
+      for (int nq = 0; nq < NQ; ++nq) {
+        const bf16x8 operand = QUERIES_IN_LDS ? my_queries[(s * NQ + nq) * 64] : q[QUERIES_IN_LDS ? 0 : nq][s];
+        acc[nq] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k[s], operand, acc[nq], 0, 0, 0);
+      }
 #pragma unroll
     for (int nq = 0; nq < NQ; ++nq) s_scores[half][nq][kt][lane] = acc[nq];
     plane = next_plane;
@@ -304,7 +321,16 @@ static int launch(hipStream_t stream, const AttnArgs& a) {
   const int64_t tiles = ((int64_t)a.max_count * a.q_heads + 16 * NQ - 1) / (16 * NQ);
   const int splits = a.splits > 1 ? a.splits : 1;
   if (tiles * a.n_seqs > 0x7fffffff) BT_REFUSE("attention_shared: %lld tiles of rows are too many", (long long)(tiles * a.n_seqs));
-  hipLaunchKernelGGL((attention_shared_kernel<HS, NV, NQ>), dim3((unsigned)(tiles * a.n_seqs), splits), dim3(SHARED_WAVES * 64), 0, stream,
+  const size_t lds = NQ > 2 ? (size_t)2 * HS * NQ * 64 * sizeof(bf16x8) : 0;
+  if (lds > 0) {                                           // with what the kernel holds anyway: beyond what it gets without asking
+    static bool raised = false;
+    if (!raised) {
+      hipError_t err = hipFuncSetAttribute((const void*)attention_shared_kernel<HS, NV, NQ>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+      if (err != hipSuccess) BT_REFUSE("attention_shared: cannot get %zu bytes of LDS: %s", lds, hipGetErrorString(err));
+      raised = true;
+    }
+  }
+  hipLaunchKernelGGL((attention_shared_kernel<HS, NV, NQ>), dim3((unsigned)(tiles * a.n_seqs), splits), dim3(SHARED_WAVES * 64), lds, stream,
                      a, (int)tiles);
   return bt_check_launch("attention_shared");
 }
@@ -329,17 +355,20 @@ BT_EXPORT int bt_attention_shared(void* stream, const AttnArgs* args) {
   if (a.out_rows != 0 && a.out_rows < a.n_tokens) BT_REFUSE("attention_shared: a chunk-major output of %d rows for %d tokens", a.out_rows, a.n_tokens);
   if (a.splits > 1 && (!a.partial || a.splits > 64)) BT_REFUSE("attention_shared: %d runs of keys (at most 64) need a place for their results", a.splits);
   hipStream_t s = (hipStream_t)stream;
-  const bool few = (int64_t)a.max_count * a.q_heads <= 16;
+  // 64 rows a work-group where there are enough of them for every compute unit, fewer where there are not
+  const int64_t most = (int64_t)a.max_count * a.q_heads, all = (int64_t)a.n_tokens * a.q_heads * (a.splits > 1 ? a.splits : 1);
+  const int size = most <= 16 ? 1 : most < 64 || all < 64 * SHARED_MANY ? 2 : 4;
   const int v_blocks = (vd + 127) / 128;
   int rc;
-#define SHARED_FORM(HS, NV) (few ? launch<HS, NV, 1>(s, a) : launch<HS, NV, 2>(s, a))
+#define SHARED_FORM(HS, NV) (size == 1 ? launch<HS, NV, 1>(s, a) : size == 2 ? launch<HS, NV, 2>(s, a) : launch<HS, NV, 4>(s, a))
   if (hd <= 128) rc = SHARED_FORM(2, 1);
   else if (hd <= 256) rc = SHARED_FORM(4, 2);
   else if (hd <= 384) rc = SHARED_FORM(6, 3);
   else if (hd <= 512) rc = SHARED_FORM(8, 4);
   else if (hd <= 576 && v_blocks <= 4) rc = SHARED_FORM(9, 4);
-  else if (hd <= 640) rc = launch<10, 5, 1>(s, a);         // (two blocks of rows would not fit the registers)
-  else rc = launch<12, 6, 1>(s, a);
+  // (the widest: two blocks of rows would not fit the registers)
+  else if (hd <= 640) rc = size < 4 ? launch<10, 5, 1>(s, a) : launch<10, 5, 4>(s, a);
+  else rc = size < 4 ? launch<12, 6, 1>(s, a) : launch<12, 6, 4>(s, a);
 #undef SHARED_FORM
   if (rc || a.splits <= 1) return rc;
   const int64_t pairs = (int64_t)a.n_tokens * a.q_heads;

@@ -261,6 +261,86 @@ __global__ void __launch_bounds__(256) head_project_small_kernel(HeadProjectCall
     for (int extra = c.heads * c.vdim + threadIdx.x; extra < c.out_cols; extra += 256) out[extra] = from_float<T>(0.f);
 }
 
+// The same on the matrix units, for bfloat16 whose rows can be read 16 bytes at a time.  A wave takes 16 * MT tokens and
+// 16 * NT outputs of one head (v_mfma_f32_16x16x32_bf16: weights as "A" rows, tokens as "B" columns, so a lane ends with four
+// consecutive outputs of one token) and walks the rank in batches of U steps of 32 whose loads fly together; a work-group is
+// WM x WN waves.
+template <int MT, int NT, int U, int WM, int WN>
+__global__ void __launch_bounds__(WM * WN * 64) head_project_mfma_kernel(HeadProjectCall c) {
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int i16 = lane & 15, g = lane >> 4;
+  const int head = blockIdx.y;
+  const int t0 = (blockIdx.x * WM + wave / WN) * 16 * MT, v0 = (blockIdx.z * WN + wave % WN) * 16 * NT;
+  bf16_t* out = static_cast<bf16_t*>(c.out);
+  if (t0 < c.tokens && v0 < c.vdim) {
+    const bf16_t* ctx = static_cast<const bf16_t*>(c.ctx);
+    const bf16_t* W = static_cast<const bf16_t*>(c.W);
+    const bf16_t* rows[MT];
+    const bf16_t* weights[NT];
+#pragma unroll
+    for (int mt = 0; mt < MT; ++mt) {
+      const int t = t0 + 16 * mt + i16;
+      rows[mt] = ctx + (int64_t)(t < c.tokens ? t : c.tokens - 1) * c.ld_ctx + (int64_t)head * c.head_pitch;
+    }
+#pragma unroll
+    for (int nt = 0; nt < NT; ++nt) {
+      const int v = v0 + 16 * nt + i16;
+      weights[nt] = W + ((int64_t)head * c.vdim + (v < c.vdim ? v : c.vdim - 1)) * c.rank;
+    }
+    floatx4 acc[MT][NT];
+#pragma unroll
+    for (int mt = 0; mt < MT; ++mt)
+#pragma unroll
+      for (int nt = 0; nt < NT; ++nt) acc[mt][nt] = floatx4{0.f, 0.f, 0.f, 0.f};
+    const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
+    for (int r0 = 0; r0 < c.rank; r0 += 32 * U) {
+      bf16x8 x[U][MT], w[U][NT];
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int r = r0 + 32 * u + 8 * g, rr = r < c.rank ? r : 0;
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt) w[u][nt] = *reinterpret_cast<const bf16x8*>(weights[nt] + rr);
+#pragma unroll
+        for (int mt = 0; mt < MT; ++mt) x[u][mt] = *reinterpret_cast<const bf16x8*>(rows[mt] + rr);
+      }
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const bool there = r0 + 32 * u + 8 * g < c.rank;
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt) {
+          const bf16x8 weight = there ? w[u][nt] : zero8;
+#pragma unroll
+          for (int mt = 0; mt < MT; ++mt)
+            acc[mt][nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(weight, there ? x[u][mt] : zero8, acc[mt][nt], 0, 0, 0);
+        }
+      }
+    }
+#pragma unroll
+    for (int mt = 0; mt < MT; ++mt) {
+      const int t = t0 + 16 * mt + i16;
+      if (t >= c.tokens) continue;
+      const float* gate = c.gate ? c.gate + (int64_t)t * c.ld_gate : nullptr;
+      const float whole = gate && c.gate_span == 1 ? 1.0f / (1.0f + expf(-gate[head])) : 1.0f;
+#pragma unroll
+      for (int nt = 0; nt < NT; ++nt)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int v = v0 + 16 * nt + 4 * g + i, col = head * c.vdim + v;
+          if (v >= c.vdim) continue;
+          const float factor = gate && c.gate_span == 0 ? 1.0f / (1.0f + expf(-gate[col])) : whole;
+          out[(int64_t)t * c.ld_out + col] = (bf16_t)(acc[mt][nt][i] * factor);
+        }
+    }
+  }
+  // the columns behind the last head's, which the next product reads as zeros
+  const int extra = c.out_cols - c.heads * c.vdim;
+  if (extra > 0 && head == c.heads - 1 && blockIdx.z == gridDim.z - 1)
+    for (int e = threadIdx.x; e < WM * 16 * MT * extra; e += WM * WN * 64) {
+      const int t = blockIdx.x * WM * 16 * MT + e / extra;
+      if (t < c.tokens) out[(int64_t)t * c.ld_out + c.heads * c.vdim + e % extra] = (bf16_t)0.f;
+    }
+}
+
 BT_EXPORT int bt_head_project_call(void* stream, const HeadProjectCall* c) {
   if (c->tokens <= 0) return BT_OK;
   if (c->heads <= 0 || c->vdim <= 0 || c->rank <= 0)
@@ -271,6 +351,16 @@ BT_EXPORT int bt_head_project_call(void* stream, const HeadProjectCall* c) {
     BT_REFUSE("head_project: the rows do not hold %d heads", c->heads);
   if (c->gate_span != 0 && c->gate_span != 1) BT_REFUSE("head_project: gate_span %d must be 0 or 1", c->gate_span);
   if (!c->ctx || !c->W || !c->out) BT_REFUSE("head_project: missing operand");
+  if (c->dtype == 1 && c->rank % 8 == 0 && c->head_pitch % 8 == 0 && c->ld_ctx % 8 == 0 && (((uintptr_t)c->ctx | (uintptr_t)c->W) & 15) == 0) {
+    if (c->tokens <= 64) {              // a wave a work-group: as many compute units as there are blocks of outputs
+      dim3 grid((c->tokens + 15) / 16, c->heads, (c->vdim + 15) / 16);
+      hipLaunchKernelGGL((head_project_mfma_kernel<1, 1, 8, 1, 1>), grid, dim3(64), 0, (hipStream_t)stream, *c);
+    } else {
+      dim3 grid((c->tokens + 63) / 64, c->heads, (c->vdim + 127) / 128);
+      hipLaunchKernelGGL((head_project_mfma_kernel<2, 4, 4, 2, 2>), grid, dim3(256), 0, (hipStream_t)stream, *c);
+    }
+    return bt_check_launch("head_project");
+  }
   if (c->tokens <= HP_SMALL_TOKENS) {
     dim3 small(c->tokens, c->heads, (c->vdim + 63) / 64);
     if (c->dtype == 0)

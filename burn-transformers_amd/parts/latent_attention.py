@@ -173,11 +173,15 @@ class LatentAttention(Mixer):
         pair_bytes = keys * self.head_dim * 2 * (2 if step.dtype_is_bf16 else 4)
         if pair_bytes <= self.SPLIT_BYTES:
             return 1
-        tiles = 1
-        if self.shared_decode:           # (rows of 32 heads a work-group, 16 where there are no more or heads are widest)
-            tiles = -(-self.heads // (16 if self.heads <= 16 or self.head_dim > 576 else 32))
-        runs = min(compute_units(device) // (step.n_seqs * tiles), pair_bytes // self.RUN_BYTES, 64)
-        return max(1, min(runs, -(-keys // 64) if self.shared_decode else runs))
+        if not self.shared_decode:
+            return max(1, min(compute_units(device) // step.n_seqs, pair_bytes // self.RUN_BYTES, 64))
+        # The kernel for one shared head: a run of four blocks of 64 keys, or shorter ones up to eight runs.  Measured at heads
+        # of 512 + 64, us a call with 1 / 4 / 8 / 16 / 32 runs (join included): 16 heads, 8 sequences of 544 keys 37 / 24 / 20,
+        # of 4,096 230 / 70 / 43 / 34 / 38, 32 sequences of 2,048 119 / 44 / 35 / 44 / 61, one of 8,192 448 / 124 / 67 / 44 /
+        # 40; 128 heads, 8 of 4,096 238 / 75 / 54 / 45 / 62, 32 of 2,048 125 / 59 / 71.
+        rows = 64 if self.heads >= 64 else 32 if self.heads > 16 and self.head_dim <= 576 else 16      # of a work-group
+        blocks = -(-keys // 64)
+        return max(1, min(compute_units(device) // (step.n_seqs * -(-self.heads // rows)), max(blocks // 4, min(blocks, 8)), 64))
 
     SPLIT_BYTES = 128 << 10
     RUN_BYTES = 64 << 10
