@@ -58,12 +58,12 @@ struct TileOperands {
   bf16x4 v[ND][2];
 };
 
-// Issues the loads of one tile (kb a multiple of 32); nothing waits on them here, so the caller
-// can have the next tile's loads in flight while it works on the current one.
+// Issues the loads of one tile, which starts at position `kin` (0 or 32) of its block; nothing waits on them here, so the caller
+// can have the next tile's loads in flight while it works on the current one.  (The callers walk whole blocks, so that `kin` is
+// seen to be the same from one of their turns to the next and the lanes' distances are worked out once.)
 __device__ __forceinline__ void load_tile(TileOperands& t, const bf16_t* __restrict__ kplane,
-                                          const bf16_t* __restrict__ vplane, int kb) {
+                                          const bf16_t* __restrict__ vplane, int kin) {
   const int lane = threadIdx.x & 63, i16 = lane & 15, g = lane >> 4;
-  const int kin = kb & (BT_KV_BLOCK - 1);
   const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
 #pragma unroll
   for (int h = 0; h < 2; ++h)
@@ -206,15 +206,15 @@ __device__ __forceinline__ float raise_maximum(float& m, float top, float& alpha
 
 // One tile of 32 keys starting at position kb against NQ tiles of 16 queries.
 //   qpos[nq]: position of the query in column lane % 16 of tile nq, -1 if there is none.
-//   qlo[nq]: the first position that query sees (its window's or its chunk's first key, else 0); it also sees the
-//   positions below `keep`.
+//   qlo[nq]: the first position that query sees (its window's or its chunk's first key, else 0); with KEEPS it
+//   also sees the positions below `keep`.
 //   valid_end: positions >= valid_end hold no token (their values are replaced by zero).
 //   sc: what makes exponents of the dot products (form 0: one positive factor); m[] is kept in those units
 //   (powers of two).
 //   MASKED = false is for tiles every query of the wave sees whole (all keys at or before the
 //   first query's position, no window): nothing is compared or replaced there.  Columns without
 //   a query then hold numbers nobody reads.
-template <int NQ, bool MASKED>
+template <int NQ, bool MASKED, bool KEEPS>
 __device__ __forceinline__ void attend_tile(const TileOperands& tile, int kb, int valid_end,
                                             const int (&qpos)[NQ], const int (&qlo)[NQ], int keep, const Scoring& sc,
                                             const bf16x8 (&q)[NQ][NKS], floatx4 (&o)[NQ][ND],
@@ -245,11 +245,22 @@ __device__ __forceinline__ void attend_tile(const TileOperands& tile, int kb, in
 #pragma unroll
   for (int nq = 0; nq < NQ; ++nq) {
     if (MASKED) {
-      const SeenKeys seen = bt_seen_keys(qpos[nq], qlo[nq], keep);
+      if (KEEPS && kb < keep) {                     // (the same for the whole wave)
+        const SeenKeys seen = bt_seen_keys(qpos[nq], qlo[nq], keep);
 #pragma unroll
-      for (int t = 0; t < 2; ++t)
+        for (int t = 0; t < 2; ++t)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) s[nq][t][r] = seen(kb + 16 * t + 4 * g + r) ? s[nq][t][r] : -INFINITY;
+          for (int r = 0; r < 4; ++r) s[nq][t][r] = seen(kb + 16 * t + 4 * g + r) ? s[nq][t][r] : -INFINITY;
+      } else {
+        const int qp = qpos[nq], ql = qlo[nq];
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int kp = kb + 16 * t + 4 * g + r;
+            s[nq][t][r] = kp <= qp && kp >= ql ? s[nq][t][r] : -INFINITY;
+          }
+      }
     }
     if constexpr (FORM == 2) continue;          // weights that no other key has a part in
     const float m_use = m[nq] == -INFINITY ? 0.f : m[nq];
@@ -398,7 +409,7 @@ attention_prefill_kernel(AttnArgs a) {
   const int last = q0 + PREFILL_QUERIES_PER_WAVE < count ? q0 + PREFILL_QUERIES_PER_WAVE : count;
   const int hi = start + last;  // one past the position of this wave's last query
   // (the wave's first query sees furthest back)
-  const KeyWalk walk = bt_key_walk(bt_first_seen(start + q0, a.window, a.chunk) & ~31, a.keep, 32);
+  const KeyWalk walk = bt_key_walk(bt_first_seen(start + q0, a.window, a.chunk) & ~(BT_KV_BLOCK - 1), a.keep, BT_KV_BLOCK);
   const int places = walk.places(hi);
   const int valid_end = start + count;
   const bf16_t* keys = static_cast<const bf16_t*>(a.kv.keys);
@@ -411,26 +422,25 @@ attention_prefill_kernel(AttnArgs a) {
   // A fetch beyond the last tile reads the first one again instead of being skipped: with the same
   // number of loads in flight on every path, the wait before a tile is for that tile only.
   TileOperands t0, t1;
-  auto fetch = [&](TileOperands& into, int place) {
-    const int kf = walk.at(place < places ? place : 0);
-    int64_t plane = tile_plane(a, seq, kv_head, kf);
-    load_tile(into, keys + plane, values + plane, kf);
+  auto fetch = [&](TileOperands& into, int place, int kin) {           // (kin: place & 63)
+    int64_t plane = tile_plane(a, seq, kv_head, walk.at(place < places ? place : kin));
+    load_tile(into, keys + plane, values + plane, kin);
   };
   auto attend = [&](const TileOperands& tile, int place) {
     const int kb = walk.at(place);
     if (kb + 32 <= whole_until)
-      attend_tile<PREFILL_NQ, false>(tile, kb, valid_end, qpos, qlo, a.keep, sc, q, o, m, l);
+      attend_tile<PREFILL_NQ, false, false>(tile, kb, valid_end, qpos, qlo, a.keep, sc, q, o, m, l);
     else
-      attend_tile<PREFILL_NQ, true>(tile, kb, valid_end, qpos, qlo, a.keep, sc, q, o, m, l);
+      attend_tile<PREFILL_NQ, true, true>(tile, kb, valid_end, qpos, qlo, a.keep, sc, q, o, m, l);
   };
   if (places <= 0) return;   // (cannot happen: a wave with a query sees at least that query's key)
-  fetch(t0, 0);
-  fetch(t1, 32);
+  fetch(t0, 0, 0);
+  fetch(t1, 32, 32);
   for (int place = 0; place < places; place += 64) {
     attend(t0, place);
-    fetch(t0, place + 64);
+    fetch(t0, place + 64, 0);
     if (place + 32 < places) attend(t1, place + 32);
-    fetch(t1, place + 96);
+    fetch(t1, place + 96, 32);
   }
 #pragma unroll
   for (int nq = 0; nq < PREFILL_NQ; ++nq) {
@@ -504,14 +514,21 @@ __device__ __forceinline__ void attend_block(const Operands& blk, int kb, int va
 #pragma unroll
     for (int nq = 0; nq < NQ; ++nq) {
       const int qp = qpos[nq];
-      const SeenKeys seen = bt_seen_keys(qp, qlo[nq], keep);
+      if (BOUNDED && kb < keep) {                   // (the same for the whole wave)
+        const SeenKeys seen = bt_seen_keys(qp, qlo[nq], keep);
 #pragma unroll
-      for (int t = 0; t < 4; ++t)
+        for (int t = 0; t < 4; ++t)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int kp = kb + 16 * t + 4 * g + r;
-          s[nq][t][r] = (BOUNDED ? seen(kp) : kp <= qp) ? s[nq][t][r] : -INFINITY;
-        }
+          for (int r = 0; r < 4; ++r) s[nq][t][r] = seen(kb + 16 * t + 4 * g + r) ? s[nq][t][r] : -INFINITY;
+      } else {
+#pragma unroll
+        for (int t = 0; t < 4; ++t)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int kp = kb + 16 * t + 4 * g + r;
+            s[nq][t][r] = kp <= qp && (!BOUNDED || kp >= qlo[nq]) ? s[nq][t][r] : -INFINITY;
+          }
+      }
     }
   }
   float own[NQ];
@@ -1088,6 +1105,9 @@ attention_prefill_wide_kernel(AttnArgs a) {
 // reduction overlaps the other's loads (57 -> 42 us).
 #define DECODE_WAVES 8
 
+// KEEPS: some first positions stay visible beside a window or a chunk (a form of its own: the walk over two stretches of keys
+// and its test cost the other 0.3 us of 6.5).
+template <bool KEEPS>
 __global__ void __launch_bounds__(DECODE_WAVES * 64)
 attention_decode_kernel(AttnArgs a) {
   // per wave: maximum and sum of each query column, and its output row; `group` columns are real
@@ -1134,14 +1154,15 @@ attention_decode_kernel(AttnArgs a) {
 #pragma unroll
   for (int dt = 0; dt < ND; ++dt) o[0][dt] = floatx4{0.f, 0.f, 0.f, 0.f};
 
-  const KeyWalk walk = bt_key_walk(qlo[0] & ~31, a.keep, 32);
+  const KeyWalk walk = KEEPS ? bt_key_walk(qlo[0] & ~(BT_KV_BLOCK - 1), a.keep, BT_KV_BLOCK) : KeyWalk{0, qlo[0] & ~(BT_KV_BLOCK - 1)};
   const bf16_t* keys = static_cast<const bf16_t*>(a.kv.keys);
   const bf16_t* values = static_cast<const bf16_t*>(a.kv.values);
-  // the tiles of 32 keys that are kept or lie from `qlo` through the query's own position, cut into `splits` runs
+  // the tiles of 32 keys of the blocks that are kept or reach from `qlo` through the query's own position, cut into `splits` runs
   const int tiles = walk.places(pos) / 32 + 1, per_split = (tiles + splits - 1) / splits;
   const int tile_begin = split * per_split;
   const int tile_end = tile_begin + per_split < tiles ? tile_begin + per_split : tiles;
   const int first = 32 * (tile_begin + wave), end = 32 * tile_end;      // (places of the walk)
+  const int kin = first & (BT_KV_BLOCK - 1);                            // (the same every turn: a stride is four blocks)
   // plane of the tile at kb: from the blocks fetched early where they apply, else from the table
   auto plane_of = [&](int kb, int j) {
     int block = (early && j < 2) ? (j == 0 ? early_block0 : early_block1) : block_row[kb / BT_KV_BLOCK];
@@ -1150,13 +1171,12 @@ attention_decode_kernel(AttnArgs a) {
   const Scoring sc = scoring_of(a, head);
   auto fetch = [&](TileOperands& into, int place, int j) {
     if (place < end) {
-      const int kb = walk.at(place);
-      int64_t plane = plane_of(kb, j);
-      load_tile(into, keys + plane, values + plane, kb);
+      int64_t plane = plane_of(walk.at(place), j);
+      load_tile(into, keys + plane, values + plane, kin);
     }
   };
   auto attend = [&](const TileOperands& tile, int kb) {   // one form: this kernel waits for memory, not for the ALU
-    attend_tile<1, true>(tile, kb, pos + 1, qpos, qlo, a.keep, sc, q, o, m, l);
+    attend_tile<1, true, KEEPS>(tile, kb, pos + 1, qpos, qlo, a.keep, sc, q, o, m, l);
   };
   TileOperands current, next;
   fetch(next, first, 0);
@@ -1384,7 +1404,10 @@ BT_EXPORT int bt_attention_decode_bf16(void* stream, const AttnArgs* args) {
   dim3 grid(args->kv.kv_heads, args->n_seqs, splits);
   int group = args->q_heads / args->kv.kv_heads;
   size_t lds = (size_t)DECODE_WAVES * group * (HD + 2) * sizeof(float);
-  hipLaunchKernelGGL(attention_decode_kernel, grid, dim3(DECODE_WAVES * 64), lds, (hipStream_t)stream, *args);
+  if (args->keep > 0 && (args->window > 0 || args->chunk > 0))
+    hipLaunchKernelGGL(attention_decode_kernel<true>, grid, dim3(DECODE_WAVES * 64), lds, (hipStream_t)stream, *args);
+  else
+    hipLaunchKernelGGL(attention_decode_kernel<false>, grid, dim3(DECODE_WAVES * 64), lds, (hipStream_t)stream, *args);
   if (splits > 1) {
     rc = bt_check_launch("attention_decode_bf16");
     if (rc) return rc;

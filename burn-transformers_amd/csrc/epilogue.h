@@ -14,7 +14,7 @@ enum EpilogueMode {
   EPI_RESIDUAL = 4,  // out[m][n] += acc + bias                  (float: the residual stream itself)
   EPI_F32_ACT = 5,   // columns [0,n_q) -> out as in EPI_F32, those behind -> act(acc + bias) in out2 (element type T), columns
                      //   from 0: two products of the same rows as one (the skinny kernel only)
-  EPI_TURN = 6,      // out[m][n] = acc, of every turn_pitch columns the turn_dim from turn_at on rotated in neighbouring pairs
+  EPI_TURN = 6,      // out[m][n] = acc, of every turn.pitch columns the turn.dim from turn.at on rotated in neighbouring pairs
                      //   by the row's position (element type T; the skinny kernel only)
 };
 // What the skinny kernel is built for: the common modes, or one of the two that are forms of the kernel of their own.
@@ -24,6 +24,14 @@ enum Activation {
   ACT_GELU_TANH = 0,
   ACT_GELU_ERF = 1,
   ACT_SQUARED_RELU = 2,
+};
+
+// EPI_TURN: columns at + 2 i and at + 2 i + 1 of a head of `pitch` columns (a multiple of four; at and dim even) turn by the
+// angle tok_pos[m] * inv_freq[i], sine and cosine times `amplitude`.
+struct TurnedColumns {
+  const float* inv_freq;
+  int pitch, at, dim;
+  float amplitude;
 };
 
 // Mirrored field by field by a ctypes.Structure on the Python side.
@@ -38,15 +46,13 @@ struct Epilogue {
   int n_kv;
   const int* tok_seq;    // [M] index of the token's sequence in the step
   const int* tok_pos;    // [M] position of the token in its sequence
-  KvView kv;
+  union {                // (together: every kernel's arguments are as short as they were without the second)
+    KvView kv;           // EPI_QKV
+    TurnedColumns turn;  // EPI_TURN
+  };
   int out_rows;          // EPI_STORE, EPI_ACT (EPI_F32_ACT: `out2`): 0, or `out` is chunk-major with that many rows (activation_offset)
   void* out2;            // EPI_F32_ACT only
   int64_t ldo2;
-  // EPI_TURN: columns turn_at + 2 i and turn_at + 2 i + 1 of a head of turn_pitch (a multiple of four; turn_at and turn_dim
-  // even) turn by the angle tok_pos[m] * inv_freq[i], sine and cosine times `amplitude`
-  int turn_pitch, turn_at, turn_dim;
-  float amplitude;
-  const float* inv_freq;
 };
 
 // 32-bit activations.  The float32 path (T = float) uses the library's tanhf / erff; the
@@ -97,8 +103,7 @@ __device__ __forceinline__ void store4<bf16_t>(bf16_t* dst, const float* v, int 
 // value of the residual stream in EPI_RESIDUAL) and, for the key/value scatter, where the row's
 // token lives in the paged cache.
 struct EpiloguePrefetch {
-  float freq[2];     // EPI_TURN: the frequencies of the two pairs (0: not turned)
-  float add[4];
+  float add[4];      // EPI_TURN: the amplitudes of the two pairs, then their frequencies (0: not turned)
   int64_t kv_base;   // start of the (block, head) plane of the token; valid for key/value columns
   int pos;
 };
@@ -146,13 +151,13 @@ __device__ __forceinline__ EpiloguePrefetch epilogue_prefetch(const Epilogue& e,
 __device__ __forceinline__ EpiloguePrefetch epilogue_prefetch_turn(const Epilogue& e, int M, int m, int n0) {
   EpiloguePrefetch p = {};
   p.pos = e.tok_pos[m < M ? m : M - 1];
-  const int j = n0 % e.turn_pitch - e.turn_at;       // (even: the pairs of four columns are 0, 1 and 2, 3)
+  const int j = n0 % e.turn.pitch - e.turn.at;       // (even: the pairs of four columns are 0, 1 and 2, 3)
 #pragma unroll
   for (int i = 0; i < 2; ++i) {
-    const bool turned = j + 2 * i >= 0 && j + 2 * i < e.turn_dim;
-    const float f = e.inv_freq[turned ? (j + 2 * i) >> 1 : 0];
-    p.freq[i] = turned ? f : 0.f;
-    p.add[i] = turned ? e.amplitude : 1.f;
+    const bool turned = j + 2 * i >= 0 && j + 2 * i < e.turn.dim;
+    const float f = e.turn.inv_freq[turned ? (j + 2 * i) >> 1 : 0];
+    p.add[i] = turned ? e.turn.amplitude : 1.f;
+    p.add[2 + i] = turned ? f : 0.f;
   }
   return p;
 }
@@ -170,7 +175,7 @@ __device__ __forceinline__ void epilogue4_prefetched(const Epilogue& e, int N, i
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
       float sn = 0.f, cs = 1.f;
-      if (p.freq[i] != 0.f) sincosf((float)p.pos * p.freq[i], &sn, &cs);
+      if (p.add[2 + i] != 0.f) sincosf((float)p.pos * p.add[2 + i], &sn, &cs);
       v[2 * i] = p.add[i] * (acc[2 * i] * cs - acc[2 * i + 1] * sn);
       v[2 * i + 1] = p.add[i] * (acc[2 * i + 1] * cs + acc[2 * i] * sn);
     }

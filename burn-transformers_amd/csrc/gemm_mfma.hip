@@ -847,10 +847,10 @@ static int check_operands(const char* who, int elems, const void* A, int64_t lda
   if (e.mode < 0 || e.mode > 6 || e.out == nullptr) BT_REFUSE("%s: bad epilogue", who);
   if (e.mode == EPI_F32_ACT && (!e.out2 || e.n_q <= 0 || e.n_q >= N || e.n_q % 4 != 0))
     BT_REFUSE("%s: %d of %d columns in 32-bit, the others activated: a multiple of four, and a place for each", who, e.n_q, N);
-  if (e.mode == EPI_TURN && (e.turn_pitch <= 0 || e.turn_pitch % 4 != 0 || N % e.turn_pitch != 0 || e.turn_at < 0 || e.turn_at % 2 != 0 ||
-                             e.turn_dim <= 0 || e.turn_dim % 2 != 0 || e.turn_at + e.turn_dim > e.turn_pitch || !e.tok_pos || !e.inv_freq || e.bias))
+  if (e.mode == EPI_TURN && (e.turn.pitch <= 0 || e.turn.pitch % 4 != 0 || N % e.turn.pitch != 0 || e.turn.at < 0 || e.turn.at % 2 != 0 ||
+                             e.turn.dim <= 0 || e.turn.dim % 2 != 0 || e.turn.at + e.turn.dim > e.turn.pitch || !e.tok_pos || !e.turn.inv_freq || e.bias))
     BT_REFUSE("%s: heads of %d columns (a multiple of four) in %d, turned in neighbouring pairs from %d on (%d columns, both even), without a bias",
-              who, e.turn_pitch, N, e.turn_at, e.turn_dim);
+              who, e.turn.pitch, N, e.turn.at, e.turn.dim);
   if (splits < 1 || (splits > 1 && e.mode != EPI_F32))
     BT_REFUSE("%s: K can be split %d ways only into 32-bit partial sums", who, splits);
   if (e.out_rows != 0 && ((e.mode != EPI_STORE && e.mode != EPI_ACT && e.mode != EPI_F32_ACT) || e.out_rows < M))

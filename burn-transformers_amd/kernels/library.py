@@ -37,12 +37,20 @@ class KvView(ctypes.Structure):
                 ("block_stride", _c_i64), ("head_stride", _c_i64)]
 
 
+class TurnedColumns(ctypes.Structure):
+    _fields_ = [("inv_freq", _c_ptr), ("pitch", _c_int), ("at", _c_int), ("dim", _c_int), ("amplitude", _c_float)]
+
+
+class _ModeArguments(ctypes.Union):
+    _fields_ = [("kv", KvView), ("turn", TurnedColumns)]
+
+
 class Epilogue(ctypes.Structure):
+    _anonymous_ = ("of_mode",)
     _fields_ = [("mode", _c_int), ("act", _c_int), ("bias", _c_ptr), ("out", _c_ptr),
                 ("ldo", _c_i64), ("split_stride", _c_i64), ("n_q", _c_int), ("n_kv", _c_int),
-                ("tok_seq", _c_ptr), ("tok_pos", _c_ptr), ("kv", KvView), ("out_rows", _c_int), ("out2", _c_ptr),
-                ("ldo2", _c_i64), ("turn_pitch", _c_int), ("turn_at", _c_int), ("turn_dim", _c_int), ("amplitude", _c_float),
-                ("inv_freq", _c_ptr)]
+                ("tok_seq", _c_ptr), ("tok_pos", _c_ptr), ("of_mode", _ModeArguments), ("out_rows", _c_int), ("out2", _c_ptr),
+                ("ldo2", _c_i64)]
 
 
 class AttnArgs(ctypes.Structure):
@@ -696,8 +704,8 @@ def epilogue_turn(out, pitch, turn_at, turn_dim, inv_freq, tok_pos, amplitude=1.
     """``out`` [M, N] in the products' type; of every head of ``pitch`` columns (a multiple of four) the ``turn_dim`` from
     ``turn_at`` on (both even) are turned in neighbouring pairs by the row's position, as ``latent_query`` does with
     ``neighbours``: a product of up to 64 rows (the skinny kernel)."""
-    return Epilogue(mode=EPI_TURN, out=out.data_ptr(), ldo=out.stride(0), tok_pos=tok_pos.data_ptr(), turn_pitch=pitch,
-                    turn_at=turn_at, turn_dim=turn_dim, amplitude=amplitude, inv_freq=inv_freq.data_ptr())
+    return Epilogue(mode=EPI_TURN, out=out.data_ptr(), ldo=out.stride(0), tok_pos=tok_pos.data_ptr(),
+                    turn=TurnedColumns(inv_freq=inv_freq.data_ptr(), pitch=pitch, at=turn_at, dim=turn_dim, amplitude=amplitude))
 
 
 def epilogue_residual(x, bias=None):
